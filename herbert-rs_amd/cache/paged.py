@@ -5,7 +5,8 @@ the same need share a group. A group of keys and values owns one pool
 [entries, 2, pages, kv_heads, PAGE_TOKENS, head_dim], a page list of its own
 and a page table [slots, pages per slot]; the page index is shared by the
 group's entries, so one table serves them all. A group with a window gives
-back the pages that no later query can see. A group of fixed-size state owns
+back the pages that no later query can see (and holds on to those of the first
+positions, where the window keeps some). A group of fixed-size state owns
 [entries, slots, *shape] and is cleared for a slot when the slot is taken.
 
 Beyond the slots and pages that sequences can hold there is one more of each:
@@ -56,7 +57,9 @@ class KVGroup:
         self.table = torch.zeros((n_slots + 1, self.pages_per_slot), dtype=torch.int32, device=device)
         self.table[n_slots] = n_pages
         # a slot holds the logical pages [first_page, held_end): it fills from the front as it grows,
-        # a window gives pages back at the front, a roll-back at the end
+        # a window gives pages back at the front, a roll-back at the end. Where the window keeps the first
+        # positions, it also holds those of the first `kept` pages that lie before first_page
+        self.kept = pages_for(need.keep_first) if need.window else 0
         self.first_page = np.zeros(n_slots, dtype=np.int64)
         self.held_end = [0] * n_slots
 
@@ -90,7 +93,8 @@ class KVGroup:
             self.table.device)
 
     def release_unseen(self, slot, length):
-        """With a window: give back pages wholly before the oldest key a later query sees."""
+        """With a window: give back pages wholly before the oldest key a later query sees (but the first pages,
+        where the window keeps the first positions)."""
         if not self.need.window:
             return
         # a query at position >= length sees keys >= length + 1 - window
@@ -98,7 +102,7 @@ class KVGroup:
         row = self.table_host[slot]
         p = int(self.first_page[slot])
         while (p + 1) * PAGE_TOKENS <= oldest:
-            if row[p] >= 0:
+            if row[p] >= 0 and p >= self.kept:
                 self.pages.give_back(int(row[p]))
                 row[p] = -1
             p += 1
@@ -333,6 +337,6 @@ class Cache:
                     raise CacheError(f"free slot {slot} still holds pages")
                 has = np.nonzero(g.table_host[slot] >= 0)[0].tolist()
                 first, end = int(g.first_page[slot]), g.held_end[slot]
-                if has != list(range(first, end)):
+                if has != list(range(min(g.kept, first, end))) + list(range(first, end)):
                     raise CacheError(f"slot {slot} holds the pages {has}, not the stretch [{first}, {end}) "
-                                     "it keeps count of")
+                                     f"it keeps count of beside the first {g.kept}")

@@ -32,6 +32,9 @@ __device__ __forceinline__ void rotate_pair(float a, float b, float angle, float
 // unchanged) -> the row's r. q [T, H, qd + rot] float32: every head's last `rot` rotated the same way
 // into q_full[t, h, rank ...] (q_full [T, H, rank + rot] float32; its first `rank` are written by the
 // product with W_uk^T). One block a token.
+// Queries that come from a latent of their own are not there yet when the cache's row is written: the kernel then
+// runs twice, first with H = 0 and down's neighbour columns q_down [T, q_rank] (rows down_ld apart), which are
+// RMS-normed with q_norm_w into c_q [T, q_rank] (the product that makes the queries reads it), then for the queries alone.
 template <class TC>
 __global__ void latent_write_kernel(const float* __restrict__ down, int down_ld, const float* __restrict__ norm_w,
                                     const float* __restrict__ q, int q_ld, float* __restrict__ q_full,
@@ -39,7 +42,8 @@ __global__ void latent_write_kernel(const float* __restrict__ down, int down_ld,
                                     const int* __restrict__ seq_of, const int* __restrict__ slots,
                                     const int* __restrict__ page_table, int max_pages, int page_size,
                                     TC* __restrict__ pages, int H, int qd, int rank, int rot, int rot_dims,
-                                    float eps, int write_cache) {
+                                    float eps, int write_cache, const float* __restrict__ q_down, int q_rank,
+                                    const float* __restrict__ q_norm_w, TC* __restrict__ c_q) {
     __shared__ float red[16];
     const int t = blockIdx.x;
     const int pos = positions[t];
@@ -66,6 +70,15 @@ __global__ void latent_write_kernel(const float* __restrict__ down, int down_ld,
             row[rank + i] = hb_from_float<TC>(v);
         }
     }
+    if (q_down) {
+        const float* in = q_down + (size_t)t * down_ld;
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < q_rank; i += blockDim.x) ss = fmaf(in[i], in[i], ss);
+        ss = hb_block_sum(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)q_rank + eps);
+        for (int i = threadIdx.x; i < q_rank; i += blockDim.x)
+            c_q[(size_t)t * q_rank + i] = hb_from_float<TC>(in[i] * inv * q_norm_w[i]);
+    }
     for (int e = threadIdx.x; e < H * rot; e += blockDim.x) {
         const int h = e / rot, i = e % rot;
         const float* in = q + (size_t)t * q_ld + (size_t)h * (qd + rot) + qd;
@@ -90,17 +103,20 @@ extern "C" int hb_latent_write(const float* down, int down_ld, const float* norm
                                void* q_plain, const float* inv_freq, const int* positions, const int* seq_of, const int* slots,
                                const int* page_table, int max_pages, int page_size, void* pages, int dtype, int T,
                                int H, int qd, int rank, int rot, int rot_dims, float eps, int write_cache,
-                               hipStream_t stream) {
-    HB_REQUIRE(T > 0 && H > 0 && rank > 0 && rot >= 0 && qd >= 0, "latent write: empty input");
+                               const float* q_down, int q_rank, const float* q_norm_w, void* c_q, hipStream_t stream) {
+    HB_REQUIRE(!q_down || (q_rank > 0 && q_norm_w && c_q), "latent write: a query latent needs its norm and a place");
+    HB_REQUIRE(T > 0 && (H > 0 || (H == 0 && (q_down || write_cache))) && rank > 0 && rot >= 0 && qd >= 0, "latent write: empty input");
     HB_REQUIRE(rot_dims >= 0 && rot_dims <= rot && rot_dims % 2 == 0, "latent write: %d rotated of %d", rot_dims, rot);
     if (dtype == HB_F32)
         latent_write_kernel<float><<<T, 256, 0, stream>>>(down, down_ld, norm_w, q, q_ld, q_full, (bf16*)q_plain, inv_freq, positions, seq_of, slots,
                                                           page_table, max_pages, page_size, (float*)pages, H, qd,
-                                                          rank, rot, rot_dims, eps, write_cache);
+                                                          rank, rot, rot_dims, eps, write_cache, q_down, q_rank, q_norm_w,
+                                                          (float*)c_q);
     else if (dtype == HB_BF16)
         latent_write_kernel<bf16><<<T, 256, 0, stream>>>(down, down_ld, norm_w, q, q_ld, q_full, (bf16*)q_plain, inv_freq, positions, seq_of, slots,
                                                          page_table, max_pages, page_size, (bf16*)pages, H, qd,
-                                                         rank, rot, rot_dims, eps, write_cache);
+                                                         rank, rot, rot_dims, eps, write_cache, q_down, q_rank, q_norm_w,
+                                                          (bf16*)c_q);
     else
         HB_REQUIRE(false, "latent write: unknown dtype %d", dtype);
     HB_CHECK_LAUNCH("latent_write");
@@ -112,14 +128,15 @@ extern "C" int hb_latent_write(const float* down, int down_ld, const float* norm
 // chunks of 64 that start at multiples of 64 of the absolute position, with an online softmax, so
 // the rounding depends on the positions only, not on how the tokens were cut into steps or batches.
 // out[t, h, :rank] = sum_j p_j c_j, times sigmoid(gate[t * gate_ld + h]) if a gate is given (the
-// head's output is linear in it, so the gate may be applied before W_uv).
+// head's output is linear in it, so the gate may be applied before W_uv). With sinks [H] the softmax's
+// denominator of head h also holds exp(sinks[h]), unscaled, once, without key or value.
 template <class TC, class TO>
 __global__ void __launch_bounds__(HB_WAVE)
 latent_attention_plain_kernel(const float* __restrict__ q_full, const TC* __restrict__ pages,
                               TO* __restrict__ out, const float* __restrict__ gate, int gate_ld,
                               const int* __restrict__ positions, const int* __restrict__ seq_of,
                               const int* __restrict__ slots, const int* __restrict__ page_table, int max_pages,
-                              int page_size, int H, int rank, int rot, float scale) {
+                              int page_size, int H, int rank, int rot, float scale, const float* __restrict__ sinks) {
     __shared__ float qs[HB_MAX_KEY];
     __shared__ float ps[HB_WAVE];
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
@@ -132,6 +149,7 @@ latent_attention_plain_kernel(const float* __restrict__ q_full, const TC* __rest
 
     const int hi = pos + 1;
     float m = -INFINITY, l = 0.f;
+    if (sinks) m = sinks[h], l = 1.0f;
     float acc[ACC_REGS];
 #pragma unroll
     for (int i = 0; i < ACC_REGS; ++i) acc[i] = 0.f;
@@ -181,7 +199,8 @@ latent_attention_plain_kernel(const float* __restrict__ q_full, const TC* __rest
 extern "C" int hb_latent_attention_plain(const float* q_full, const void* pages, void* out, int dtype,
                                          const float* gate, int gate_ld, const int* positions, const int* seq_of,
                                          const int* slots, const int* page_table, int max_pages, int page_size,
-                                         int T, int H, int rank, int rot, float scale, hipStream_t stream) {
+                                         int T, int H, int rank, int rot, float scale, const float* sinks,
+                                         hipStream_t stream) {
     HB_REQUIRE(T > 0 && H > 0 && H <= 65535, "latent attention: empty input or too many heads");
     HB_REQUIRE(rank > 0 && rank <= HB_MAX_RANK && rot >= 0 && rank + rot <= HB_MAX_KEY,
                "latent attention: a latent of %d + %d, the kernel takes up to %d + %d", rank, rot, HB_MAX_RANK,
@@ -190,11 +209,11 @@ extern "C" int hb_latent_attention_plain(const float* q_full, const void* pages,
     if (dtype == HB_F32)
         latent_attention_plain_kernel<float, float><<<grid, HB_WAVE, 0, stream>>>(
             q_full, (const float*)pages, (float*)out, gate, gate_ld, positions, seq_of, slots, page_table, max_pages,
-            page_size, H, rank, rot, scale);
+            page_size, H, rank, rot, scale, sinks);
     else if (dtype == HB_BF16)
         latent_attention_plain_kernel<bf16, bf16><<<grid, HB_WAVE, 0, stream>>>(
             q_full, (const bf16*)pages, (bf16*)out, gate, gate_ld, positions, seq_of, slots, page_table, max_pages,
-            page_size, H, rank, rot, scale);
+            page_size, H, rank, rot, scale, sinks);
     else
         HB_REQUIRE(false, "latent attention: unknown dtype %d", dtype);
     HB_CHECK_LAUNCH("latent_attention_plain");
@@ -234,7 +253,7 @@ latent_attention_mfma_kernel(const float* __restrict__ q_full, const bf16* __res
                              const float* __restrict__ gate, int gate_ld, const int* __restrict__ positions,
                              const int* __restrict__ seq_of, const int* __restrict__ slots,
                              const int* __restrict__ page_table, int max_pages, int page_size, int H, int rank,
-                             int rot, float scale, int splits, int chunks_per_split) {
+                             int rot, float scale, int splits, int chunks_per_split, const float* __restrict__ sinks) {
     __shared__ __attribute__((aligned(16))) __bf16 Vt[RB * 16 * LA_VT_STRIDE];
     const int HB = (H + 15) / 16;
     const int t = blockIdx.x / HB, hb = blockIdx.x % HB, split = blockIdx.y;
@@ -347,6 +366,7 @@ latent_attention_mfma_kernel(const float* __restrict__ q_full, const bf16* __res
     // acc[db][i]: number 16 db + 4 g + i of head n's sum
     const size_t row = (size_t)t * H + h;
     if (splits == 1) {
+        if (sinks) l += expf(sinks[h] - m);                 // (an infinite share, a sink far above every score, leaves 0)
         float w = l > 0.f ? 1.0f / l : 0.f;
         if (gate) w *= 1.0f / (1.0f + expf(-gate[(size_t)t * gate_ld + h]));
 #pragma unroll
@@ -371,7 +391,8 @@ latent_attention_mfma_kernel(const float* __restrict__ q_full, const bf16* __res
 // denominators, times sigmoid(gate). One block a (token, head).
 __global__ void __launch_bounds__(256)
 latent_merge_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml, bf16* __restrict__ out,
-                    const float* __restrict__ gate, int gate_ld, int H, int rank, int splits) {
+                    const float* __restrict__ gate, int gate_ld, int H, int rank, int splits,
+                    const float* __restrict__ sinks) {
     __shared__ float share[HB_WAVE + 1];          // the ranges' weights, and the row's factor
     const size_t row = blockIdx.x;
     if (threadIdx.x < HB_WAVE) {
@@ -382,7 +403,8 @@ latent_merge_kernel(const float* __restrict__ part_acc, const float* __restrict_
         const float ls = has ? part_ml[(row * splits + lane) * 2 + 1] : 0.f;
         const float m = hb_wave_max(ms);
         const float ws = ms > -INFINITY ? expf(ms - m) : 0.f;
-        const float l = hb_wave_sum(ls * ws);
+        float l = hb_wave_sum(ls * ws);
+        if (sinks) l += expf(sinks[row % H] - m);           // once, whatever the ranges
         float w = l > 0.f ? 1.0f / l : 0.f;
         if (gate) w *= 1.0f / (1.0f + expf(-gate[(row / H) * gate_ld + row % H]));
         share[lane] = ws;
@@ -411,7 +433,7 @@ extern "C" int hb_latent_attention_mfma(const float* q_full, const void* pages, 
                                         float* part_ml, const float* gate, int gate_ld, const int* positions,
                                         const int* seq_of, const int* slots, const int* page_table, int max_pages,
                                         int page_size, int T, int H, int rank, int rot, float scale, int splits,
-                                        int chunks_per_split, hipStream_t stream) {
+                                        int chunks_per_split, const float* sinks, hipStream_t stream) {
     HB_REQUIRE(T > 0 && H > 0, "latent attention: empty input");
     HB_REQUIRE(rank > 0 && rank % 32 == 0 && rank <= 512 && rot % 32 == 0 && rank + rot <= 640,
                "latent attention: the matrix-core kernel takes a latent and a rotated part in steps of 32, up to 512 + 128, not %d + %d", rank, rot);
@@ -424,14 +446,14 @@ extern "C" int hb_latent_attention_mfma(const float* q_full, const void* pages, 
 #define LA_LAUNCH(RBV, KSV)                                                                                      \
     latent_attention_mfma_kernel<RBV, KSV><<<grid, HB_WAVE, 0, stream>>>(                                          \
         q_full, (const bf16*)pages, (bf16*)out, part_acc, part_ml, gate, gate_ld, positions, seq_of, slots,      \
-        page_table, max_pages, page_size, H, rank, rot, scale, splits, chunks_per_split)
+        page_table, max_pages, page_size, H, rank, rot, scale, splits, chunks_per_split, sinks)
     if (rank <= 128 && rank + rot <= 256) LA_LAUNCH(8, 8);
     else if (rank <= 256 && rank + rot <= 384) LA_LAUNCH(16, 12);
     else LA_LAUNCH(32, 20);
 #undef LA_LAUNCH
     HB_CHECK_LAUNCH("latent_attention_mfma");
     if (splits > 1) {
-        latent_merge_kernel<<<(unsigned)((long long)T * H), 256, 0, stream>>>(part_acc, part_ml, (bf16*)out, gate, gate_ld, H, rank, splits);
+        latent_merge_kernel<<<(unsigned)((long long)T * H), 256, 0, stream>>>(part_acc, part_ml, (bf16*)out, gate, gate_ld, H, rank, splits, sinks);
         HB_CHECK_LAUNCH("latent_merge");
     }
     return 0;

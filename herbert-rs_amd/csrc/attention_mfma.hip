@@ -56,6 +56,33 @@ __device__ __forceinline__ int first_visible(int pos, int window, int chunk) {
     return (window > 0 && pos + 1 > window) ? pos + 1 - window : 0;
 }
 
+// A window that keeps the sequence's first keys as well (a query at i sees j <= i with i - j < window or
+// j < keep_first), and a bias by distance, added to the scores: the kernels' EXT form. A head's biases lie in
+// units of the raw dot products (bias / scale) along the keys: rel[h * ld + at + len - 1 - n] for the distance
+// n = i - j, with the value of n = len - 1 once more for every n beyond it (REL_FRONT of them lie before it, for
+// runs of keys that cross that border) and REL_BACK unused numbers behind n = 0 (keys behind the query,
+// which the mask hides). Scores start from their bias: it is what the accumulators hold before the first product.
+#define REL_FRONT 8
+#define REL_BACK 64
+struct AttnExtras {
+    const float* rel;       // null: no bias
+    int len, ld, at;
+    int keep_first;
+};
+
+// The pages that queries with the first visible key lo walk: those of the kept first keys, then those from lo's
+// on, counted without the gap between them. page = v < kept ? v : v + skip.
+struct PageWalk {
+    int kept, skip;
+    __device__ __forceinline__ PageWalk(int lo, int keep_first) {
+        kept = keep_first > 0 ? (keep_first + PAGE - 1) / PAGE : 0;
+        const int lo_page = lo / PAGE;
+        skip = lo_page > kept ? lo_page - kept : 0;
+    }
+    __device__ __forceinline__ int page(int v) const { return v < kept ? v : v + skip; }
+    __device__ __forceinline__ int upto(int page_idx) const { return page_idx - skip; }      // of a page >= lo's
+};
+
 // Capped scores: s <- cap tanh(s / cap), in the units of the raw dot products (cap = softcap / scale, so that
 // the scaled score is softcap tanh(scale s / softcap)). tanh t = 1 - 2 / (1 + e^(2t)): e^(2t) infinite gives 1,
 // zero gives -1.
@@ -75,7 +102,8 @@ __device__ __forceinline__ int acc_key(int kb, int g2, int i) { return kb * 32 +
 
 // One page of scores: mask, online-softmax update, P^T as MFMA operands.
 // st[kb]: S^T accumulators (raw dot products). c = scale * log2(e).
-// Keys k with lo <= page0 + k <= hi are visible; MASKED = false: the caller knows that all are.
+// Keys k with lo <= page0 + k <= hi (and the sequence's first `keep`) are visible; MASKED = false: the caller
+// knows that all are.
 // m is the reference of the exponents, not always the maximum: it is moved up (and the sums so
 // far scaled by corr < 1) only when a score exceeds it by more than 8 / c, that is when a
 // probability would exceed 2^8 times the largest so far; till then corr is 1 and the caller
@@ -99,7 +127,7 @@ __device__ __forceinline__ float sink_share(float sink, float m, float c) {
 }
 template <bool MASKED>
 __device__ __forceinline__ void softmax_page(f32x16 st[2], int g2, int page0, int lo, int hi, float c,
-                                             float& m, float& l, float& corr, bf16x8 pb[2][2]) {
+                                             float& m, float& l, float& corr, bf16x8 pb[2][2], int keep = 0) {
     float mx = -INFINITY;
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb)
@@ -107,7 +135,7 @@ __device__ __forceinline__ void softmax_page(f32x16 st[2], int g2, int page0, in
         for (int i = 0; i < 16; ++i) {
             if (MASKED) {
                 const int key = page0 + acc_key(kb, g2, i);
-                st[kb][i] = (key >= lo && key <= hi) ? st[kb][i] : -INFINITY;
+                st[kb][i] = ((key >= lo || key < keep) && key <= hi) ? st[kb][i] : -INFINITY;
             }
             mx = fmaxf(mx, st[kb][i]);
         }
@@ -145,7 +173,7 @@ __device__ __forceinline__ void rescale(f32x16 (&oacc)[NACC], float corr) {
 // need be. Returns m * c (what is taken off the scaled scores), corr as softmax_page does.
 template <bool MASKED>
 __device__ __forceinline__ float softmax_reference(f32x16 st[2], int g2, int page0, int lo, int hi, float c,
-                                                   float& m, float& corr) {
+                                                   float& m, float& corr, int keep = 0) {
     float mx = -INFINITY;
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb)
@@ -153,7 +181,7 @@ __device__ __forceinline__ float softmax_reference(f32x16 st[2], int g2, int pag
         for (int i = 0; i < 16; ++i) {
             if (MASKED) {
                 const int key = page0 + acc_key(kb, g2, i);
-                st[kb][i] = (key >= lo && key <= hi) ? st[kb][i] : -INFINITY;
+                st[kb][i] = ((key >= lo || key < keep) && key <= hi) ? st[kb][i] : -INFINITY;
             }
             mx = fmaxf(mx, st[kb][i]);
         }
@@ -215,7 +243,8 @@ struct PrefillLane {
 // kst: the stage of the next page's keys; vst: the stage of this page's values. After the last
 // page the scores "of the next" are worked out all the same, from whatever that stage holds,
 // and never looked at: a second copy of the code without them costs more registers than a wave has.
-template <int HD>
+// STARTED: nxt already holds what the scores start from (else zero).
+template <int HD, bool STARTED = false>
 __device__ __forceinline__ void prefill_step_products(const bf16* kst, const bf16* vst, f32x16 (&st)[2],
                                                       f32x16 (&nxt)[2], f32x16 (&oacc)[HD / 32],
                                                       const bf16x8 (&qreg)[HD / 16], const PrefillLane& ln, float c,
@@ -241,10 +270,12 @@ __device__ __forceinline__ void prefill_step_products(const bf16* kst, const bf1
         }
     };
     (void)KRPB;
+    if (!STARTED) {
 #pragma unroll
-    for (int kb = 0; kb < 2; ++kb)
+        for (int kb = 0; kb < 2; ++kb)
 #pragma unroll
-        for (int e = 0; e < 16; ++e) nxt[kb][e] = 0.f;
+            for (int e = 0; e < 16; ++e) nxt[kb][e] = 0.f;
+    }
     bf16x8 ops[NM];
     bf16x8 pb[4];
     float sum = 0.f;
@@ -280,6 +311,41 @@ __device__ __forceinline__ void prefill_step_products(const bf16* kst, const bf1
     l = l * corr + sum;      // this lane's keys only; the two halves are added at the end
 }
 
+// The biases of one wave's next page of scores (EXT): 32 queries from pos0 on against 64 keys from page0 on are
+// 95 neighbouring distances, which the lanes ask for a page ahead (ask), put into the wave's own stretch of LDS
+// (128 numbers) and hand out from there (start: what the accumulators begin with).
+struct PageBias {
+    const float* row;        // this head's biases, at n = len - 1
+    float* buf;
+    int last, lane;
+    float v0, v1;
+    __device__ __forceinline__ PageBias(const AttnExtras& ext, int head, float* lds, int lane_)
+        : row(ext.rel + (size_t)head * ext.ld + ext.at), buf(lds), last(ext.len - 1), lane(lane_), v0(0.f), v1(0.f) {}
+    __device__ __forceinline__ float at(int n) const {
+        n = n > last ? last : n;
+        return row[last - (n > 0 ? n : 0)];
+    }
+    __device__ __forceinline__ void ask(int pos0, int page0) {
+        const int n = pos0 + 31 - page0 - lane;
+        v0 = at(n);
+        v1 = at(n - 64);
+    }
+    __device__ __forceinline__ void start(f32x16 (&st)[2], int c32, int g2) {
+        __builtin_amdgcn_wave_barrier();
+        buf[lane] = v0;
+        buf[lane + 64] = v1;
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+        const float* p = buf + 31 - c32;
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+            for (int i = 0; i < 16; ++i) st[kb][i] = p[acc_key(kb, g2, i)];
+        __builtin_amdgcn_wave_barrier();
+    }
+};
+#define PAGE_BIAS_FLOATS 128
+
 // A workgroup: 32 queries x up to 4 query heads of one kv head, by eight waves in two groups of
 // four (a wave a head in each group). The groups take the tile's pages in turn, the first the
 // even ones and the second the odd ones, each with a reference, a sum and an output of its
@@ -292,7 +358,7 @@ __device__ __forceinline__ void prefill_step_products(const bf16* kst, const bf1
 // reads of 16 rows at one chunk fall into 16 different bank groups.
 // Workgroups are numbered by falling work (the host sorts the tiles): a CU that is done takes
 // the heaviest tile left.
-template <int HD>
+template <int HD, bool EXT>
 __global__ void __launch_bounds__(512, 1)
 attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache,
                     const bf16* __restrict__ v_cache, bf16* __restrict__ out,
@@ -300,7 +366,7 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache
                     const int* __restrict__ tile_rows, const int* __restrict__ positions,
                     const int* __restrict__ slots, const int* __restrict__ page_table, int max_pages, int nq,
                     int nkv, float c, int window, int per_tile, const float* __restrict__ sinks, int chunked,
-                    float cap) {
+                    float cap, AttnExtras ext) {
     constexpr int KCH = HD / 8;                   // 16-byte chunks of a key row
     constexpr int KRPB = 128 / HD > 0 ? 128 / HD : 1;   // key rows in 256 bytes
     constexpr int KROWS = 512 / HD;               // key rows a load instruction brings (1 KB)
@@ -310,7 +376,7 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache
     // compiler knows which loads-to-LDS may alias a read and waits for every load in flight
     // (s_waitcnt vmcnt(0)) before the first read that follows, which undoes the ring: the loads of
     // the next pages would be waited for at once. What has to have landed is waited for by hand.
-    extern __shared__ __attribute__((aligned(1024))) bf16 attn_lds[];     // [group][keys [2][STAGE], values [2][STAGE]]
+    extern __shared__ __attribute__((aligned(1024))) bf16 attn_lds[];     // [group][keys [2][STAGE], values [2][STAGE]], EXT: [wave][PAGE_BIAS_FLOATS]
 
     const int w = blockIdx.x;
     const int tile = w / per_tile, y = w % per_tile;
@@ -339,11 +405,14 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache
     const int hi_tile = pos0 + rows - 1;                                     // last visible key
     const int lo_tile = first_visible(pos0, window, chunked);
     const int lo_last = first_visible(hi_tile, window, chunked);            // what the tile's last query sees first
-    const int first_page = lo_tile / PAGE, last_page = hi_tile / PAGE;
+    const int keep = EXT ? ext.keep_first : 0;
+    const PageWalk walk(lo_tile, keep);
+    // (EXT: pages are counted along the walk)
+    const int first_page = EXT ? 0 : lo_tile / PAGE, last_page = EXT ? walk.upto(hi_tile / PAGE) : hi_tile / PAGE;
     // this group's pages: first_page + grp, + 2, ...; the first group has as many as the second or one more
     const int steps = (last_page - first_page) / 2 + 1;                      // of the first group: every wave loops so often
     const int mine = last_page - first_page - grp >= 0 ? (last_page - first_page - grp) / 2 + 1 : 0;
-    auto page_of = [&](int i) { return first_page + grp + 2 * i; };
+    auto page_of = [&](int i) { const int v = first_page + grp + 2 * i; return EXT ? walk.page(v) : v; };
 
     // this lane's part of the loads of a page: element offsets within the page's keys and values
     int k_off[LOADS], v_off[LOADS];
@@ -395,11 +464,20 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache
     const PrefillLane ln = {c32, g2, krow, {k_read[0], k_read[1]}, v_swz};
     // raw scores of the page in a key stage; the two key blocks alternate, so that no MFMA waits
     // for the one before it
-    auto scores = [&](int stage, f32x16 (&st)[2]) {
+    PageBias bias(ext, h, (float*)(attn_lds + 8 * STAGE) + wave8 * PAGE_BIAS_FLOATS, lane);
+    const bool biased = EXT && ext.rel != nullptr;
+    auto start = [&](f32x16 (&st)[2]) {
+        if (biased) {
+            bias.start(st, c32, g2);
+            return;
+        }
 #pragma unroll
         for (int kb = 0; kb < 2; ++kb)
 #pragma unroll
             for (int i = 0; i < 16; ++i) st[kb][i] = 0.f;
+    };
+    auto scores = [&](int stage, f32x16 (&st)[2]) {
+        start(st);
 #pragma unroll
         for (int s = 0; s < HD / 16; ++s)
 #pragma unroll
@@ -422,20 +500,28 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache
         // a page that every query of the tile sees whole needs no mask
         const int page0 = page_of(i) * PAGE;
         if (cap != 0.f) cap_scores(st, cap);
-        if (page0 + PAGE - 1 <= pos0 && page0 >= lo_last)
+        if (EXT) {
+            start(nxt);                                             // (asked for a step ago)
+            if (biased) bias.ask(pos0, page_of(i + 2) * PAGE);
+        }
+        if (page0 + PAGE - 1 <= pos0 && (page0 >= lo_last || (EXT && page0 + PAGE <= keep)))
             mc = softmax_reference<false>(st, g2, page0, lo_q, pos_q, c, m, corr);
         else
-            mc = softmax_reference<true>(st, g2, page0, lo_q, pos_q, c, m, corr);
+            mc = softmax_reference<true>(st, g2, page0, lo_q, pos_q, c, m, corr, keep);
         rescale(oacc, corr);          // rarely: the reference moves lazily
         // (the parity of the step is known where the code is written out, twice a round: the stage
         // of an operand is then a constant offset of its read and costs no register)
         constexpr int PAR = decltype(parity_tag)::value;
-        prefill_step_products<HD>(Ks + ((PAR + 1) & 1) * STAGE, Vs + PAR * STAGE, st, nxt, oacc, qreg, ln, c, mc, corr, l);
+        prefill_step_products<HD, EXT>(Ks + ((PAR + 1) & 1) * STAGE, Vs + PAR * STAGE, st, nxt, oacc, qreg, ln, c, mc, corr, l);
     };
     hb_wait_vmcnt<0>();
     hb_workgroup_barrier();
     f32x16 sa[2], sb[2];
-    if (active && mine > 0) scores(0, sa);
+    if (active && mine > 0) {
+        if (biased) bias.ask(pos0, page_of(0) * PAGE);
+        scores(0, sa);
+        if (biased) bias.ask(pos0, page_of(1) * PAGE);
+    }
     for (int i = 0; i < steps; i += 2) {           // two steps a round: the scores change places, nothing is copied
         step(std::integral_constant<int, 0>{}, i, sa, sb);
         if (i + 1 < steps) step(std::integral_constant<int, 1>{}, i + 1, sb, sa);
@@ -493,7 +579,7 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache
 // Every wave issues the same number of loads in every step (past the last page: that page again,
 // into a stage nobody reads any more), so that the wait before the barrier can count: all but
 // the loads of the step before have landed.
-template <int HD>
+template <int HD, bool EXT>
 __global__ void __launch_bounds__(512, 1)
 attn_prefill_long_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache,
                          const bf16* __restrict__ v_cache, bf16* __restrict__ out,
@@ -501,14 +587,14 @@ attn_prefill_long_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
                          const int* __restrict__ tile_rows, const int* __restrict__ positions,
                          const int* __restrict__ slots, const int* __restrict__ page_table, int max_pages,
                          int nq, int nkv, float c, int window, int per_tile,
-                         const float* __restrict__ sinks, int chunked, float cap) {
+                         const float* __restrict__ sinks, int chunked, float cap, AttnExtras ext) {
     constexpr int KCH = HD / 8;
     constexpr int KRPB = 128 / HD > 0 ? 128 / HD : 1;
     constexpr int KROWS = 512 / HD;
     constexpr int INSTRS = HD / 8;                // load instructions (1 KB each) for the keys of a page; as many for the values
     constexpr int PL = INSTRS >= 8 ? INSTRS / 8 : 1;   // of which a wave issues (with fewer than 8, the first waves one each)
     constexpr int STAGE = PAGE * HD;
-    extern __shared__ __attribute__((aligned(1024))) bf16 attn_lds[];     // keys [3][STAGE], values [3][STAGE]
+    extern __shared__ __attribute__((aligned(1024))) bf16 attn_lds[];     // keys [3][STAGE], values [3][STAGE], EXT: [wave][PAGE_BIAS_FLOATS]
     bf16* const Ks = attn_lds;
     bf16* const Vs = attn_lds + 3 * STAGE;
 
@@ -540,10 +626,17 @@ attn_prefill_long_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     const int lo_last = first_visible(hi_half, window, chunked);             // what the half's last query sees first
     // the workgroup's pages: from the first a row of the tile sees to the last
     const int lo_tile = first_visible(tile_pos0, window, chunked);
-    const int first_page = lo_tile / PAGE, last_page = (tile_pos0 + tile_n - 1) / PAGE;
+    const int keep = EXT ? ext.keep_first : 0;
+    const PageWalk walk(lo_tile, keep);                                       // (EXT: pages are counted along the walk)
+    const int first_page = EXT ? 0 : lo_tile / PAGE, hi_page = (tile_pos0 + tile_n - 1) / PAGE;
+    const int last_page = EXT ? walk.upto(hi_page) : hi_page;
     const int steps = last_page - first_page + 1;
-    const int mine = active ? hi_half / PAGE - first_page + 1 : 0;            // this half's steps: pages up to its own last
-    auto page_of = [&](int i) { return first_page + (i < steps ? i : steps - 1); };   // past the end: the last page again
+    // this half's steps: pages up to its own last
+    const int mine = active ? (EXT ? walk.upto(hi_half / PAGE) : hi_half / PAGE) - first_page + 1 : 0;
+    auto page_of = [&](int i) {                                               // past the end: the last page again
+        const int v = first_page + (i < steps ? i : steps - 1);
+        return EXT ? walk.page(v) : v;
+    };
 
     int k_off[PL], v_off[PL];
     const bool loads = INSTRS >= 8 || wave8 < INSTRS;
@@ -602,6 +695,18 @@ attn_prefill_long_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     for (int kb = 0; kb < 2; ++kb) ln.k_read[kb] = ((kb * 32 + krow) / KRPB) % KCH;
     ln.v_swz = (c32 >> 1) & 7;
 
+    PageBias bias(ext, h, (float*)(attn_lds + 6 * STAGE) + wave8 * PAGE_BIAS_FLOATS, lane);
+    const bool biased = EXT && ext.rel != nullptr;
+    auto start = [&](f32x16 (&st)[2]) {
+        if (biased) {
+            bias.start(st, c32, g2);
+            return;
+        }
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+            for (int i = 0; i < 16; ++i) st[kb][i] = 0.f;
+    };
     auto step = [&](int i, f32x16 (&st)[2], f32x16 (&nxt)[2]) {
         // landed, for every wave after the barrier: all but what the step before asked for, that is
         // the keys of page i + 1 and the values of page i; and nobody reads any more the stages that
@@ -614,12 +719,16 @@ attn_prefill_long_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
         float corr, mc;
         const int page0 = page_of(i) * PAGE;
         if (cap != 0.f) cap_scores(st, cap);
-        if (page0 + PAGE - 1 <= pos0 && page0 >= lo_last)
+        if (EXT) {
+            start(nxt);                                             // (asked for a step ago)
+            if (biased) bias.ask(pos0, page_of(i + 2) * PAGE);      // (more loads in flight: the count above only waits for more)
+        }
+        if (page0 + PAGE - 1 <= pos0 && (page0 >= lo_last || (EXT && page0 + PAGE <= keep)))
             mc = softmax_reference<false>(st, g2, page0, lo_q, pos_q, c, m, corr);
         else
-            mc = softmax_reference<true>(st, g2, page0, lo_q, pos_q, c, m, corr);
+            mc = softmax_reference<true>(st, g2, page0, lo_q, pos_q, c, m, corr, keep);
         rescale(oacc, corr);
-        prefill_step_products<HD>(Ks + ((i + 1) % 3) * STAGE, Vs + (i % 3) * STAGE, st, nxt, oacc, qreg, ln, c, mc,
+        prefill_step_products<HD, EXT>(Ks + ((i + 1) % 3) * STAGE, Vs + (i % 3) * STAGE, st, nxt, oacc, qreg, ln, c, mc,
                                   corr, l);
     };
     // the first page's scores: its keys are the oldest of the five sets of loads (and of the
@@ -628,10 +737,9 @@ attn_prefill_long_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     hb_workgroup_barrier();
     f32x16 sa[2], sb[2];
     if (mine > 0) {
-#pragma unroll
-        for (int kb = 0; kb < 2; ++kb)
-#pragma unroll
-            for (int i = 0; i < 16; ++i) sa[kb][i] = 0.f;
+        if (biased) bias.ask(pos0, page_of(0) * PAGE);
+        start(sa);
+        if (biased) bias.ask(pos0, page_of(1) * PAGE);
 #pragma unroll
         for (int s2 = 0; s2 < HD / 16; ++s2)
 #pragma unroll
@@ -684,7 +792,7 @@ struct DecodeFusion {
     int q_temp_every;
 };
 
-template <int HD, bool FUSED, int QS = 1>
+template <int HD, bool FUSED, bool EXT, int QS = 1>
 __global__ void __launch_bounds__(64)
 attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16* __restrict__ v_cache,
                    float* __restrict__ partial_o, float* __restrict__ partial_ml,
@@ -692,7 +800,7 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
                    const int* __restrict__ page_table, int max_pages, int nq, int nkv, float c, int window,
                    int pages_per_split, DecodeFusion fu, bf16* __restrict__ out,
                    const int* __restrict__ ranges, int n_seqs, const float* __restrict__ sinks, int chunked,
-                   float cap) {
+                   float cap, AttnExtras ext) {
     // ranges == null: the grid is (sequence, kv head, range), every sequence cut into gridDim.z
     // ranges of pages_per_split pages (those past a sequence's end hold nothing).
     // ranges != null (sequences of unequal lengths): the grid is (1, kv head, item);
@@ -719,9 +827,13 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
     const int ctx = context_lens[b];                 // keys 0 .. ctx-1; the query sits at ctx-1
     const int hi = ctx - 1;
     const int lo = first_visible(hi, window, chunked);
-    const int first_page = lo / PAGE + split * pages_per_split;
+    const int keep = EXT ? ext.keep_first : 0;
+    const PageWalk walk(lo, keep);                   // (EXT: pages are counted along the walk)
+    auto page_at = [&](int v) { return EXT ? walk.page(v) : v; };
+    const int hp = EXT ? walk.upto(hi / PAGE) : hi / PAGE;       // the page of the new position
+    const int first_page = (EXT ? 0 : lo / PAGE) + split * pages_per_split;
     int last_page = first_page + pages_per_split - 1;
-    if (last_page > hi / PAGE) last_page = hi / PAGE;
+    if (last_page > hp) last_page = hp;
     const int* pt = page_table + (size_t)slots[b] * max_pages;
     const int head = kvh * G + (c32 < G ? c32 : G - 1);
 
@@ -741,7 +853,6 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
     constexpr int PER = 64 / HALF;                 // heads a round of the wave covers
     constexpr int PRE = 4;                         // rounds whose inputs are loaded ahead
     const int j = lane % HALF, sub = lane / HALF;
-    const int hp = hi / PAGE;
     const bool writer = FUSED && fu.write_kv && hp >= first_page && hp < first_page + pages_per_split;
     float cs = 1.f, sn = 0.f, qw0 = 1.f, qw1 = 1.f, kw0 = 1.f, kw1 = 1.f;
     float xq0[PRE], xq1[PRE], k0 = 0.f, k1 = 0.f, v0 = 0.f, v1 = 0.f;
@@ -785,7 +896,7 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
                 kw0 = fu.k_norm_w[j];
                 kw1 = fu.k_norm_w[j + HALF];
             }
-            new_page = pt[hp];
+            new_page = pt[page_at(hp)];
         }
     }
     f32x16 oacc[HD / 32];
@@ -802,14 +913,38 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
     bf16x8 va[HD / 32][2][2];
 #define LOAD_K(PAGE_IDX)                                                                     \
     {                                                                                        \
-        const bf16* kp = k_cache + ((size_t)pt[PAGE_IDX] * nkv + kvh) * PAGE * HD + g2 * (HD / 2); \
+        const bf16* kp = k_cache + ((size_t)pt[page_at(PAGE_IDX)] * nkv + kvh) * PAGE * HD + g2 * (HD / 2); \
         _Pragma("unroll") for (int kb = 0; kb < 2; ++kb)                                     \
             _Pragma("unroll") for (int s = 0; s < HD / 16; ++s)                              \
                 ka[kb][s] = *(const bf16x8*)(kp + (size_t)(kb * 32 + krow) * HD + s * 8);    \
     }
+// (EXT: what the scores of a page start from: a lane's head, four runs of 8 neighbouring keys)
+    const bool biased = EXT && ext.rel != nullptr;
+    const float* const rel = biased ? ext.rel + (size_t)head * ext.ld + ext.at : nullptr;
+    f32x16 from[2];
+    auto load_bias = [&](int v) {
+        if (!biased) {
+#pragma unroll
+            for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+                for (int i = 0; i < 16; ++i) from[kb][i] = 0.f;
+            return;
+        }
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+            for (int h2 = 0; h2 < 2; ++h2) {
+                int x = ext.len - 1 - (hi - (page_at(v) * PAGE + acc_key(kb, g2, 8 * h2)));
+                x = x < -REL_FRONT ? -REL_FRONT : x;
+                typedef float f32x4u __attribute__((ext_vector_type(4), aligned(4)));
+                const f32x4u r0 = *(const f32x4u*)(rel + x), r1 = *(const f32x4u*)(rel + x + 4);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) from[kb][8 * h2 + e] = r0[e], from[kb][8 * h2 + 4 + e] = r1[e];
+            }
+    };
 #define LOAD_V(PAGE_IDX)                                                                     \
     {                                                                                        \
-        const bf16* vp = v_cache + ((size_t)pt[PAGE_IDX] * nkv + kvh) * HD * PAGE + g2 * 8;  \
+        const bf16* vp = v_cache + ((size_t)pt[page_at(PAGE_IDX)] * nkv + kvh) * HD * PAGE + g2 * 8;  \
         _Pragma("unroll") for (int d = 0; d < HD / 32; ++d)                                  \
             _Pragma("unroll") for (int kb = 0; kb < 2; ++kb)                                 \
                 _Pragma("unroll") for (int h2 = 0; h2 < 2; ++h2)                             \
@@ -898,24 +1033,27 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
 #pragma unroll
         for (int s2 = 0; s2 < HD / 16; ++s2) qreg[s2] = *(const bf16x8*)(qrow + s2 * 8);
     }
+    if (EXT && first_page <= last_page) load_bias(first_page);
     for (int page_idx = first_page; page_idx <= last_page; ++page_idx) {
         f32x16 st[2];
 #pragma unroll
         for (int kb = 0; kb < 2; ++kb) {
 #pragma unroll
-            for (int i = 0; i < 16; ++i) st[kb][i] = 0.f;
+            for (int i = 0; i < 16; ++i) st[kb][i] = EXT ? from[kb][i] : 0.f;
 #pragma unroll
             for (int s = 0; s < HD / 16; ++s)
                 st[kb] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ka[kb][s], qreg[s], st[kb], 0, 0, 0);
         }
         if (page_idx < last_page) LOAD_K(page_idx + 1)
+        if (EXT && page_idx < last_page) load_bias(page_idx + 1);
         float corr;
         bf16x8 pb[2][2];
         if (cap != 0.f) cap_scores(st, cap);
-        if (page_idx * PAGE >= lo && page_idx * PAGE + PAGE - 1 <= hi)
-            softmax_page<false>(st, g2, page_idx * PAGE, lo, hi, c, m, l, corr, pb);
+        const int page0 = page_at(page_idx) * PAGE;
+        if ((page0 >= lo || (EXT && page0 + PAGE <= keep)) && page0 + PAGE - 1 <= hi)
+            softmax_page<false>(st, g2, page0, lo, hi, c, m, l, corr, pb);
         else
-            softmax_page<true>(st, g2, page_idx * PAGE, lo, hi, c, m, l, corr, pb);
+            softmax_page<true>(st, g2, page0, lo, hi, c, m, l, corr, pb, keep);
         rescale(oacc, corr);
 #pragma unroll
         for (int d = 0; d < HD / 32; ++d) {
@@ -1041,12 +1179,24 @@ attn_decode_merge_kernel(const float* __restrict__ partial_o, const float* __res
 // ---------------------------------------------------------------- launchers
 #define LOG2E 1.4426950408889634f
 
+static int check_extras(const float* rel, int rel_len, int rel_ld, int keep_first, int window, int chunk, float softcap) {
+    if (!rel && keep_first == 0) return 0;
+    HB_REQUIRE(!rel || (rel_len > 0 && rel_ld >= REL_FRONT + rel_len + REL_BACK), "attention: a table of %d biases in rows of %d", rel_len, rel_ld);
+    HB_REQUIRE(keep_first >= 0 && (keep_first == 0 || window > 0), "attention: kept first keys go with a window");
+    HB_REQUIRE(chunk == 0 && softcap == 0.f, "attention: a bias by distance and kept first keys do not go with chunks and capped scores");
+    return 0;
+}
+
 extern "C" int hb_attn_prefill_mfma(const void* q, const void* k_cache, const void* v_cache, void* out,
                                     const int* tile_seq, const int* tile_row0, const int* tile_rows,
                                     int num_tiles, const int* positions, const int* slots,
                                     const int* page_table, int max_pages, int page_size, int nq, int nkv,
                                     int hd, float scale, int window, int tile_height, const float* sinks,
-                                    int chunk, float softcap, hipStream_t stream) {
+                                    int chunk, float softcap, const float* rel, int rel_len, int rel_ld,
+                                    int keep_first, hipStream_t stream) {
+    const bool extended = rel || keep_first > 0;
+    if (check_extras(rel, rel_len, rel_ld, keep_first, window, chunk, softcap)) return 1;
+    const AttnExtras ext = {rel, rel_len, rel_ld, REL_FRONT, keep_first};
     HB_REQUIRE(num_tiles > 0 && nq > 0 && nkv > 0 && nq % nkv == 0, "attn_prefill: bad sizes");
     HB_REQUIRE(page_size == PAGE, "attn_prefill: pages must hold %d tokens", PAGE);
     HB_REQUIRE(window >= 0 && chunk >= 0 && !(window > 0 && chunk > 0), "attn_prefill: bad window or chunk");
@@ -1061,20 +1211,26 @@ extern "C" int hb_attn_prefill_mfma(const void* q, const void* k_cache, const vo
     const float cap = softcap / scale;          // in the units of the raw dot products
     // tiles of 32 tokens: two groups of waves, each with two stages of keys and two of values;
     // tiles of 64: one ring of three stages of keys and three of values
-    const size_t lds = (size_t)(tile_height == 64 ? 6 : 8) * PAGE * hd * sizeof(bf16);
-#define LAUNCH_PREFILL(KERNEL, HDV)                                                                      \
+    const size_t lds = (size_t)(tile_height == 64 ? 6 : 8) * PAGE * hd * sizeof(bf16) +
+                       (extended ? 8 * PAGE_BIAS_FLOATS * sizeof(float) : 0);
+#define LAUNCH_PREFILL_FORM(KERNEL, HDV, FORM)                                                           \
     do {                                                                                                 \
         static bool allowed = false;            /* once a process (the attribute is the function's) */   \
         if (lds > 64 * 1024 && !allowed) {                                                               \
-            hipError_t e_ = hipFuncSetAttribute((const void*)KERNEL<HDV>,                                \
+            hipError_t e_ = hipFuncSetAttribute((const void*)KERNEL<HDV, FORM>,                          \
                                                 hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);   \
             HB_REQUIRE(e_ == hipSuccess, "attn_prefill: cannot have %zu bytes of LDS: %s", lds, hipGetErrorString(e_)); \
             allowed = true;                                                                              \
         }                                                                                                \
-        KERNEL<HDV><<<total, 512, lds, stream>>>((const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, \
+        KERNEL<HDV, FORM><<<total, 512, lds, stream>>>((const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, \
                                                  (bf16*)out, tile_seq, tile_row0, tile_rows, positions, slots, \
                                                  page_table, max_pages, nq, nkv, c, window, per_tile, sinks, \
-                                                 chunk, cap); \
+                                                 chunk, cap, ext); \
+    } while (0)
+#define LAUNCH_PREFILL(KERNEL, HDV)                                                                      \
+    do {                                                                                                 \
+        if (extended) LAUNCH_PREFILL_FORM(KERNEL, HDV, true);                                            \
+        else LAUNCH_PREFILL_FORM(KERNEL, HDV, false);                                                    \
     } while (0)
     if (tile_height == 64) {
         if (hd == 32) LAUNCH_PREFILL(attn_prefill_long_kernel, 32);
@@ -1088,6 +1244,7 @@ extern "C" int hb_attn_prefill_mfma(const void* q, const void* k_cache, const vo
         else HB_REQUIRE(false, "attn_prefill: head_dim %d is not one of 32, 64, 128", hd);
     }
 #undef LAUNCH_PREFILL
+#undef LAUNCH_PREFILL_FORM
     HB_CHECK_LAUNCH("attn_prefill");
     return 0;
 }
@@ -1102,7 +1259,11 @@ extern "C" int hb_attn_decode_mfma(const void* q, void* k_cache, void* v_cache, 
                                    const float* k_norm_w, const float* cos_t, const float* sin_t, float eps,
                                    int write_kv, int qkv_slices, size_t slice_stride, const int* ranges,
                                    float q_temp_coef, int q_temp_every, const float* sinks, int chunk,
-                                   float softcap, hipStream_t stream) {
+                                   float softcap, const float* rel, int rel_len, int rel_ld, int keep_first,
+                                   hipStream_t stream) {
+    const bool extended = rel || keep_first > 0;
+    if (check_extras(rel, rel_len, rel_ld, keep_first, window, chunk, softcap)) return 1;
+    const AttnExtras ext = {rel, rel_len, rel_ld, REL_FRONT, keep_first};
     // ranges != null: see attn_decode_kernel; `splits` is then the number of items of the grid (the
     // partial results are [nq, splits]), pages_per_split is not read
     HB_REQUIRE(!ranges || (B >= 2 && splits >= 2 && window == 0 && chunk == 0),
@@ -1125,22 +1286,29 @@ extern "C" int hb_attn_decode_mfma(const void* q, void* k_cache, void* v_cache, 
     HB_REQUIRE((cos_t == nullptr) == (sin_t == nullptr), "attn_decode: cos and sin tables come together");
 #define DECODE_ARGS(QPTR) QPTR, (bf16*)k_cache, (bf16*)v_cache, partial_o, partial_ml, context_lens, slots, \
                           page_table, max_pages, nq, nkv, c, window, pages_per_split, fu, direct, ranges, B, \
-                          direct ? sinks : nullptr, chunk, softcap / scale
-#define LAUNCH_DECODE(HDV) do {                                                                          \
+                          direct ? sinks : nullptr, chunk, softcap / scale, ext
+#define LAUNCH_DECODE_FORM(HDV, FORM) do {                                                               \
     if (qkv)                                                                                             \
-        attn_decode_kernel<HDV, true><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr));                    \
+        attn_decode_kernel<HDV, true, FORM><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr));              \
     else                                                                                                 \
-        attn_decode_kernel<HDV, false><<<grid, 64, 0, stream>>>(DECODE_ARGS((const bf16*)q));            \
+        attn_decode_kernel<HDV, false, FORM><<<grid, 64, 0, stream>>>(DECODE_ARGS((const bf16*)q));      \
     } while (0)
-    if (qkv_slices == 2) attn_decode_kernel<128, true, 2><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr));
-    else if (qkv_slices == 4) attn_decode_kernel<128, true, 4><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr));
-    else if (qkv_slices == 8) attn_decode_kernel<128, true, 8><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr));
+#define LAUNCH_DECODE(HDV) do { if (extended) LAUNCH_DECODE_FORM(HDV, true); else LAUNCH_DECODE_FORM(HDV, false); } while (0)
+#define LAUNCH_SLICES(QSV) do {                                                                          \
+    if (extended) attn_decode_kernel<128, true, true, QSV><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr)); \
+    else attn_decode_kernel<128, true, false, QSV><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr));       \
+    } while (0)
+    if (qkv_slices == 2) LAUNCH_SLICES(2);
+    else if (qkv_slices == 4) LAUNCH_SLICES(4);
+    else if (qkv_slices == 8) LAUNCH_SLICES(8);
     else
     if (hd == 32) LAUNCH_DECODE(32);
     else if (hd == 64) LAUNCH_DECODE(64);
     else if (hd == 128) LAUNCH_DECODE(128);
     else HB_REQUIRE(false, "attn_decode: head_dim %d is not one of 32, 64, 128", hd);
 #undef LAUNCH_DECODE
+#undef LAUNCH_DECODE_FORM
+#undef LAUNCH_SLICES
 #undef DECODE_ARGS
     HB_CHECK_LAUNCH("attn_decode");
     if (!direct) {

@@ -17,12 +17,12 @@
 HB_MODULE_ERROR_SLOT()
 
 // ---------------------------------------------------------------- embedding
-// x[t, :] = float(table[ids[t], :]); the residual stream is float32.
+// x[t, :] = float(table[ids[t], :]) * mult; the residual stream is float32.
 // PACKED: the table is stored in the MFMA kernels' order [H / 32][V / 16][64 lanes][8], element
 // (n, k) at ((k / 32 * (V / 16) + n / 16) * 64 + (k / 8 % 4) * 16 + n % 16) * 8 + k % 8.
 template <class TW, bool PACKED>
 __global__ void embed_kernel(const int* __restrict__ ids, const TW* __restrict__ table,
-                             float* __restrict__ x, int H, int V) {
+                             float* __restrict__ x, int H, int V, float mult) {
     const int t = blockIdx.x;
     const int n = ids[t];
     float* out = x + (size_t)t * H;
@@ -36,7 +36,7 @@ __global__ void embed_kernel(const int* __restrict__ ids, const TW* __restrict__
         const TW* blk = table + (size_t)(n / 16) * 512 + (n % 16) * 8;
         const size_t plane = (size_t)(V / 16) * 512;
         for (int k = threadIdx.x; k < H; k += blockDim.x)
-            out[k] = hb_to_float(blk[(size_t)(k / 32) * plane + ((k / 8) % 4) * 128 + (k % 8)]);
+            out[k] = hb_to_float(blk[(size_t)(k / 32) * plane + ((k / 8) % 4) * 128 + (k % 8)]) * mult;
     } else {
         const TW* row = table + (size_t)n * H;
         if (sizeof(TW) == 2 && H % 8 == 0) {
@@ -47,29 +47,29 @@ __global__ void embed_kernel(const int* __restrict__ ids, const TW* __restrict__
                 float v[8];
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
-                    v[2 * e] = __uint_as_float(w[e] << 16);
-                    v[2 * e + 1] = __uint_as_float(w[e] & 0xffff0000u);
+                    v[2 * e] = __uint_as_float(w[e] << 16) * mult;
+                    v[2 * e + 1] = __uint_as_float(w[e] & 0xffff0000u) * mult;
                 }
                 *(float4*)(out + i) = float4{v[0], v[1], v[2], v[3]};
                 *(float4*)(out + i + 4) = float4{v[4], v[5], v[6], v[7]};
             }
             return;
         }
-        for (int i = threadIdx.x; i < H; i += blockDim.x) out[i] = hb_to_float(row[i]);
+        for (int i = threadIdx.x; i < H; i += blockDim.x) out[i] = hb_to_float(row[i]) * mult;
     }
 }
 
 extern "C" int hb_embed(const int* ids, const void* table, int table_dtype, float* x, int T, int H, int V,
-                        int packed, hipStream_t stream) {
+                        int packed, float mult, hipStream_t stream) {
     HB_REQUIRE(T > 0 && H > 0, "embed: empty input (T=%d, H=%d)", T, H);
     HB_REQUIRE(!packed || (table_dtype == HB_BF16 && H % 32 == 0 && V % 16 == 0),
                "embed: a packed table is bfloat16 with a width in steps of 32 and rows in steps of 16");
     if (table_dtype == HB_F32)
-        embed_kernel<float, false><<<T, 256, 0, stream>>>(ids, (const float*)table, x, H, V);
+        embed_kernel<float, false><<<T, 256, 0, stream>>>(ids, (const float*)table, x, H, V, mult);
     else if (table_dtype == HB_BF16 && packed)
-        embed_kernel<bf16, true><<<T, 256, 0, stream>>>(ids, (const bf16*)table, x, H, V);
+        embed_kernel<bf16, true><<<T, 256, 0, stream>>>(ids, (const bf16*)table, x, H, V, mult);
     else if (table_dtype == HB_BF16)
-        embed_kernel<bf16, false><<<T, 256, 0, stream>>>(ids, (const bf16*)table, x, H, V);
+        embed_kernel<bf16, false><<<T, 256, 0, stream>>>(ids, (const bf16*)table, x, H, V, mult);
     else
         HB_REQUIRE(false, "embed: unknown table dtype %d", table_dtype);
     HB_CHECK_LAUNCH("embed");
@@ -431,9 +431,10 @@ extern "C" int hb_qk_norm_rope_write(const float* qkv, int ld_qkv, const float* 
 
 // ------------------------------------------------------------------- gated linear units
 // act[t, i] = f(gu[t, i]) * gu[t, I + i] with f = silu, g / (1 + exp(-g)), or the tanh form of gelu,
-// 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))).
+// 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))), or relu, max(g, 0).
 #define HB_ACT_SILU 0
 #define HB_ACT_GELU_TANH 1
+#define HB_ACT_RELU 2
 __device__ __forceinline__ float hb_gelu_tanh(float z) {
     return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
@@ -446,21 +447,24 @@ __global__ void swiglu_kernel(const float* __restrict__ gu, TOut* __restrict__ a
     const int i = (int)(idx - t * I);
     const float g = gu[t * 2 * I + i];
     const float u = gu[t * 2 * I + I + i];
-    const float f = ACT == HB_ACT_GELU_TANH ? hb_gelu_tanh(g) : g / (1.0f + expf(-g));
+    const float f = ACT == HB_ACT_GELU_TANH ? hb_gelu_tanh(g) : ACT == HB_ACT_RELU ? fmaxf(g, 0.f) : g / (1.0f + expf(-g));
     act[idx] = hb_from_float<TOut>(f * u);
 }
 
 extern "C" int hb_swiglu(const float* gu, void* act, int act_dtype, int T, int I, int activation, hipStream_t stream) {
     HB_REQUIRE(T > 0 && I > 0, "swiglu: empty input");
-    HB_REQUIRE(activation == HB_ACT_SILU || activation == HB_ACT_GELU_TANH, "swiglu: unknown activation %d", activation);
+    HB_REQUIRE(activation == HB_ACT_SILU || activation == HB_ACT_GELU_TANH || activation == HB_ACT_RELU,
+               "swiglu: unknown activation %d", activation);
     HB_REQUIRE(act_dtype == HB_F32 || act_dtype == HB_BF16, "swiglu: unknown output dtype %d", act_dtype);
     const size_t total = (size_t)T * I;
     const unsigned blocks = (unsigned)((total + 255) / 256);
     if (act_dtype == HB_F32) {
         if (activation == HB_ACT_SILU) swiglu_kernel<float, HB_ACT_SILU><<<blocks, 256, 0, stream>>>(gu, (float*)act, I, total);
+        else if (activation == HB_ACT_RELU) swiglu_kernel<float, HB_ACT_RELU><<<blocks, 256, 0, stream>>>(gu, (float*)act, I, total);
         else swiglu_kernel<float, HB_ACT_GELU_TANH><<<blocks, 256, 0, stream>>>(gu, (float*)act, I, total);
     } else {
         if (activation == HB_ACT_SILU) swiglu_kernel<bf16, HB_ACT_SILU><<<blocks, 256, 0, stream>>>(gu, (bf16*)act, I, total);
+        else if (activation == HB_ACT_RELU) swiglu_kernel<bf16, HB_ACT_RELU><<<blocks, 256, 0, stream>>>(gu, (bf16*)act, I, total);
         else swiglu_kernel<bf16, HB_ACT_GELU_TANH><<<blocks, 256, 0, stream>>>(gu, (bf16*)act, I, total);
     }
     HB_CHECK_LAUNCH("swiglu");
@@ -553,6 +557,100 @@ extern "C" int hb_scale(float* x, float s, size_t n, hipStream_t stream) {
     const size_t blocks = (n + 255) / 256;
     scale_kernel<<<(unsigned)(blocks > 4096 ? 4096 : blocks), 256, 0, stream>>>(x, s, n);
     HB_CHECK_LAUNCH("scale");
+    return 0;
+}
+
+// ------------------------------------------- dynamic tanh, and the sums that join the stream between two of them
+// A norm without mean and variance, n(v) = tanh(alpha v) w + b. What stands between two products of a layer that
+// norms before and after each of its parts is one pass over the rows, since nothing here needs a whole row:
+//   s = x[r] + n_after(part[r]) + extra[r] + step;   x_out[r] = s;   y[r] = n_before(s)
+// part (a part's output), extra (rows of their own), step (one vector for all rows), x_out and y are each there or
+// not; r = rows ? rows[i] : i picks the rows of x (with rows: only x and y). Everything float32 but y's storage.
+struct DynTanh {
+    const float* w;      // null: there is no such norm
+    const float* b;
+    float alpha;
+};
+
+template <class TOut, bool QUADS>
+__global__ void __launch_bounds__(256)
+tanh_join_kernel(const float* x, const float* __restrict__ part, DynTanh after, const float* __restrict__ extra,
+                 const float* __restrict__ step, float* x_out, DynTanh before, TOut* __restrict__ y,
+                 const int* __restrict__ rows, int H, unsigned total) {
+    const unsigned idx = blockIdx.x * 256u + threadIdx.x;       // a quad of four neighbours, or one number
+    if (idx >= total) return;
+    constexpr int N = QUADS ? 4 : 1;
+    const unsigned per = QUADS ? H / 4 : H;
+    const unsigned i = idx / per, c = (idx - i * per) * N;
+    const size_t from = (size_t)(rows ? rows[i] : i) * H + c, at = (size_t)i * H + c;
+    auto load = [&](const float* p) {
+        hb_f4 v = {0.f, 0.f, 0.f, 0.f};
+        if (QUADS) v = *(const hb_f4*)p;
+        else v[0] = *p;
+        return v;
+    };
+    hb_f4 s = load(x + from);
+    if (part) {
+        const hb_f4 p = load(part + at), w = load(after.w + c), b = load(after.b + c);
+#pragma unroll
+        for (int e = 0; e < N; ++e) s[e] += tanhf(after.alpha * p[e]) * w[e] + b[e];
+    }
+    if (extra) s += load(extra + at);
+    if (step) s += load(step + c);
+    if (x_out) {
+        if (QUADS) *(hb_f4*)(x_out + at) = s;
+        else x_out[at] = s[0];
+    }
+    if (y) {
+        const hb_f4 w = load(before.w + c), b = load(before.b + c);
+#pragma unroll
+        for (int e = 0; e < N; ++e) s[e] = tanhf(before.alpha * s[e]) * w[e] + b[e];
+        if (QUADS) store_four(y + at, s);
+        else y[at] = hb_from_float<TOut>(s[0]);
+    }
+}
+
+extern "C" int hb_tanh_join(const float* x, const float* part, float alpha_after, const float* w_after,
+                            const float* b_after, const float* extra, const float* step, float* x_out,
+                            float alpha_before, const float* w_before, const float* b_before, void* y, int y_dtype,
+                            const int* rows, int R, int H, hipStream_t stream) {
+    HB_REQUIRE(R > 0 && H > 0, "tanh norm: empty input (R=%d, H=%d)", R, H);
+    HB_REQUIRE(x && (x_out || y), "tanh norm: nothing to do");
+    HB_REQUIRE(!part || (w_after && b_after), "tanh norm: a part's output without the norm that it passes");
+    HB_REQUIRE(!y || (w_before && b_before), "tanh norm: rows to write without their norm");
+    HB_REQUIRE(!rows || (!part && !extra && !step && !x_out), "tanh norm: rows are not gathered while a sum is added");
+    HB_REQUIRE(y_dtype == HB_F32 || y_dtype == HB_BF16, "tanh norm: unknown output dtype %d", y_dtype);
+    const uintptr_t all = (uintptr_t)x | (uintptr_t)part | (uintptr_t)w_after | (uintptr_t)b_after | (uintptr_t)extra |
+                          (uintptr_t)step | (uintptr_t)x_out | (uintptr_t)w_before | (uintptr_t)b_before | (uintptr_t)y;
+    const bool quads = H % 4 == 0 && all % 16 == 0;
+    const size_t total = (size_t)R * H / (quads ? 4 : 1);
+    HB_REQUIRE(total < (1ull << 31), "tanh norm: too many rows");
+    const unsigned blocks = (unsigned)((total + 255) / 256);
+    const DynTanh after = {w_after, b_after, alpha_after}, before = {w_before, b_before, alpha_before};
+#define HB_TANH_JOIN(T, Q) tanh_join_kernel<T, Q><<<blocks, 256, 0, stream>>>(x, part, after, extra, step, x_out, before, (T*)y, rows, H, (unsigned)total)
+    if (y_dtype == HB_F32) {
+        if (quads) HB_TANH_JOIN(float, true);
+        else HB_TANH_JOIN(float, false);
+    } else {
+        if (quads) HB_TANH_JOIN(bf16, true);
+        else HB_TANH_JOIN(bf16, false);
+    }
+#undef HB_TANH_JOIN
+    HB_CHECK_LAUNCH("tanh_join");
+    return 0;
+}
+
+// ---------------------------------------------------------------- x = cap tanh(x / cap) (float32, in place)
+__global__ void softcap_kernel(float* x, float cap, size_t n) {
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x)
+        x[i] = cap * tanhf(x[i] / cap);
+}
+
+extern "C" int hb_softcap(float* x, float cap, size_t n, hipStream_t stream) {
+    HB_REQUIRE(n > 0 && cap > 0.f, "softcap: empty input, or a cap that is not positive");
+    const size_t blocks = (n + 255) / 256;
+    softcap_kernel<<<(unsigned)(blocks > 4096 ? 4096 : blocks), 256, 0, stream>>>(x, cap, n);
+    HB_CHECK_LAUNCH("softcap");
     return 0;
 }
 

@@ -6,6 +6,8 @@ The forward pass follows the reference's drivers
 run the schedule's entries in order on the packed rows, then the final norm
 and the head on the wanted rows only.
 """
+import torch
+
 from ..errors import ConfigError
 from ..kernels import ops
 from ..parts import StepContext, build
@@ -51,6 +53,11 @@ class Model:
                 if not 0 <= e.cache < i or self.schedule[e.cache].cache is not None:
                     raise ConfigError(f"schedule entry {i} must read the cache of an earlier entry "
                                       "that owns one")
+        self.pass_input = None
+        if any(e.starts_pass is not None for e in self.schedule):
+            if spec.pass_input is None:
+                raise ConfigError("the schedule names passes, but the model says nothing of what joins the stream there")
+            self.pass_input = build("pass_input", spec.pass_input)
         self.loaded = False
 
     # ---- weights
@@ -65,6 +72,8 @@ class Model:
 
     def _weight_parts(self):
         parts = [self.embedding, self.head]
+        if self.pass_input is not None:
+            parts.append(self.pass_input)
         for b in self.blocks:
             parts.extend(b.parts())
         return parts
@@ -76,6 +85,8 @@ class Model:
         for b in self.blocks:
             for p in b.parts():
                 p.load(tensors, rt)
+        if self.pass_input is not None:
+            self.pass_input.load(tensors, rt)
         self.head.load(tensors, rt, embedding=self.embedding)
         self.loaded = True
 
@@ -106,14 +117,27 @@ class Model:
     def _forward(self, rt, meta, cache, logits_out=None):
         ctx = StepContext(rt=rt, meta=meta, cache=cache, logits_out=logits_out)
         x = self.embedding.forward(ctx, meta.token_ids)
+        embedded = None
+        if self.pass_input is not None and self.pass_input.reads_embedding:
+            embedded = rt.buffer("embedding_output", tuple(x.shape), torch.float32)
+            ops.tanh_join(x, x_out=embedded)         # (a copy)
         for i, e in enumerate(self.schedule):
+            if e.starts_pass is not None:
+                joins = self.pass_input.rows(e.starts_pass, embedded)
+                if getattr(self.blocks[e.layer], "takes_pass_input", False):
+                    ctx.pass_input = joins
+                else:
+                    ops.tanh_join(x, extra=joins[0], step=joins[1], x_out=x)
             ctx.entry = i
             ctx.cache_entry = i if e.cache is None else e.cache
             ctx.owns_cache = e.cache is None
             # the norm that the residual stream meets after this block, for parts that can prepare it
             ctx.norm_after_block = None
             ctx.next_block = self.blocks[self.schedule[i + 1].layer] if i + 1 < len(self.schedule) else None
-            if i + 1 < len(self.schedule):
+            if ctx.next_block is not None and self.schedule[i + 1].starts_pass is not None \
+                    and not getattr(ctx.next_block, "takes_pass_input", False):
+                ctx.next_block = None       # x changes before that block: nothing of its first norm may be prepared
+            if ctx.next_block is not None:
                 first_norm = getattr(self.blocks[self.schedule[i + 1].layer], "first_norm", None)
                 if first_norm is not None:
                     ctx.norm_after_block = (first_norm(), i + 1)

@@ -20,7 +20,9 @@ _SZ = ctypes.c_size_t
 # module -> function -> argument types (every function returns int, 0 = ok)
 SIGNATURES = {
     "elementwise": {
-        "hb_embed": [_P, _P, _I, _P, _I, _I, _I, _I, _P],
+        "hb_embed": [_P, _P, _I, _P, _I, _I, _I, _I, _F, _P],
+        "hb_tanh_join": [_P, _P, _F, _P, _P, _P, _P, _P, _F, _P, _P, _P, _I, _P, _I, _I, _P],
+        "hb_softcap": [_P, _F, _SZ, _P],
         "hb_rmsnorm": [_P, _P, _P, _I, _P, _I, _I, _F, _P],
         "hb_qk_norm_rope_write": [_P, _I, _P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _P, _P, _P, _I,
                                   _I, _I, _I, _I, _F, _I, _I, ctypes.c_size_t, _F, _I, _P],
@@ -55,9 +57,10 @@ SIGNATURES = {
         "hb_channel_decay": [_P, _I, _P, _P, _P, _I, _I, _I, _P],
     },
     "attention_latent": {
-        "hb_latent_write": [_P, _I, _P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P],
-        "hb_latent_attention_mfma": [_P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P],
-        "hb_latent_attention_plain": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _P],
+        "hb_latent_write": [_P, _I, _P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _I,
+                            _P, _P, _P],
+        "hb_latent_attention_mfma": [_P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P, _P],
+        "hb_latent_attention_plain": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _P, _P],
     },
     "moe": {
         "hb_moe_route": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P],
@@ -67,7 +70,8 @@ SIGNATURES = {
         "hb_grouped_mfma": [_P, _I, _SZ, _P, _I, _I, _P, _I, _SZ, _I, _P, _I, _P, _P, _P, _I, _I, _I, _F, _F, _F, _I, _P],
     },
     "attention_plain": {
-        "hb_attention_plain": [_P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _P, _I, _F, _P],
+        "hb_attention_plain": [_P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _P, _I, _F, _P, _I, _I, _I, _I,
+                               _P],
     },
     "sampling": {
         "hb_argmax": [_P, _I, _I, _I, _P, _P, _P, _I, _P],

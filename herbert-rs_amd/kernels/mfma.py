@@ -387,9 +387,9 @@ def gemm_swiglu(a, w_interleaved, out, packed=False, norm=None, tile=0, row_scal
 
 
 lib.register_signatures("attention_mfma", {
-    "hb_attn_prefill_mfma": [_P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I, _P, _I, _F, _P],
+    "hb_attn_prefill_mfma": [_P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I, _P, _I, _F, _P, _I, _I, _I, _P],
     "hb_attn_decode_mfma": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I,
-                            _P, _P, _P, _P, _P, _F, _I, _I, ctypes.c_size_t, _P, _F, _I, _P, _I, _F, _P],
+                            _P, _P, _P, _P, _P, _F, _I, _I, ctypes.c_size_t, _P, _F, _I, _P, _I, _F, _P, _I, _I, _I, _P],
 })
 
 ATTENTION_HEAD_DIMS = (32, 64, 128)
@@ -451,10 +451,19 @@ def _prefill_tiles(meta, height=QUERY_TILE):
     return tiles
 
 
+def _extras_args(bias, keep_first, nq):
+    """The C arguments of a bias by distance (an ops.DistanceBias whose values are divided by the score's scale: the
+    kernels add it to the raw dot products) and of a window's kept first keys."""
+    if bias is None:
+        return None, 0, 0, int(keep_first or 0)
+    bias.check(nq)
+    return bias.rows.data_ptr(), bias.length, bias.rows.shape[1], int(keep_first or 0)
+
+
 DECODE_WAVES = 1024       # waves of the decode kernel that the 256 CUs hold at a time
 
 
-def _decode_split(meta, nkv, window, chunk=0):
+def _decode_split(meta, nkv, window, chunk=0, keep_first=0):
     """(ranges, pages per range): as many ranges as still give no more waves than the GPU holds at
     a time, every range at least one page. With one range the kernel writes the output itself and
     no merge runs. (Measured at 4 K tokens a sequence: what costs is a second, partly filled round
@@ -462,7 +471,8 @@ def _decode_split(meta, nkv, window, chunk=0):
     10.6 ms. 40 sequences: 3 ranges, 960 waves, 8.9 ms; 4 ranges, 1280 waves, 10.0 ms.)"""
     span = (meta.context_bucket + 63) // 64     # by bucket, so that a captured graph's grid stays right
     if window or chunk:
-        span = min(span, ((window or chunk) + 63) // 64 + 1)     # a chunk's keys lie on as many pages as a window's
+        # a chunk's keys lie on as many pages as a window's; kept first keys on pages of their own before them
+        span = min(span, ((window or chunk) + 63) // 64 + 1 + (keep_first + 63) // 64)
     pairs = meta.num_seqs * nkv
     if 2 * pairs >= DECODE_WAVES:
         # (how evenly the waves sit is a matter of the sequences themselves: padding rows' waves end at once)
@@ -536,15 +546,18 @@ def decode_fusable(meta, kv, nq, nkv, hd, rot_dims, dtype):
 
 
 def attention_decode_fused(qkv, q_norm_w, k_norm_w, cos, sin, meta, kv, out, nq, nkv, hd, eps, scale, window,
-                           qkv_slices=None, scratch=None, q_temp=None):
+                           qkv_slices=None, scratch=None, q_temp=None, sinks=None, bias=None, keep_first=0):
     """One token a sequence: per-head norm (if weights are given), rotation (if tables are given),
     the new key and value written to the pages, and attention over them, in one kernel (+ merge).
     qkv f32 [B, (nq + 2 nkv) hd]; cos / sin f32 [max_pos, hd / 2]; out bf16 [B, nq hd].
     qkv_slices = (slices, pointer, floats between two), as gemm(..., defer_slices=True) returns it:
     the projection's sums are still in that many slices, which the kernel adds up as it loads them
     (qkv itself is then not read). q_temp = (coef, every): a query at position p is multiplied by
-    1 + coef ln(floor((p + 1) / every) + 1) after its norm."""
+    1 + coef ln(floor((p + 1) / every) + 1) after its norm. sinks, bias, keep_first: as for `attention`."""
     B = meta.num_seqs
+    extras = _extras_args(bias, keep_first, nq)
+    if sinks is not None:
+        _check(sinks, "sinks", torch.float32, (nq,))
     coef, every = ops.query_temperature_args(q_temp)
     _check(qkv, "qkv", torch.float32, (B, (nq + 2 * nkv) * hd))
     _check(out, "out", torch.bfloat16, (B, nq * hd))
@@ -572,7 +585,7 @@ def attention_decode_fused(qkv, q_norm_w, k_norm_w, cos, sin, meta, kv, out, nq,
         (splits, ranges), per = listed, 1
         po, pml = _partial_buffers(scratch, qkv.device, nq, splits, hd)
     else:
-        (splits, per), ranges = _decode_split(meta, nkv, window), None
+        (splits, per), ranges = _decode_split(meta, nkv, window, 0, extras[3]), None
         po, pml = _partial_buffers(scratch, qkv.device, B * nq, splits, hd)
     n_slices, src, stride = qkv_slices if qkv_slices is not None else (1, qkv.data_ptr(), 0)
     if n_slices > 1 and (n_slices not in DEFERRED_SLICES or hd != 128 or stride < qkv.numel()):
@@ -583,21 +596,25 @@ def attention_decode_fused(qkv, q_norm_w, k_norm_w, cos, sin, meta, kv, out, nq,
              window, splits, per, src, None if q_norm_w is None else q_norm_w.data_ptr(),
              None if k_norm_w is None else k_norm_w.data_ptr(), None if cos is None else cos.data_ptr(),
              None if sin is None else sin.data_ptr(), float(eps), 1, n_slices, stride,
-             None if ranges is None else ranges.data_ptr(), coef, every, None, 0, 0.0, _stream())
+             None if ranges is None else ranges.data_ptr(), coef, every, None if sinks is None else sinks.data_ptr(), 0, 0.0,
+             *extras, _stream())
 
 
 DEFERRED_SLICES = (2, 4, 8)     # numbers of slices of the projection that the decode kernel adds up itself
 
 
 def attention(q, meta, kv, out, nq, nkv, hd, scale, window, tile_height=None, scratch=None, sinks=None, chunk=None,
-              softcap=None):
+              softcap=None, bias=None, keep_first=0):
     """Causal (and windowed) attention of the step's tokens over their slots' pages.
     sinks f32 [nq]: the softmax's denominator of head h also holds exp(sinks[h]), once, without key or value.
     chunk: a query sees the keys of its own chunk of that many positions only, the chunks counted from the
     sequence's start (not together with a window). softcap: a scaled score s becomes softcap tanh(s / softcap).
+    bias: an ops.DistanceBias added to the raw dot products (its values divided by the scale); keep_first (with a
+    window): the sequence's first so many keys are seen as well; neither goes with chunk or softcap.
     One token a sequence: the split decode kernel; otherwise one of the two tiled prompt kernels
     (tile_height 32 or 64 asks for one by name; None: the host's choice, see _prefill_tile_height)."""
     T = q.shape[0]
+    extras = _extras_args(bias, keep_first, nq)
     _check(q, "q", torch.bfloat16, (T, nq * hd))
     _check(out, "out", torch.bfloat16, (T, nq * hd))
     pages = kv.k.shape[0]
@@ -620,13 +637,13 @@ def attention(q, meta, kv, out, nq, nkv, hd, scale, window, tile_height=None, sc
             (splits, ranges), per = listed, 1
             po, pml = _partial_buffers(scratch, q.device, nq, splits, hd)
         else:
-            (splits, per), ranges = _decode_split(meta, nkv, window, chunk), None
+            (splits, per), ranges = _decode_split(meta, nkv, window, chunk, extras[3]), None
             po, pml = _partial_buffers(scratch, q.device, T * nq, splits, hd)
         lib.call("attention_mfma", "hb_attn_decode_mfma", q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(),
                  out.data_ptr(), po.data_ptr(), pml.data_ptr(), meta.context_lens.data_ptr(),
                  meta.slots.data_ptr(), kv.page_table.data_ptr(), kv.page_table.shape[1], kv.page_size,
                  T, nq, nkv, hd, float(scale), window, splits, per, None, None, None, None, None, 0.0, 0, 1, 0,
-                 None if ranges is None else ranges.data_ptr(), 0.0, 0, sinks_ptr, chunk, softcap, _stream())
+                 None if ranges is None else ranges.data_ptr(), 0.0, 0, sinks_ptr, chunk, softcap, *extras, _stream())
         return
     _check(meta.positions, "positions", torch.int32, (T,))
     height = tile_height or _prefill_tile_height(meta, nkv, nq // nkv)
@@ -637,4 +654,4 @@ def attention(q, meta, kv, out, nq, nkv, hd, scale, window, tile_height=None, sc
              out.data_ptr(), tile_seq.data_ptr(), tile_row0.data_ptr(), tile_rows.data_ptr(), n_tiles,
              meta.positions.data_ptr(), meta.slots.data_ptr(), kv.page_table.data_ptr(),
              kv.page_table.shape[1], kv.page_size, nq, nkv, hd, float(scale), window, height, sinks_ptr, chunk, softcap,
-             _stream())
+             *extras, _stream())

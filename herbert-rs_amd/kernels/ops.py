@@ -76,8 +76,8 @@ def _ptr(t):
     return None if t is None else t.data_ptr()
 
 
-def embed(ids, table, out, packed=False):
-    """out[t, :] = table[ids[t], :] as float32. ids int32 [T], table [V, H], out f32 [T, H].
+def embed(ids, table, out, packed=False, scale=1.0):
+    """out[t, :] = table[ids[t], :] * scale as float32. ids int32 [T], table [V, H], out f32 [T, H].
     packed: the table is stored in the MFMA kernels' order ([H / 32, V / 16, 64, 8])."""
     T = ids.shape[0]
     _check(ids, "ids", torch.int32, (T,))
@@ -85,7 +85,7 @@ def embed(ids, table, out, packed=False):
     H = table.shape[1]
     _check(out, "out", torch.float32, (T, H))
     lib.call("elementwise", "hb_embed", ids.data_ptr(), table.data_ptr(), dtype_code(table),
-             out.data_ptr(), T, H, table.shape[0], 1 if packed else 0, _stream())
+             out.data_ptr(), T, H, table.shape[0], 1 if packed else 0, float(scale), _stream())
 
 
 def rmsnorm(x, weight, out, eps, rows=None):
@@ -187,11 +187,33 @@ def qk_norm_rope_write(qkv, q_norm_w, k_norm_w, cos, sin, rot_dims, meta, cache,
              n_slices, stride, coef, every, _stream())
 
 
-def attention_plain(q, meta, cache, out, nq, nkv, hd, scale, window, sinks=None, chunk=None, softcap=None):
+class DistanceBias:
+    """A bias by distance as the attention kernels read it: rows f32 [heads, ld] with a head's values along the keys,
+    rows[h, at + length - 1 - n] for the distance n = i - j, and the value of n = length - 1 for every n beyond it
+    (FRONT of those once more before `at`, BACK unused ones behind n = 0)."""
+    FRONT, BACK = 8, 64
+
+    def __init__(self, by_distance):
+        """by_distance f32 [length, heads] on the GPU: the biases of the distances 0 .. length - 1."""
+        self.length, heads = by_distance.shape
+        rows = torch.zeros((heads, self.FRONT + self.length + self.BACK), dtype=torch.float32, device=by_distance.device)
+        rows[:, :self.FRONT] = by_distance[-1][:, None]
+        rows[:, self.FRONT:self.FRONT + self.length] = by_distance.flip(0).t()
+        self.rows, self.at = rows.contiguous(), self.FRONT
+
+    def check(self, heads):
+        _check(self.rows, "distance bias", torch.float32, (heads, self.FRONT + self.length + self.BACK))
+
+
+def attention_plain(q, meta, cache, out, nq, nkv, hd, scale, window, sinks=None, chunk=None, softcap=None, bias=None,
+                    keep_first=0):
     """Causal (and windowed) attention of every token over its slot's pages. sinks f32 [nq]: the softmax's
     denominator of head h also holds exp(sinks[h]). chunk: a query sees the keys of its own chunk of that many
     positions only (counted from the sequence's start; not together with a window). softcap: a scaled score s
-    becomes softcap tanh(s / softcap)."""
+    becomes softcap tanh(s / softcap). bias: a DistanceBias, added to the scaled scores. keep_first (with a window):
+    the sequence's first so many keys are seen as well."""
+    if bias is not None:
+        bias.check(nq)
     T = q.shape[0]
     if sinks is not None:
         _check(sinks, "sinks", torch.float32, (nq,))
@@ -204,14 +226,16 @@ def attention_plain(q, meta, cache, out, nq, nkv, hd, scale, window, sinks=None,
              cache.v.data_ptr(), out.data_ptr(), dtype_code(q), meta.positions.data_ptr(),
              meta.seq_of.data_ptr(), meta.slots.data_ptr(), cache.page_table.data_ptr(),
              cache.page_table.shape[1], cache.page_size, T, nq, nkv, hd, float(scale),
-             int(window or 0), _ptr(sinks), int(chunk or 0), float(softcap or 0.0), _stream())
+             int(window or 0), _ptr(sinks), int(chunk or 0), float(softcap or 0.0),
+             None if bias is None else bias.rows.data_ptr(), 0 if bias is None else bias.rows.shape[1],
+             0 if bias is None else bias.at, 0 if bias is None else bias.length, int(keep_first or 0), _stream())
 
 
-GLU_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+GLU_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "relu": 2}
 
 
 def swiglu(gu, out, activation="silu"):
-    """out[t, i] = f(gu[t, i]) * gu[t, I + i]; gu f32 [T, 2I]; f "silu" or "gelu_tanh"."""
+    """out[t, i] = f(gu[t, i]) * gu[t, I + i]; gu f32 [T, 2I]; f "silu", "gelu_tanh" or "relu"."""
     if activation not in GLU_ACTIVATIONS:
         raise BackendError(f"gated linear unit: unknown activation {activation!r}")
     _check(gu, "gate_up", torch.float32, (None, None))
@@ -403,6 +427,50 @@ def scale(x, factor):
     """x *= factor in place; x float32."""
     _check(x, "x", torch.float32)
     lib.call("elementwise", "hb_scale", x.data_ptr(), float(factor), x.numel(), _stream())
+
+
+def softcap(x, cap):
+    """x = cap tanh(x / cap) in place; x float32."""
+    _check(x, "x", torch.float32)
+    if not cap > 0:
+        raise BackendError("softcap: the cap must be positive")
+    lib.call("elementwise", "hb_softcap", x.data_ptr(), float(cap), x.numel(), _stream())
+
+
+def tanh_join(x, part=None, after=None, extra=None, step=None, x_out=None, before=None, y=None, rows=None):
+    """s = x + n_after(part) + extra + step, row by row; x_out = s (x itself, or other rows); y = n_before(s), with
+    n(v) = tanh(alpha v) w + b and after, before = (alpha, w f32 [H], b f32 [H]). x, part, extra, x_out f32 [T, H],
+    step f32 [H], y [R, H] in any storage type; each of part, extra, step, x_out, y may be None. rows int32 [R]
+    (y only, no sums): the rows of x that are normed."""
+    _check(x, "x", torch.float32, (None, None))
+    T, H = x.shape
+    R = T
+    if rows is not None:
+        _check(rows, "rows", torch.int32, (None,))
+        R = rows.shape[0]
+        if part is not None or extra is not None or step is not None or x_out is not None:
+            raise BackendError("tanh norm: rows are not gathered while a sum is added")
+    for t, name in ((part, "part"), (extra, "extra"), (x_out, "x_out")):
+        if t is not None:
+            _check(t, name, torch.float32, (T, H))
+    if step is not None:
+        _check(step, "step", torch.float32, (H,))
+    if (part is None) != (after is None) or (y is None) != (before is None):
+        raise BackendError("tanh norm: a part's output and the rows to write come with their norms")
+    if x_out is None and y is None:
+        raise BackendError("tanh norm: nothing to do")
+    alpha_a, w_a, b_a = after if after is not None else (0.0, None, None)
+    alpha_b, w_b, b_b = before if before is not None else (0.0, None, None)
+    for t, name in ((w_a, "weight after"), (b_a, "bias after"), (w_b, "weight before"), (b_b, "bias before")):
+        if t is not None:
+            _check(t, name, torch.float32, (H,))
+    if y is not None:
+        _check(y, "y", None, (R, H))
+        if y.data_ptr() in (x.data_ptr(), None if part is None else part.data_ptr()):
+            raise BackendError("tanh norm: the normed rows must be other rows than the sum's")
+    lib.call("elementwise", "hb_tanh_join", x.data_ptr(), _ptr(part), float(alpha_a), _ptr(w_a), _ptr(b_a), _ptr(extra),
+             _ptr(step), _ptr(x_out), float(alpha_b), _ptr(w_b), _ptr(b_b), _ptr(y),
+             dtype_code(y) if y is not None else F32, _ptr(rows), R, H, _stream())
 
 
 def gemm_plain_batched(a, w, c, M, N, K, lda, ldw, ldc, batch, batch_a, batch_w, batch_c):

@@ -27,6 +27,11 @@ the keys of its own chunk of that many positions only, the chunks counted from t
 (over the whole projection, or head by head with weights that all heads share), rotates and writes the cache in
 one kernel of its own; rotation and values of another size than the keys go together there.
 
+Three further options go with either form (not in the reference): `keep_first` (with a window: the sequence's first
+so many keys are seen as well; the cache keeps their pages), `distance_bias=(bias_max,)` (a learned bias by the
+distance of query and key, a table [rows, heads] whose rows the stored tensor counts, is added to the scaled
+score; see position.distance_bucket), `sink="unit"` (the softmax's denominator also holds 1).
+
 The kernels keep one head size for queries, keys and values. Where a model's
 key and value sizes differ, or where the matrix cores (heads of 32, 64, 128)
 would otherwise refuse a head, the part runs them at a larger size whose
@@ -44,6 +49,7 @@ from ..kernels import mfma, ops, recurrent
 from ..weights import TensorNeed
 from .base import Part
 from .linear import Linear
+from .position import bias_by_distance
 from .registry import register
 
 
@@ -62,6 +68,15 @@ def _sink_init(shape, gen, device, std, norm_std):
     return torch.randn(shape, generator=gen, device=device, dtype=torch.float32)
 
 
+RANDOM_BIAS_ROWS = 32
+
+
+def _distance_init(shape, gen, device, std, norm_std):
+    """Biases by distance of a random model: as large as its scores, so that a wrong row shows."""
+    return torch.randn((RANDOM_BIAS_ROWS if shape[0] is None else shape[0], shape[1]), generator=gen, device=device,
+                       dtype=torch.float32)
+
+
 @register("mixer", "attention")
 class Attention(Part):
     graph_safe = True
@@ -69,9 +84,9 @@ class Attention(Part):
     def __init__(self, hidden_size, num_heads, num_kv_heads, head_dim, eps, position, names,
                  qk_norm=True, window=None, scale=None, shared=None, reads_cache_only=False,
                  value_dim=None, q_temp=None, conv=None, sink=False, gate=False, bias=False, chunk=None,
-                 softcap=None):
+                 softcap=None, keep_first=0, distance_bias=None):
         """names: dict with q, k, v, o (and q_norm, k_norm when qk_norm is True or "whole"; q_conv, k_conv, v_conv
-        with conv; sink with sink; g with gate; q_bias, k_bias, v_bias, o_bias with bias) -> tensor names.
+        with conv; sink with sink=True; rel with distance_bias; g with gate; q_bias, k_bias, v_bias, o_bias with bias) -> tensor names.
         qk_norm: True (a weight [head_dim] each for queries and keys), "plain" (no weights), "whole" (over all
         heads of a token at once, weights of that size) or False.
         conv: taps of a filter along time on queries, keys and values (None: none).
@@ -99,7 +114,18 @@ class Attention(Part):
         self.position = shared.position(position)
         self.qkv = self.o = self.q_norm_w = self.k_norm_w = None
         self.taps = int(conv) if conv else 0
-        self.sink, self.gate, self.bias = bool(sink), bool(gate), bool(bias)
+        if sink not in (True, False, "unit"):
+            raise ValueError(f"sink is True, False or 'unit', not {sink!r}")
+        self.unit_sink = sink == "unit"
+        self.sink, self.gate, self.bias = sink is True, bool(gate), bool(bias)
+        self.keep_first = int(keep_first)
+        if self.keep_first < 0 or (self.keep_first and self.window is None):
+            raise ValueError("keep_first is a number of positions and goes with a window")
+        self.bias_max = None if distance_bias is None else distance_bias[0]
+        self.distance_plain = self.distance_raw = None
+        if (self.keep_first or self.bias_max is not None) and (chunk or softcap):
+            raise ValueError("kept first keys and a bias by distance do not go with chunks or capped scores")
+        self.stores_fresh_rows = True        # its output projection stores into rows that hold nothing yet
         self.chunk = int(chunk) if chunk else None
         self.softcap = float(softcap) if softcap else None
         if self.chunk is not None and (self.chunk <= 0 or self.window):
@@ -118,7 +144,6 @@ class Attention(Part):
                                  "weights, no growing query and no rotation of halves")
             if self.taps > recurrent.MAX_TAPS:
                 raise ValueError(f"the filter takes up to {recurrent.MAX_TAPS} taps, not {self.taps}")
-            self.stores_fresh_rows = True        # its output projection stores into rows that hold nothing yet
 
     @property
     def q_dim(self):
@@ -152,6 +177,8 @@ class Attention(Part):
         if self.taps:
             for key, rows in (("q_conv", self.nq * self.dim), ("k_conv", self.nkv * self.dim), ("v_conv", self.nkv * self.vdim)):
                 needs[n[key]] = TensorNeed((rows, self.taps), "taps", _taps_init)
+        if self.bias_max is not None:
+            needs[n["rel"]] = TensorNeed((None, self.nq), "bias", _distance_init)
         if self.sink:
             needs[n["sink"]] = TensorNeed((self.nq,), "bias", _sink_init)
         if self.gate:
@@ -208,8 +235,8 @@ class Attention(Part):
         if self.reads_cache_only:
             return None
         if self.taps > 1:
-            return (KVNeed(self.nkv, self.hd, self.window), StateNeed((self.taps - 1, self.channels), torch.float32))
-        return KVNeed(self.nkv, self.hd, self.window)
+            return (KVNeed(self.nkv, self.hd, self.window, keep_first=self.keep_first), StateNeed((self.taps - 1, self.channels), torch.float32))
+        return KVNeed(self.nkv, self.hd, self.window, keep_first=self.keep_first)
 
     def _load_prepared(self, tensors, rt):
         n = self.names
@@ -257,9 +284,19 @@ class Attention(Part):
             ops.add_bias(x, self.o_bias_w)
 
     def load(self, tensors, rt):
+        if self.unit_sink:
+            self.sink_w = torch.zeros(self.nq, dtype=torch.float32, device=rt.device)       # exp(0) = 1
         if self.prepared:
             self._load_prepared(tensors, rt)
-            return
+        else:
+            self._load_direct(tensors, rt)
+        if self.bias_max is not None:
+            by_distance = bias_by_distance(rt.weight(tensors[self.names["rel"]], matrix=False), self.bias_max)
+            self.distance_plain = ops.DistanceBias(by_distance)
+            # (the matrix-core kernels add it to the raw dot products)
+            self.distance_raw = ops.DistanceBias(by_distance / (self.scale if self.prepared else self.kernel_scale))
+
+    def _load_direct(self, tensors, rt):
         n = self.names
         self.hd = kept = self._kept_size(rt)
         rows = [self._heads_padded(tensors[n["q"]].to(rt.device), self.nq, self.dim, kept)]
@@ -293,9 +330,10 @@ class Attention(Part):
         return True
 
     def project_out(self, ctx, attn, x):
-        """x += attn @ Wo^T, the part's last product into the residual stream."""
-        left = ctx.leave_norm(self.o, x)
-        self.o.forward(attn, x, accumulate=True, leave=None if left is None else left.leave())
+        """x += attn @ Wo^T, the part's last product into the residual stream (or into rows that hold nothing yet)."""
+        adds = ctx.adds_to(x)
+        left = ctx.leave_norm(self.o, x) if adds else None
+        self.o.forward(attn, x, accumulate=adds, leave=None if left is None else left.leave())
 
     def forward(self, ctx, y, x, fused_norm=None, row_scale=None):
         if self.prepared:
@@ -337,7 +375,8 @@ class Attention(Part):
             # one token a sequence: norm, rotation, cache write and attention in one kernel
             mfma.attention_decode_fused(qkv, self.q_norm_w, self.k_norm_w, cos, sin, ctx.meta, kv, attn,
                                         self.nq, self.nkv, self.hd, self.kernel_eps, self.kernel_scale, self.window,
-                                        qkv_slices=slices, scratch=rt.scratch, q_temp=self.q_temp)
+                                        qkv_slices=slices, scratch=rt.scratch, q_temp=self.q_temp, sinks=self.sink_w,
+                                        bias=self.distance_raw, keep_first=self.keep_first)
             self.project_out(ctx, attn, x)
             return
         q = rt.buffer("q", (T, self.q_dim))
@@ -352,7 +391,8 @@ class Attention(Part):
         if q.dtype == torch.bfloat16:
             if mfma.attention_supported(q, kv, self.nq, self.nkv, self.hd):
                 mfma.attention(q, ctx.meta, kv, out, self.nq, self.nkv, self.hd, scale, self.window,
-                               scratch=ctx.rt.scratch, sinks=self.sink_w, chunk=self.chunk, softcap=self.softcap)
+                               scratch=ctx.rt.scratch, sinks=self.sink_w, chunk=self.chunk, softcap=self.softcap,
+                               bias=self.distance_raw, keep_first=self.keep_first)
                 return
         ops.attention_plain(q, ctx.meta, kv, out, self.nq, self.nkv, self.hd, scale, self.window, sinks=self.sink_w,
-                            chunk=self.chunk, softcap=self.softcap)
+                            chunk=self.chunk, softcap=self.softcap, bias=self.distance_plain, keep_first=self.keep_first)

@@ -172,6 +172,13 @@ class StepContext:
     # such block's first norm to add to x (x += factors * delta, a factor a channel)
     pending_scaled: Any = None
 
+    # (x's address, rows, norm): a block that norms after its parts has left its last part's output, and the norm
+    # that it passes, for the next such block's first kernel to add to x
+    pending_join: Any = None
+    # set by the model where a pass over a stretch of the schedule starts, for a block that takes it: (rows f32
+    # [T, hidden] or None, vector f32 [hidden] or None) to be added to x before the block's first norm
+    pass_input: Any = None
+
     def adds_to(self, x):
         """False if x are the context's fresh rows (the part's product stores), True if it has to add."""
         return not (self.fresh_rows is not None and self.fresh_rows.data_ptr() == x.data_ptr())

@@ -6,6 +6,9 @@ and their sum joins the residual stream times a constant.
 "postnorm": x <- norm_post_mixer(alpha x + mixer(x)); x <- norm_post_ff(alpha x + feed_forward(x)): the parts
 take x as it is, and each norm comes after its sum.
 
+"sandwich": x <- x + norm_after_mixer(mixer(norm_before_mixer(x))); x <- x + norm_after_ff(ff(norm_before_ff(x))):
+a norm before and after each part.
+
 "prenorm": x += mixer(norm_input(x)); x += feed_forward(norm_post_mixer(x)), the
 arrangement of the reference's two-norm layer
 (crates/backends/backend_common/src/generic_layer.rs:1149-1151, 1234-1236,
@@ -264,3 +267,70 @@ class PostNormBlock(Part):
                          alpha_after if last else self.alpha)
         if alpha_after != 0.0:
             ctx.pending_post = (x.data_ptr(), alpha_after)
+
+
+@register("block", "sandwich")
+class SandwichBlock(Part):
+    """x <- x + after_mixer(mixer(before_mixer(x))), then x <- x + after_ff(feed_forward(before_ff(x))) (the second
+    step only where the layer has a feed-forward). The parts store their outputs in float32 rows of their own; one
+    kernel between two parts norms those rows, adds them to x and writes the normed copy of x that the next part
+    reads. A layer's last sum is left for the next layer's first kernel, if that layer is such a block too,
+    and what joins x where a pass over the layers starts is added there as well."""
+    graph_safe = True
+    takes_pass_input = True
+
+    norm_roles = ("before_mixer", "after_mixer", "before_ff", "after_ff")
+
+    def __init__(self, mixer, feed_forward, norms):
+        self.mixer = mixer
+        self.feed_forward = feed_forward
+        self.norms = norms
+        roles = self.norm_roles[:2 if feed_forward is None else 4]
+        missing = [r for r in roles if r not in norms]
+        if missing:
+            raise ValueError(f"sandwich block needs norms {missing}")
+        for role in roles:
+            if not getattr(norms[role], "joins", False):
+                raise ValueError("sandwich block: its norms must be of a kind that needs no whole row")
+
+    def parts(self):
+        parts = [self.norms["before_mixer"], self.mixer, self.norms["after_mixer"]]
+        if self.feed_forward is not None:
+            parts += [self.norms["before_ff"], self.feed_forward, self.norms["after_ff"]]
+        return parts
+
+    def forward(self, ctx, x):
+        rt = ctx.rt
+        shape = tuple(x.shape)
+        branch = rt.buffer("sandwich_branch", shape, torch.float32)
+        y = rt.buffer("sandwich_rows", shape)
+        pending, ctx.pending_join = ctx.pending_join, None
+        extra, step = ctx.pass_input if ctx.pass_input is not None else (None, None)
+        ctx.pass_input = None
+        part_rows = after = None
+        if pending is not None and pending[0] == x.data_ptr():
+            part_rows, after = pending[1], pending[2].constants()
+        changed = part_rows is not None or extra is not None or step is not None
+        ops.tanh_join(x, part_rows, after, extra, step, x if changed else None, self.norms["before_mixer"].constants(), y)
+        self._run(ctx, self.mixer, y, branch)
+        last = self.norms["after_mixer"]
+        if self.feed_forward is not None:
+            ops.tanh_join(x, branch, last.constants(), x_out=x, before=self.norms["before_ff"].constants(), y=y)
+            self._run(ctx, self.feed_forward, y, branch)
+            last = self.norms["after_ff"]
+        if isinstance(ctx.next_block, SandwichBlock):
+            ctx.pending_join = (x.data_ptr(), branch, last)
+        else:
+            ops.tanh_join(x, branch, last.constants(), x_out=x)
+
+    @staticmethod
+    def _run(ctx, part, y, branch):
+        ctx.handed = ctx.norm_ahead = ctx.left = None
+        # a part that can store its rows instead of adding them says so and finds the rows in ctx.fresh_rows;
+        # for any other the rows are cleared first
+        if getattr(part, "stores_fresh_rows", False):
+            ctx.fresh_rows = branch
+        else:
+            ops.fill_u32(branch, 0)
+        part.forward(ctx, y, branch)
+        ctx.fresh_rows = None

@@ -46,9 +46,7 @@ class TokenEmbedding(Part):
 
     def forward(self, ctx, token_ids):
         x = ctx.rt.buffer("residual", (token_ids.shape[0], self.hidden_size), torch.float32)
-        ops.embed(token_ids, self.table, x, packed=self.linear.packed)
-        if self.scale is not None:
-            ops.scale(x, self.scale)
+        ops.embed(token_ids, self.table, x, packed=self.linear.packed, scale=1.0 if self.scale is None else self.scale)
         if self.norm is not None:
             self.norm.forward_in_place(ctx, x)
         return x
@@ -58,9 +56,14 @@ class TokenEmbedding(Part):
 class OutputHead(Part):
     graph_safe = True
 
-    def __init__(self, vocab_size, hidden_size, weight, tied_to_embedding, norm, shared=None, logit_scale=None):
+    def __init__(self, vocab_size, hidden_size, weight, tied_to_embedding, norm, shared=None, logit_scale=None,
+                 softcap=None):
         """weight: the head's tensor name; tied_to_embedding: use the embedding table instead;
-        logit_scale: the logits are the product times this constant (None: as they are)."""
+        logit_scale: the logits are the product times this constant (None: as they are). softcap: a logit z becomes
+        softcap tanh(z / softcap) (after the constant; None: as it is)."""
+        self.softcap = None if softcap is None else float(softcap)
+        if self.softcap is not None and self.softcap <= 0:
+            raise ValueError("the logits' cap must be positive")
         self.logit_scale = None if logit_scale is None or float(logit_scale) == 1.0 else float(logit_scale)
         self.vocab_size = int(vocab_size)
         self.hidden_size = int(hidden_size)
@@ -93,4 +96,6 @@ class OutputHead(Part):
         self.proj.forward(y, logits)
         if self.logit_scale is not None:
             ops.scale(logits, self.logit_scale)
+        if self.softcap is not None:
+            ops.softcap(logits, self.softcap)
         return logits

@@ -1,5 +1,5 @@
 """Dense feed-forwards without biases. "swiglu": down(f(gate(y)) * up(y)) with f = silu, or with `activation="gelu_tanh"`
-the tanh form of gelu. "squared_relu": down(max(up(y), 0)^2).
+the tanh form of gelu or with `activation="relu"` max(z, 0). "squared_relu": down(max(up(y), 0)^2).
 
 crates/backends/backend_common/src/generic_mlp.rs:83-96 and kernels.rs:676-687
 of the reference; gate and up are one fused matrix here so that the activations
@@ -20,7 +20,7 @@ class SwiGLU(Part):
     stores_fresh_rows = True     # its last product stores into rows that hold nothing yet (StepContext.adds_to)
 
     def __init__(self, hidden_size, intermediate_size, names, shared=None, activation="silu"):
-        """names: dict with gate, up, down -> tensor names. activation: "silu" or "gelu_tanh" (on the gate)."""
+        """names: dict with gate, up, down -> tensor names. activation: "silu", "gelu_tanh" or "relu" (on the gate)."""
         if activation not in ops.GLU_ACTIVATIONS:
             raise ValueError(f"the gated unit's activation is one of {sorted(ops.GLU_ACTIVATIONS)}, not {activation!r}")
         self.activation = activation

@@ -82,3 +82,45 @@ class LayerNorm(Part):
         """x <- norm(x), float32: for a norm that is part of the residual stream itself."""
         ops.layernorm(x, self.w, x, self.eps)
         return x
+
+
+def _alpha_init(shape, gen, device, std, norm_std):
+    """A random model's inner factor: rows of a size around one land where the tangent bends."""
+    import torch
+    return 0.6 + 0.2 * torch.rand(shape, generator=gen, device=device, dtype=torch.float32)
+
+
+@register("norm", "dynamic_tanh")
+class DynamicTanh(Part):
+    """y = tanh(alpha x) w + b: no mean, no variance, a stored factor alpha inside and a bias outside. Nothing
+    of it needs a whole row, so the sums that join the residual stream between two such norms run in the
+    same kernel (`joins`: a block may hand `constants()` to ops.tanh_join)."""
+    graph_safe = True
+    joins = True
+
+    def __init__(self, size, weight, eps=None):
+        """weight: the tensor's name; its neighbours are weight + ".alpha" (a scalar) and weight + ".b". eps is
+        taken like any norm's and not used."""
+        self.size = int(size)
+        self.weight_name = weight
+        self.w = self.b = None
+        self.alpha = 0.0
+
+    def tensor_needs(self):
+        return {self.weight_name: TensorNeed((self.size,), "scale"),
+                self.weight_name + ".alpha": TensorNeed((), "scale", _alpha_init),
+                self.weight_name + ".b": TensorNeed((self.size,), "bias", _around_zero)}
+
+    def load(self, tensors, rt):
+        self.w = rt.weight(tensors[self.weight_name], matrix=False)
+        self.b = rt.weight(tensors[self.weight_name + ".b"], matrix=False)
+        self.alpha = float(tensors[self.weight_name + ".alpha"].float().item())
+
+    def constants(self):
+        return self.alpha, self.w, self.b
+
+    def forward(self, ctx, x, rows=None, name="normed"):
+        n = x.shape[0] if rows is None else rows.shape[0]
+        y = ctx.rt.buffer(name, (n, self.size))
+        ops.tanh_join(x, before=self.constants(), y=y, rows=rows)
+        return y

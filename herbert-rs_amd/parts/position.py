@@ -17,6 +17,26 @@ from .base import Part
 from .registry import register
 
 
+def distance_bucket(n, rows, bias_max):
+    """The row of a table of `rows` learned biases that the distance n takes: a row a distance for the first half of
+    them, then rows that grow with the distance's logarithm up to bias_max, the last row from there on."""
+    half = rows // 2
+    if n < half:
+        return n
+    return min(rows - 1, half + math.floor(math.log(n / half) / math.log(bias_max / half) * (rows - half)))
+
+
+def bias_by_distance(table, bias_max):
+    """table f32 [rows, heads] -> f32 [length, heads]: the biases of the distances 0 .. length - 1, the last of which
+    holds for every distance beyond it."""
+    rows = table.shape[0]
+    if rows < 2 or not bias_max > rows // 2:
+        raise ValueError(f"a table of {rows} biases needs two rows and a largest distance beyond half of them, not {bias_max}")
+    length = max(rows // 2, math.ceil(bias_max)) + 1
+    index = torch.tensor([distance_bucket(n, rows, bias_max) for n in range(length)], dtype=torch.long)
+    return table[index.to(table.device)].contiguous()
+
+
 @register("position", "none")
 class NoPosition(Part):
     graph_safe = True

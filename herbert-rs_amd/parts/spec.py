@@ -27,9 +27,12 @@ class LayerSpec:
 @dataclass(frozen=True)
 class ScheduleEntry:
     """One run of a layer. `cache` None: the entry owns a cache of its own; an int: it reads
-    the cache of that earlier entry of the schedule and writes none."""
+    the cache of that earlier entry of the schedule and writes none. `starts_pass`: the number of the pass over a
+    stretch of the schedule that starts with this entry (the model's `pass_input` part says what joins the stream
+    there), or None."""
     layer: int
     cache: Optional[int] = None
+    starts_pass: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -43,3 +46,4 @@ class ModelSpec:
     final_norm: PartSpec
     head: PartSpec
     eos_token_id: Optional[int] = None
+    pass_input: Optional[PartSpec] = None      # a part of the category "pass_input", for a schedule that names passes
