@@ -21,7 +21,7 @@ step is what the generation loop does for a token: the step function (a HIP-grap
 greedy choice on the GPU, and the chosen tokens read by the host, which as in that loop reads
 the tokens of a step while the next step, fed from the GPU, already runs.
 
-`--workload vipalorn|modasun|mefatar|bozasun --size small|medium|wide` measures one of the other designs instead (random weights at
+`--workload vipalorn|modasun|mefatar|bozasun|mutedra --size small|medium|wide` measures one of the other designs instead (random weights at
 sizes that resemble a real model's layers) beside the closest other model at equal size, through the generation
 loop; the default workload and its JSON line stay as they are.
 """
@@ -229,10 +229,31 @@ def bozasun_configs(size):
     return boz, family_configs(size)[0]
 
 
+def mutedra_configs(size):
+    """(Mutedra config dict, Qwen3 config dict, Vipalorn config dict) of one size, as many layer runs as the others have
+    layers: the first two layers run twice. Every other layer is a softmax attention over the last 1,024 keys and the
+    first four (a bias by distance up to 2,560, a one in the denominator), of the rest most are latent attentions
+    with a rotated part, a sink and a gate a head, every third one without positions, all with queries from a latent of
+    a quarter of the width; every layer has a dense feed-forward as wide as the dense decoder's. The dense decoder is
+    the closest model by its layers' work, Vipalorn the one that has a latent attention."""
+    W, L, H, D, V, rank, rot, E, top, ff, vocab = FAMILY_SIZES[size]
+    mlp = {"kind": "dense", "ff": top * ff}
+    plain = {"heads": H, "dim": D, "vdim": V, "kv_rank": rank, "q_rank": W // 4, "scale": D ** -0.5}
+    rotated = dict(plain, rot_dim=rot, scale=(D + rot) ** -0.5, rot={"base": 10000.0, "dims": rot})
+    attention = {"heads": H, "kv_heads": H // 2, "dim": D, "vdim": V, "scale": D ** -0.5, "bias_max": 2560,
+                 "mask": {"size": 1024, "keep_first": 4}}
+    kinds = [("latent_attention_2", rotated), ("attention", attention), ("latent_attention", plain), ("attention", attention),
+             ("latent_attention_2", rotated), ("attention", attention)]
+    layers = [{"type": kinds[i % 6][0], "mixer": kinds[i % 6][1], "mlp": mlp} for i in range(L - 2)]
+    mut = {"architecture": "Mutedra", "vocab": vocab, "width": W, "layers": layers, "norm": {"eps": 1e-5},
+           "embedding": {"scale": 1.0}, "loop": {"start": 0, "stop": 2, "times": 2}, "logit_softcap": 30.0}
+    return (mut,) + family_configs(size)[::-1]
+
+
 def run_family(args, names=("vipalorn", "qwen3"), configs=family_configs):
     """Prompt and decode throughput of a design at one size (random weights) beside the closest other model at
-    equal size (Vipalorn beside the dense Qwen3 decoder, Modasun beside Vipalorn, Mefatar beside Modasun, Bozasun beside Vipalorn), both through the generation
-    loop: prompts of 512 and 2,048 tokens alone, and batches of 1, 8 and 32 sequences of 1,024 prompt tokens
+    equal size (Vipalorn beside the dense Qwen3 decoder, Modasun beside Vipalorn, Mefatar beside Modasun, Bozasun beside
+    Vipalorn, Mutedra beside the dense decoder and Vipalorn), all through the generation loop: prompts of 512 and 2,048 tokens alone, and batches of 1, 8 and 32 sequences of 1,024 prompt tokens
     decoding `--steps` tokens each."""
     import torch
     import herbert_rs_amd as hb
@@ -284,7 +305,7 @@ def run_family(args, names=("vipalorn", "qwen3"), configs=family_configs):
             "config": {"model": f"{design} {args.size}", "sizes": dict(zip(
                 ("width", "layers", "heads", "key_dim", "value_dim", "latent_rank", "rotated", "experts", "top", "expert_ff", "vocab"),
                 FAMILY_SIZES[args.size])), "global_batch": 8, "parallelism": "single GPU"},
-            names[0]: v, names[1] + "_equal_size": out[names[1]]}
+            names[0]: v, **{n + "_equal_size": out[n] for n in names[1:]}}
 
 
 def main():
@@ -303,7 +324,8 @@ def main():
     ap.add_argument("--no-long", action="store_true",
                     help="skip the further sizes and lengths (contexts of 16 K and 32 K, batch 128 and 256, long prompts)")
     ap.add_argument("--size", default="medium", choices=sorted(FAMILY_SIZES), help="layer sizes of --workload vipalorn, modasun, mefatar and bozasun")
-    ap.add_argument("--workload", default="headline", choices=["headline", "qwen3-1.7b", "qwen3-32b", "vipalorn", "modasun", "mefatar", "bozasun"],
+    ap.add_argument("--workload", default="headline", choices=["headline", "qwen3-1.7b", "qwen3-32b", "vipalorn", "modasun", "mefatar", "bozasun",
+                                                                "mutedra"],
                     help="headline: BASELINE.json configs[2]; qwen3-*: configs[3] and configs[4]; vipalorn, modasun, mefatar: "
                          "that design at --size beside the closest other model at equal size")
     ap.add_argument("--prefill-tokens", type=int, default=2048, help="length of the prompt of the prefill figure")
@@ -332,6 +354,9 @@ def main():
     if args.workload == "mefatar":
         print(json.dumps(run_family(args, names=("mefatar", "modasun"), configs=mefatar_configs)))
         return 0
+    if args.workload == "mutedra":
+        print(json.dumps(run_family(args, names=("mutedra", "qwen3", "vipalorn"), configs=mutedra_configs)))
+        return
     if args.workload == "bozasun":
         print(json.dumps(run_family(args, names=("bozasun", "vipalorn"), configs=bozasun_configs)))
         return 0
