@@ -566,6 +566,7 @@ extern "C" int hb_scale(float* x, float s, size_t n, hipStream_t stream) {
 //   s = x[r] + n_after(part[r]) + extra[r] + step;   x_out[r] = s;   y[r] = n_before(s)
 // part (a part's output), extra (rows of their own), step (one vector for all rows), x_out and y are each there or
 // not; r = rows ? rows[i] : i picks the rows of x (with rows: only x and y). Everything float32 but y's storage.
+// slices > 1: part's product was cut into that many slices of K, slice_stride floats apart, added up here in order.
 struct DynTanh {
     const float* w;      // null: there is no such norm
     const float* b;
@@ -574,7 +575,7 @@ struct DynTanh {
 
 template <class TOut, bool QUADS>
 __global__ void __launch_bounds__(256)
-tanh_join_kernel(const float* x, const float* __restrict__ part, DynTanh after, const float* __restrict__ extra,
+tanh_join_kernel(const float* x, const float* __restrict__ part, int slices, size_t slice_stride, DynTanh after, const float* __restrict__ extra,
                  const float* __restrict__ step, float* x_out, DynTanh before, TOut* __restrict__ y,
                  const int* __restrict__ rows, int H, unsigned total) {
     const unsigned idx = blockIdx.x * 256u + threadIdx.x;       // a quad of four neighbours, or one number
@@ -591,7 +592,9 @@ tanh_join_kernel(const float* x, const float* __restrict__ part, DynTanh after, 
     };
     hb_f4 s = load(x + from);
     if (part) {
-        const hb_f4 p = load(part + at), w = load(after.w + c), b = load(after.b + c);
+        hb_f4 p = load(part + at);
+        const hb_f4 w = load(after.w + c), b = load(after.b + c);
+        for (int i2 = 1; i2 < slices; ++i2) p += load(part + i2 * slice_stride + at);
 #pragma unroll
         for (int e = 0; e < N; ++e) s[e] += tanhf(after.alpha * p[e]) * w[e] + b[e];
     }
@@ -610,24 +613,25 @@ tanh_join_kernel(const float* x, const float* __restrict__ part, DynTanh after, 
     }
 }
 
-extern "C" int hb_tanh_join(const float* x, const float* part, float alpha_after, const float* w_after,
+extern "C" int hb_tanh_join(const float* x, const float* part, int slices, size_t slice_stride, float alpha_after, const float* w_after,
                             const float* b_after, const float* extra, const float* step, float* x_out,
                             float alpha_before, const float* w_before, const float* b_before, void* y, int y_dtype,
                             const int* rows, int R, int H, hipStream_t stream) {
     HB_REQUIRE(R > 0 && H > 0, "tanh norm: empty input (R=%d, H=%d)", R, H);
     HB_REQUIRE(x && (x_out || y), "tanh norm: nothing to do");
+    HB_REQUIRE(slices >= 1 && (slices == 1 || (part && slice_stride >= (size_t)R * H)), "tanh norm: bad slices");
     HB_REQUIRE(!part || (w_after && b_after), "tanh norm: a part's output without the norm that it passes");
     HB_REQUIRE(!y || (w_before && b_before), "tanh norm: rows to write without their norm");
     HB_REQUIRE(!rows || (!part && !extra && !step && !x_out), "tanh norm: rows are not gathered while a sum is added");
     HB_REQUIRE(y_dtype == HB_F32 || y_dtype == HB_BF16, "tanh norm: unknown output dtype %d", y_dtype);
     const uintptr_t all = (uintptr_t)x | (uintptr_t)part | (uintptr_t)w_after | (uintptr_t)b_after | (uintptr_t)extra |
                           (uintptr_t)step | (uintptr_t)x_out | (uintptr_t)w_before | (uintptr_t)b_before | (uintptr_t)y;
-    const bool quads = H % 4 == 0 && all % 16 == 0;
+    const bool quads = H % 4 == 0 && all % 16 == 0 && (slices == 1 || slice_stride % 4 == 0);
     const size_t total = (size_t)R * H / (quads ? 4 : 1);
     HB_REQUIRE(total < (1ull << 31), "tanh norm: too many rows");
     const unsigned blocks = (unsigned)((total + 255) / 256);
     const DynTanh after = {w_after, b_after, alpha_after}, before = {w_before, b_before, alpha_before};
-#define HB_TANH_JOIN(T, Q) tanh_join_kernel<T, Q><<<blocks, 256, 0, stream>>>(x, part, after, extra, step, x_out, before, (T*)y, rows, H, (unsigned)total)
+#define HB_TANH_JOIN(T, Q) tanh_join_kernel<T, Q><<<blocks, 256, 0, stream>>>(x, part, slices, slice_stride, after, extra, step, x_out, before, (T*)y, rows, H, (unsigned)total)
     if (y_dtype == HB_F32) {
         if (quads) HB_TANH_JOIN(float, true);
         else HB_TANH_JOIN(float, false);

@@ -12,10 +12,11 @@
 // on instead of run (see NormHandoff).
 // In both the weight rows are the MFMA's first operand, so a lane ends up with runs of four
 // consecutive n of one m: row-major stores of C are vector stores.
-// Epilogues: 0 store float32, 1 add to float32 (the residual stream), 2 SwiGLU to bfloat16
+// Epilogues: 0 store float32, 1 add to float32 (the residual stream), 2 SwiGLU (or another gated unit) to bfloat16
 // (weight rows interleaved in blocks of 16: gate rows, then the up rows of the same outputs),
 // 3 (tiled, an entry point of its own) the q/k/v projection with per-head norm, rotation and
-// cache write.
+// cache write, 4 (few rows, an entry point of its own) the sums pass a norm without mean and variance and join the
+// residual stream, which passes another one (see TanhJoin).
 // In xigh/herbert-rs: crates/backends/backend_bf16/src/kernels.rs:154-164 is the product; the inputs are rounded to
 // bfloat16 before they are multiplied, as crates/backends/backend_bf16_avx512/src/avx512_bf16_matvec.S:1-12 does
 // (float32 sums); SwiGLU in the epilogue as crates/backends/backend_metal/shaders/fused_gate_up_swiglu.metal:27-83;
@@ -37,12 +38,35 @@ typedef float f32x16 __attribute__((ext_vector_type(16)));
 #define EPI_ADD 1
 #define EPI_SWIGLU 2
 #define EPI_QKV 3
+#define EPI_JOIN 4
 
 // silu(g) u with the hardware's reciprocal (1 ulp; the result is rounded to bfloat16): a full division
 // is a dozen instructions, and the epilogue of a 256 x 256 tile does 128 of these a lane
 __device__ __forceinline__ float silu_mul(float g, float u) {
     return g * __builtin_amdgcn_rcpf(1.0f + __expf(-g)) * u;
 }
+
+// the gated unit of epilogue 2: silu(g) u or max(g, 0) u
+#define GLU_SILU 0
+#define GLU_RELU 1
+template <int GLU>
+__device__ __forceinline__ float glu_mul(float g, float u) {
+    return GLU == GLU_RELU ? fmaxf(g, 0.f) * u : silu_mul(g, u);
+}
+
+// What epilogue 4 does with a product's sums p (a part's output): s = x + n_after(p) + extra + step, n(v) =
+// tanh(alpha v) w + b; x <- s, y = bf16(n_before(s)). extra [M, N] and step [N] may be null, and so may y.
+struct TanhJoin {
+    float alpha_after;
+    const float* w_after;
+    const float* b_after;
+    const float* extra;
+    const float* step;
+    float alpha_before;
+    const float* w_before;
+    const float* b_before;
+    bf16* y;                     // [M, N]
+};
 
 // ---------------------------------------------------------------- few rows
 // Workgroup: WAVES waves, NB blocks of 16 weight rows, MB blocks of 16 activation rows (built for
@@ -91,12 +115,13 @@ struct NormHandoff {
     int scale_parts;
     float scale_eps;             // the width of the normed rows is this product's K
     float emit_eps;
+    int glu;                     // the gated unit of epilogue 2
 };
 
 template <int MB, int NB, int WAVES, int EPI, bool PACKED, bool NORM>
 __global__ void __launch_bounds__(WAVES * 64)
 gemm_skinny_kernel(const void* __restrict__ Xv, const bf16* __restrict__ W, void* __restrict__ Cv, int M,
-                   int N, int K, int ldc, const float* __restrict__ norm_w, float eps, NormHandoff hand) {
+                   int N, int K, int ldc, const float* __restrict__ norm_w, float eps, NormHandoff hand, TanhJoin join) {
     constexpr int U = NORM ? 2 : ((NB + MB <= 4) ? 4 : 2);
     const bf16* X = (const bf16*)Xv;
     const float* XF = (const float*)Xv;
@@ -156,6 +181,25 @@ gemm_skinny_kernel(const void* __restrict__ Xv, const bf16* __restrict__ W, void
                 c_before[a][i] = in ? ((const float*)Cv)[(size_t)r16 * ldc + n] : 0.f;
                 g_ahead[a][i] = in && hand.emit_g ? hand.emit_g[n] : 0.f;
             }
+    }
+    // (epilogue 4: the stream, the vectors of the two norms, and what else joins)
+    f32x4 j_x[NB], j_wa[NB], j_ba[NB], j_wb[NB], j_bb[NB];
+    if (EPI == EPI_JOIN && wave == 0) {
+#pragma unroll
+        for (int a = 0; a < NB; ++a) {
+            // (N in steps of 16: every lane's four columns exist)
+            const int n = n0 + a * 16 + g4 * 4;
+            const int m = r16 < M ? r16 : M - 1;
+            j_x[a] = *(const f32x4*)((const float*)Cv + (size_t)m * ldc + n);
+            if (join.extra) j_x[a] += *(const f32x4*)(join.extra + (size_t)m * N + n);
+            if (join.step) j_x[a] += *(const f32x4*)(join.step + n);
+            j_wa[a] = *(const f32x4*)(join.w_after + n);
+            j_ba[a] = *(const f32x4*)(join.b_after + n);
+            if (join.y) {
+                j_wb[a] = *(const f32x4*)(join.w_before + n);
+                j_bb[a] = *(const f32x4*)(join.b_before + n);
+            }
+        }
     }
     const int mine = wave < nsteps ? (nsteps - wave + WAVES - 1) / WAVES : 0;   // this wave's steps
     const int groups = mine / U;
@@ -324,6 +368,24 @@ gemm_skinny_kernel(const void* __restrict__ Xv, const bf16* __restrict__ W, void
     }
 
     // lane: m = b * 16 + r16, n = n0 + a * 16 + g4 * 4 + i
+    if (EPI == EPI_JOIN) {
+        if (r16 >= M) return;
+#pragma unroll
+        for (int a = 0; a < NB; ++a) {
+            const int n = n0 + a * 16 + g4 * 4;
+            f32x4 x = j_x[a];
+            bf16x4 y;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) x[i] += tanhf(join.alpha_after * acc[a][0][i]) * j_wa[a][i] + j_ba[a][i];
+            *(f32x4*)((float*)Cv + (size_t)r16 * ldc + n) = x;
+            if (join.y) {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) y[i] = (__bf16)(tanhf(join.alpha_before * x[i]) * j_wb[a][i] + j_bb[a][i]);
+                *(bf16x4*)((__bf16*)join.y + (size_t)r16 * N + n) = y;
+            }
+        }
+        return;
+    }
     if (EPI == EPI_SWIGLU) {
         bf16* C = (bf16*)Cv;
         const int out_n0 = n0 / 2;
@@ -337,7 +399,9 @@ gemm_skinny_kernel(const void* __restrict__ Xv, const bf16* __restrict__ W, void
                 for (int i = 0; i < 4; ++i) {
                     const int n = out_n0 + (a / 2) * 16 + g4 * 4 + i;
                     if (n < N / 2)
-                        C[(size_t)m * ldc + n] = hb_from_float<bf16>(silu_mul(acc[a][b][i], acc[a + 1][b][i]));
+                        C[(size_t)m * ldc + n] = hb_from_float<bf16>(
+                            hand.glu == GLU_RELU ? glu_mul<GLU_RELU>(acc[a][b][i], acc[a + 1][b][i])
+                                                 : glu_mul<GLU_SILU>(acc[a][b][i], acc[a + 1][b][i]));
                 }
             }
     } else {
@@ -477,6 +541,7 @@ gemm_slices_norm_kernel(const float* __restrict__ partial, float* __restrict__ C
 
 // The same for the SwiGLU epilogue: column j of the output pairs the sums of the gate row
 // 32 (j / 16) + j % 16 and of the up row 16 further on; C bf16 [M, N / 2].
+template <int GLU>
 __global__ void gemm_slices_swiglu_kernel(const float* __restrict__ partial, bf16* __restrict__ C, int M, int N,
                                           int ldc, int slices) {
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -489,7 +554,7 @@ __global__ void gemm_slices_swiglu_kernel(const float* __restrict__ partial, bf1
         gate += partial[(size_t)s * M * N + at];
         up += partial[(size_t)s * M * N + at + 16];
     }
-    C[(size_t)m * ldc + j] = hb_from_float<bf16>(silu_mul(gate, up));
+    C[(size_t)m * ldc + j] = hb_from_float<bf16>(glu_mul<GLU>(gate, up));
 }
 
 template <int MB, int NB, int WAVES>
@@ -502,7 +567,7 @@ static void launch_skinny(const void* X, const void* W, void* C, int M, int N, i
     const bf16* w = (const bf16*)W;
 #define SKINNY_GO(EPIV, PK, NM)                                                                        \
     gemm_skinny_kernel<MB, NB, WAVES, EPIV, PK, NM><<<blocks, WAVES * 64, lds, stream>>>(X, w, C, M, N, K, \
-                                                                                          ldc, norm_w, eps, hand)
+                                                                                          ldc, norm_w, eps, hand, TanhJoin{})
     if (norm_w) {       // the normed input never meets the add epilogue; built for one block of rows
         if constexpr (MB == 1 && WAVES == 4) {
             if (packed) {
@@ -565,7 +630,7 @@ __device__ __forceinline__ bool tile_of_workgroup(int m_tiles, int n_tiles, int&
 }
 
 // A wave's sums to memory. m_base, n_base: first row and column of the wave's tile.
-template <int EPI, int TN32, int TM32>
+template <int EPI, int TN32, int TM32, int GLU = GLU_SILU>
 __device__ __forceinline__ void store_wave_tile(const f32x16 (&acc)[TN32][TM32], void* Cv, int M, int N, int ldc,
                                                 int m_base, int n_base, int c32, int g2) {
 #pragma unroll
@@ -584,14 +649,14 @@ __device__ __forceinline__ void store_wave_tile(const f32x16 (&acc)[TN32][TM32],
                         bf16x4 v;
 #pragma unroll
                         for (int j = 0; j < 4; ++j)
-                            v[j] = (__bf16)silu_mul(acc[a][b][4 * q + j], acc[a][b][4 * q + 8 + j]);
+                            v[j] = (__bf16)glu_mul<GLU>(acc[a][b][4 * q + j], acc[a][b][4 * q + 8 + j]);
                         *(bf16x4*)((__bf16*)C + (size_t)m * ldc + n) = v;
                     } else {
 #pragma unroll
                         for (int j = 0; j < 4; ++j)
                             if (n + j < N / 2)
                                 C[(size_t)m * ldc + n + j] = hb_from_float<bf16>(
-                                    silu_mul(acc[a][b][4 * q + j], acc[a][b][4 * q + 8 + j]));
+                                    glu_mul<GLU>(acc[a][b][4 * q + j], acc[a][b][4 * q + 8 + j]));
                     }
                 }
         } else {
@@ -685,7 +750,7 @@ __device__ __forceinline__ void store_wave_tile_lds(const f32x16 (&acc)[TN32][TM
 // along the rows: an instruction stores whole rows, 128 contiguous bytes for a tile 128 wide.
 // n_base: the wave's first column among the interleaved gate/up columns. Needs ldc in steps of
 // 8 and C aligned to 16 bytes.
-template <int TN32, int TM32>
+template <int TN32, int TM32, int GLU>
 __device__ __forceinline__ void store_wave_tile_swiglu_lds(const f32x16 (&acc)[TN32][TM32], bf16* C, int M, int N,
                                                            int ldc, int m_base, int n_base, int lane, bf16* stage) {
     constexpr int CH = 2 * TN32;            // 16-byte chunks of a row: 16 outputs a piece of 32 columns
@@ -704,7 +769,7 @@ __device__ __forceinline__ void store_wave_tile_swiglu_lds(const f32x16 (&acc)[T
                 const int row = 32 * b + c32;
                 bf16x4 v;
 #pragma unroll
-                for (int j = 0; j < 4; ++j) v[j] = (__bf16)silu_mul(acc[a][b][4 * q + j], acc[a][b][4 * q + 8 + j]);
+                for (int j = 0; j < 4; ++j) v[j] = (__bf16)glu_mul<GLU>(acc[a][b][4 * q + j], acc[a][b][4 * q + 8 + j]);
                 *(bf16x4*)((__bf16*)stage + row * (CH * 8) + place(row, 2 * a + q) * 8 + 4 * g2) = v;
             }
     const int rrow = lane / CH, rchunk = lane % CH;
@@ -840,6 +905,7 @@ struct RowScale {
     const float* partial;        // [parts, MP]; null: no scaling
     int parts;
     float eps;
+    int glu;                     // the gated unit of epilogue 2
 };
 
 // K in steps of 64. A step's weights are two k-steps of 32 (blocks as above); its activations lie
@@ -1068,8 +1134,13 @@ gemm_tile_kernel(const bf16* __restrict__ X, const bf16* __restrict__ W, void* _
         constexpr bool SWIGLU_VIA_LDS = EPI == EPI_SWIGLU && BM >= 128 && REGION >= 32 * TM32 * TN32 * 32;
         if (SWIGLU_VIA_LDS && !sliced && (ldc & 7) == 0 && ((size_t)Cv & 15) == 0) {
             hb_workgroup_barrier();
-            store_wave_tile_swiglu_lds<TN32, TM32>(acc, (bf16*)Cv, M, N, ldc, m0 + wm * TMB * 16, n0 + wn * TNB * 16, lane,
-                                                   (bf16*)((char*)lds + wave * REGION));
+            bf16* const stage = (bf16*)((char*)lds + wave * REGION);
+            if (scale.glu == GLU_RELU)
+                store_wave_tile_swiglu_lds<TN32, TM32, GLU_RELU>(acc, (bf16*)Cv, M, N, ldc, m0 + wm * TMB * 16,
+                                                                 n0 + wn * TNB * 16, lane, stage);
+            else
+                store_wave_tile_swiglu_lds<TN32, TM32, GLU_SILU>(acc, (bf16*)Cv, M, N, ldc, m0 + wm * TMB * 16,
+                                                                 n0 + wn * TNB * 16, lane, stage);
         } else if (VIA_LDS && (ld & 3) == 0 && (N & 3) == 0 && ((size_t)dst & 15) == 0) {
             hb_workgroup_barrier();
             float* const stage = (float*)((char*)lds + wave * REGION);
@@ -1081,6 +1152,8 @@ gemm_tile_kernel(const bf16* __restrict__ X, const bf16* __restrict__ W, void* _
                                                              n0 + wn * TNB * 16, lane, stage);
         } else if (sliced) {
             store_wave_tile<EPI_STORE, TN32, TM32>(acc, dst, M, N, N, m0 + wm * TMB * 16, n0 + wn * TNB * 16, c32, g2);
+        } else if (EPI == EPI_SWIGLU && scale.glu == GLU_RELU) {
+            store_wave_tile<EPI, TN32, TM32, GLU_RELU>(acc, Cv, M, N, ldc, m0 + wm * TMB * 16, n0 + wn * TNB * 16, c32, g2);
         } else {
             store_wave_tile<EPI, TN32, TM32>(acc, Cv, M, N, ldc, m0 + wm * TMB * 16, n0 + wn * TNB * 16, c32, g2);
         }
@@ -1093,7 +1166,7 @@ gemm_tile_kernel(const bf16* __restrict__ X, const bf16* __restrict__ W, void* _
 template <int EPI, bool PACKED, int TNB, int TMB, int WNW, int WMW, int STAGES>
 __global__ void __launch_bounds__(64 * WNW * WMW)
 gemm_tile32_kernel(const bf16* __restrict__ X, const bf16* __restrict__ W, void* __restrict__ Cv, int M, int N,
-                   int K, int ldc, int m_tiles, int n_tiles) {
+                   int K, int ldc, int m_tiles, int n_tiles, int glu) {
     constexpr int NW = WNW * WMW;
     constexpr int BN = 16 * TNB * WNW, BM = 16 * TMB * WMW;
     constexpr int WBLK = BN / 16, XBLK = BM / 16, BLKS = WBLK + XBLK;   // 1 KB blocks of a stage
@@ -1201,7 +1274,10 @@ gemm_tile32_kernel(const bf16* __restrict__ X, const bf16* __restrict__ W, void*
         if (t + 1 < nsteps) run_step(1, t + 1);
     }
     hb_wait_vmcnt<0>();      // the loads past the end (repeats of the last step) have landed too
-    store_wave_tile<EPI, TN32, TM32>(acc, Cv, M, N, ldc, m0 + wm * TMB * 16, n0 + wn * TNB * 16, c32, g2);
+    if (EPI == EPI_SWIGLU && glu == GLU_RELU)
+        store_wave_tile<EPI, TN32, TM32, GLU_RELU>(acc, Cv, M, N, ldc, m0 + wm * TMB * 16, n0 + wn * TNB * 16, c32, g2);
+    else
+        store_wave_tile<EPI, TN32, TM32>(acc, Cv, M, N, ldc, m0 + wm * TMB * 16, n0 + wn * TNB * 16, c32, g2);
 }
 
 // More than 64 KB of dynamic LDS has to be allowed per kernel, once.
@@ -1267,7 +1343,7 @@ static int launch_tile64(const void* X, const void* W, void* C, int M, int N, in
 // counts on rows of a power of two of 16-byte chunks).
 template <int TNB, int TMB, int WNW, int WMW, int WST, int XST>
 static int launch_tile64_swiglu(const void* X, const void* W, void* C, int M, int N, int K, int ldc, int epi,
-                                int packed, hipStream_t stream, int slices) {
+                                int packed, hipStream_t stream, int slices, RowScale scale) {
     constexpr int BN = 16 * TNB * WNW, BM = 16 * TMB * WMW;
     HB_REQUIRE(epi == EPI_SWIGLU && slices == 1, "gemm_mfma: this tile takes the SwiGLU product whole only");
     HB_REQUIRE(K % 64 == 0, "gemm_mfma: K=%d is no multiple of 64", K);
@@ -1278,14 +1354,14 @@ static int launch_tile64_swiglu(const void* X, const void* W, void* C, int M, in
     const bf16* w = (const bf16*)W;
     if (packed)
         return launch_tiles(gemm_tile_kernel<EPI_SWIGLU, true, TNB, TMB, WNW, WMW, WST, XST>, lds, 64 * WNW * WMW, total, 1,
-                            x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream, (float*)nullptr, QkvEpilogue{}, RowScale{});
+                            x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream, (float*)nullptr, QkvEpilogue{}, scale);
     return launch_tiles(gemm_tile_kernel<EPI_SWIGLU, false, TNB, TMB, WNW, WMW, WST, XST>, lds, 64 * WNW * WMW, total, 1,
-                        x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream, (float*)nullptr, QkvEpilogue{}, RowScale{});
+                        x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream, (float*)nullptr, QkvEpilogue{}, scale);
 }
 
 template <int TNB, int TMB, int WNW, int WMW, int STAGES>
 static int launch_tile32(const void* X, const void* W, void* C, int M, int N, int K, int ldc, int epi, int packed,
-                         hipStream_t stream) {
+                         hipStream_t stream, int glu) {
     constexpr int BN = 16 * TNB * WNW, BM = 16 * TMB * WMW;
     const int m_tiles = (M + BM - 1) / BM, n_tiles = (N + BN - 1) / BN;
     const long total = (long)m_tiles * n_tiles;
@@ -1294,7 +1370,7 @@ static int launch_tile32(const void* X, const void* W, void* C, int M, int N, in
     const bf16* x = (const bf16*)X;
     const bf16* w = (const bf16*)W;
     const int slices = 1;
-#define EXTRA
+#define EXTRA , glu
     TILE_DISPATCH(gemm_tile32_kernel, TNB, TMB, WNW, WMW, STAGES);
 #undef EXTRA
 }
@@ -1342,6 +1418,18 @@ extern "C" int hb_gemm_qkv_mfma(const void* X, const void* W, int M, int K, int 
 // the number of K slices; tile -1: nothing takes this product with what is asked of it. The flags
 // say whether the input is normed on the way (norm_w), a norm is left behind (emit_g) or a handed-on
 // one is finished (scale_partial).
+// The few-row kernel's estimated time (us). Workgroups of 16 (or 64) weight rows, each streaming at a rate of its
+// own: about 24 KB/us alone on a CU (more if some CUs stay empty), 28 KB/us for a CU with several of 16 rows;
+// more rows cost more reads of the activations. 320 workgroups on 256 CUs take as long as 512.
+static double few_rows_cost(int M, int N, int K, int epi) {
+    const int nb = (epi == EPI_SWIGLU || N >= 16384) ? 4 : 1;
+    const long wgs = (N + 16 * nb - 1) / (16 * nb);
+    const double rounds = wgs <= 256 ? 1 : (wgs <= 512 ? 2 : wgs / 256.0 + 0.5);
+    double rate = (wgs <= 256 || nb == 4 ? 24e3 : 28e3) / (1 + 0.02 * M);
+    if (wgs < 256) rate *= 1 + 0.6 * (256 - wgs) / 256.0;
+    return 3.0 + rounds * 32.0 * nb * K / rate;
+}
+
 struct GemmPlan { int tile, slices; double cost = -1; };      // cost: the estimated time in us where the plan was chosen by one
 static GemmPlan plan_gemm(int M, int N, int K, int ldc, int epi, bool norm_w, bool emit_g, bool scale_partial,
                           int tile_hint, size_t workspace_floats, bool deferred = false) {
@@ -1366,15 +1454,7 @@ static GemmPlan plan_gemm(int M, int N, int K, int ldc, int epi, bool norm_w, bo
         double best = -1;
         bool skinny = false;
         if (M <= 16) {
-            // Workgroups of 16 (or 64) weight rows, each streaming at a rate of its own: about
-            // 24 KB/us alone on a CU (more if some CUs stay empty), 28 KB/us for a CU with several of 16 rows;
-            // more rows cost more reads of the activations. 320 workgroups on 256 CUs take as long as 512.
-            const int nb = (epi == EPI_SWIGLU || N >= 16384) ? 4 : 1;
-            const long wgs = (N + 16 * nb - 1) / (16 * nb);
-            const double rounds = wgs <= 256 ? 1 : (wgs <= 512 ? 2 : wgs / 256.0 + 0.5);
-            double rate = (wgs <= 256 || nb == 4 ? 24e3 : 28e3) / (1 + 0.02 * M);
-            if (wgs < 256) rate *= 1 + 0.6 * (256 - wgs) / 256.0;
-            best = 3.0 + rounds * 32.0 * nb * K / rate;
+            best = few_rows_cost(M, N, K, epi);
             skinny = true;
         }
         if (!norm_w && K % 64 == 0) {
@@ -1525,7 +1605,8 @@ extern "C" double hb_gemm_mfma_plan_cost(int M, int N, int K, int epi, int norme
 }
 
 // C (+)= X @ W^T. X [M, K] bf16, W [N, K] bf16. epi 0: C f32 [M, N] stored; 1: added to;
-// 2: W's rows are gate/up interleaved in blocks of 16 and C is bf16 [M, N / 2] = silu(gate) * up.
+// 2: W's rows are gate/up interleaved in blocks of 16 and C is bf16 [M, N / 2] = silu(gate) * up (glu 0), or
+// max(gate, 0) * up (glu 1).
 // packed != 0: W is stored as [K / 32][N / 16][64 lanes][8]: lane = 16 * (k / 8 % 4) + n % 16.
 // All blocks of one k-step lie together: workgroups that advance through K side by side read one
 // contiguous stretch of memory at a time, as a streaming copy would.
@@ -1537,8 +1618,9 @@ extern "C" int hb_gemm_mfma(const void* X, const void* W, void* C, int M, int N,
                             int packed, const float* norm_w, float eps, int tile_hint, float* workspace,
                             size_t workspace_floats, const float* emit_g, void* emit_xg, float* emit_partial,
                             const float* scale_partial, int scale_parts, float scale_eps, float emit_eps,
-                            int* deferred_slices, hipStream_t stream) {
-    const NormHandoff hand = {emit_g, (bf16*)emit_xg, emit_partial, scale_partial, scale_parts, scale_eps, emit_eps};
+                            int* deferred_slices, int glu, hipStream_t stream) {
+    const NormHandoff hand = {emit_g, (bf16*)emit_xg, emit_partial, scale_partial, scale_parts, scale_eps, emit_eps, glu};
+    HB_REQUIRE(glu == GLU_SILU || (glu == GLU_RELU && epi == EPI_SWIGLU), "gemm_mfma: unknown gated unit %d", glu);
     const bool emit_whole = emit_g && !emit_partial;      // the second kernel of a product cut into slices norms
     HB_REQUIRE(!scale_partial || (M <= 16 && !norm_w), "gemm_mfma: a norm is handed on for at most 16 rows");
     HB_REQUIRE(!emit_g || (epi == EPI_ADD && emit_xg && !norm_w), "gemm_mfma: only the adding product leaves a norm behind");
@@ -1553,7 +1635,7 @@ extern "C" int hb_gemm_mfma(const void* X, const void* W, void* C, int M, int N,
     HB_REQUIRE(K % 32 == 0, "gemm_mfma: K=%d is no multiple of 32", K);
     HB_REQUIRE(epi != EPI_SWIGLU || N % 32 == 0, "gemm_mfma: the SwiGLU epilogue needs N %% 32 == 0");
     HB_REQUIRE(ldc >= (epi == EPI_SWIGLU ? N / 2 : N), "gemm_mfma: output row stride %d too small", ldc);
-    const RowScale row_scale = {scale_partial, scale_parts, scale_eps};
+    const RowScale row_scale = {scale_partial, scale_parts, scale_eps, glu};
     // deferred_slices != null (plain store only): if K is cut into slices, they are left in the
     // workspace [slice][M][N] for the caller's next kernel to add up, and their number is written
     // there; 1 means C holds the product as usual.
@@ -1572,11 +1654,11 @@ extern "C" int hb_gemm_mfma(const void* X, const void* W, void* C, int M, int N,
     if (rows_main > 0) {
         const size_t out_bytes = epi == EPI_SWIGLU ? sizeof(bf16) : sizeof(float);
         const int rc = hb_gemm_mfma(X, W, C, rows_main, N, K, ldc, epi, packed, nullptr, eps, 0, workspace, workspace_floats,
-                                    nullptr, nullptr, nullptr, nullptr, 0, 0.f, 0.f, nullptr, stream);
+                                    nullptr, nullptr, nullptr, nullptr, 0, 0.f, 0.f, nullptr, glu, stream);
         if (rc != 0) return rc;
         return hb_gemm_mfma((const bf16*)X + (size_t)rows_main * K, W, (char*)C + (size_t)rows_main * ldc * out_bytes,
                             M - rows_main, N, K, ldc, epi, packed, nullptr, eps, 0, workspace, workspace_floats, nullptr,
-                            nullptr, nullptr, nullptr, 0, 0.f, 0.f, nullptr, stream);
+                            nullptr, nullptr, nullptr, 0, 0.f, 0.f, nullptr, glu, stream);
     }
     if (plan.tile == 0) {
         pick_skinny(X, W, C, M, N, K, ldc, epi, packed, norm_w, eps, stream, hand);
@@ -1590,18 +1672,18 @@ extern "C" int hb_gemm_mfma(const void* X, const void* W, void* C, int M, int N,
     switch (tile) {
         // (ring depths, measured with weights that come from HBM: a third weight stage gains a
         // tenth for 256 x 128 and nothing for the other two; a third activation stage nothing)
-        case 188: rc = launch_tile64<8, 8, 2, 2, 2, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace); break;   // 256 x 256
-        case 142: rc = launch_tile64<8, 4, 2, 2, 3, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace); break;   // 256 (n) x 128 (m)
-        case 186: rc = launch_tile64<8, 6, 2, 2, 2, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace); break;   // 256 (n) x 192 (m)
-        case 122: rc = launch_tile64<4, 4, 2, 2, 2, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace); break;   // 128 x 128, two to a CU
-        case 124: rc = launch_tile64<2, 4, 4, 1, 3, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace); break;   // 128 (n) x 64 (m)
+        case 188: rc = launch_tile64<8, 8, 2, 2, 2, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace, row_scale); break;   // 256 x 256
+        case 142: rc = launch_tile64<8, 4, 2, 2, 3, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace, row_scale); break;   // 256 (n) x 128 (m)
+        case 186: rc = launch_tile64<8, 6, 2, 2, 2, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace, row_scale); break;   // 256 (n) x 192 (m)
+        case 122: rc = launch_tile64<4, 4, 2, 2, 2, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace, row_scale); break;   // 128 x 128, two to a CU
+        case 124: rc = launch_tile64<2, 4, 4, 1, 3, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace, row_scale); break;   // 128 (n) x 64 (m)
         case 112: rc = launch_tile64<2, 2, 4, 1, 3, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace, row_scale); break;   // 128 (n) x 32 (m)
-        case 184: rc = launch_tile64<4, 4, 4, 1, 3, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace); break;   // 256 (n) x 64 (m)
-        case 168: rc = launch_tile64_swiglu<6, 8, 2, 2, 2, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices); break;   // 192 (n) x 256 (m)
-        case 164: rc = launch_tile64_swiglu<6, 2, 1, 2, 3, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices); break;   // 96 (n) x 64 (m), two waves one above the other
+        case 184: rc = launch_tile64<4, 4, 4, 1, 3, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, workspace, row_scale); break;   // 256 (n) x 64 (m)
+        case 168: rc = launch_tile64_swiglu<6, 8, 2, 2, 2, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, row_scale); break;   // 192 (n) x 256 (m)
+        case 164: rc = launch_tile64_swiglu<6, 2, 1, 2, 3, 2>(X, W, C, M, N, K, ldc, epi, packed, stream, slices, row_scale); break;   // 96 (n) x 64 (m), two waves one above the other
         case 123:                                                                                                           // 128 x 128, K in steps of 32
             HB_REQUIRE(slices == 1, "gemm_mfma: this tile does not cut K");
-            return launch_tile32<4, 4, 2, 2, 4>(X, W, C, M, N, K, ldc, epi, packed, stream);
+            return launch_tile32<4, 4, 2, 2, 4>(X, W, C, M, N, K, ldc, epi, packed, stream, glu);
         default: HB_REQUIRE(false, "gemm_mfma: unknown tile %d", tile);
     }
     if (rc == 0 && slices > 1 && deferred_slices) {
@@ -1620,13 +1702,47 @@ extern "C" int hb_gemm_mfma(const void* X, const void* W, void* C, int M, int N,
             else
                 gemm_slices_norm_kernel<256, 8, 2><<<M, 256, 0, stream>>>(workspace, (float*)C, M, N, ldc, slices, emit_g,
                                                                            emit_eps, (bf16*)emit_xg, emit_partial);
+        else if (epi == EPI_SWIGLU && glu == GLU_RELU)
+            gemm_slices_swiglu_kernel<GLU_RELU><<<(unsigned)((total / 2 + 255) / 256), 256, 0, stream>>>(
+                workspace, (bf16*)C, M, N, ldc, slices);
         else if (epi == EPI_SWIGLU)
-            gemm_slices_swiglu_kernel<<<(unsigned)((total / 2 + 255) / 256), 256, 0, stream>>>(workspace, (bf16*)C, M, N,
-                                                                                             ldc, slices);
+            gemm_slices_swiglu_kernel<GLU_SILU><<<(unsigned)((total / 2 + 255) / 256), 256, 0, stream>>>(
+                workspace, (bf16*)C, M, N, ldc, slices);
         else
             gemm_slices_kernel<<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(workspace, (float*)C, M, N, ldc,
                                                                                   slices, epi == EPI_ADD);
         HB_CHECK_LAUNCH("gemm_slices");
     }
     return rc;
+}
+
+// 1 where the few-row kernel should do such a product and what follows it (TanhJoin) at once: it is estimated to be done
+// sooner than the best plain product and a kernel for the rest (about 3.5 us).
+extern "C" int hb_gemm_mfma_joins(int M, int N, int K, size_t workspace_floats) {
+    if (M > 16 || K % 32 || N % 16) return 0;
+    const GemmPlan p = plan_gemm(M, N, K, N, EPI_STORE, false, false, false, 0, workspace_floats, true);
+    return p.tile == 0 || p.cost < 0 || few_rows_cost(M, N, K, EPI_STORE) <= p.cost + 3.5;
+}
+
+// The product of at most 16 rows with TanhJoin behind it: x [M, N] float32 is the residual stream, y bf16 [M, N] or
+// null; N in steps of 16, every pointer on a 16-byte border.
+extern "C" int hb_gemm_mfma_join(const void* X, const void* W, float* x, int M, int N, int K, int packed, float alpha_after,
+                                 const float* w_after, const float* b_after, const float* extra, const float* step,
+                                 float alpha_before, const float* w_before, const float* b_before, void* y,
+                                 hipStream_t stream) {
+    HB_REQUIRE(M > 0 && M <= 16 && N > 0 && N % 16 == 0 && K > 0 && K % 32 == 0, "gemm_mfma: no joining product of M=%d, N=%d, K=%d", M, N, K);
+    HB_REQUIRE(x && w_after && b_after && (!y || (w_before && b_before)), "gemm_mfma: a joining product needs its norms");
+    HB_REQUIRE((((uintptr_t)x | (uintptr_t)w_after | (uintptr_t)b_after | (uintptr_t)extra | (uintptr_t)step |
+                 (uintptr_t)w_before | (uintptr_t)b_before | (uintptr_t)y) & 15) == 0, "gemm_mfma: a joining product's vectors lie on 16-byte borders");
+    const TanhJoin join = {alpha_after, w_after, b_after, extra, step, alpha_before, w_before, b_before, (bf16*)y};
+    constexpr int WAVES = 8;
+    const dim3 blocks(N / 16);
+    const size_t lds = ((size_t)(WAVES / 2) * 4 * 64 + WAVES * 16) * sizeof(float);
+#define JOIN_GO(PK) gemm_skinny_kernel<1, 1, WAVES, EPI_JOIN, PK, false><<<blocks, WAVES * 64, lds, stream>>>( \
+        X, (const bf16*)W, x, M, N, K, N, nullptr, 0.f, NormHandoff{}, join)
+    if (packed) JOIN_GO(true);
+    else JOIN_GO(false);
+#undef JOIN_GO
+    HB_CHECK_LAUNCH("gemm_join");
+    return 0;
 }

@@ -121,13 +121,13 @@ class Model:
         if self.pass_input is not None and self.pass_input.reads_embedding:
             embedded = rt.buffer("embedding_output", tuple(x.shape), torch.float32)
             ops.tanh_join(x, x_out=embedded)         # (a copy)
+        # what joins x before an entry, where a pass starts there
+        joins = [None if e.starts_pass is None else self.pass_input.rows(e.starts_pass, embedded) for e in self.schedule]
         for i, e in enumerate(self.schedule):
-            if e.starts_pass is not None:
-                joins = self.pass_input.rows(e.starts_pass, embedded)
-                if getattr(self.blocks[e.layer], "takes_pass_input", False):
-                    ctx.pass_input = joins
-                else:
-                    ops.tanh_join(x, extra=joins[0], step=joins[1], x_out=x)
+            ctx.pass_input = joins[i]
+            ctx.next_pass_input = joins[i + 1] if i + 1 < len(joins) else None
+            if ctx.pass_input is not None and not getattr(self.blocks[e.layer], "takes_pass_input", False):
+                ops.tanh_join(x, extra=joins[i][0], step=joins[i][1], x_out=x)
             ctx.entry = i
             ctx.cache_entry = i if e.cache is None else e.cache
             ctx.owns_cache = e.cache is None

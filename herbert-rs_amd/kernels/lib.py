@@ -21,7 +21,7 @@ _SZ = ctypes.c_size_t
 SIGNATURES = {
     "elementwise": {
         "hb_embed": [_P, _P, _I, _P, _I, _I, _I, _I, _F, _P],
-        "hb_tanh_join": [_P, _P, _F, _P, _P, _P, _P, _P, _F, _P, _P, _P, _I, _P, _I, _I, _P],
+        "hb_tanh_join": [_P, _P, _I, _SZ, _F, _P, _P, _P, _P, _P, _F, _P, _P, _P, _I, _P, _I, _I, _P],
         "hb_softcap": [_P, _F, _SZ, _P],
         "hb_rmsnorm": [_P, _P, _P, _I, _P, _I, _I, _F, _P],
         "hb_qk_norm_rope_write": [_P, _I, _P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _P, _P, _P, _I,

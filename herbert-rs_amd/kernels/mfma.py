@@ -19,7 +19,9 @@ _I = ctypes.c_int
 _F = ctypes.c_float
 lib.register_signatures("gemm_mfma", {
     "hb_gemm_mfma": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _F, _I, _P, ctypes.c_size_t, _P, _P, _P, _P, _I, _F,
-                     _F, _P, _P],
+                     _F, _P, _I, _P],
+    "hb_gemm_mfma_joins": [_I, _I, _I, ctypes.c_size_t],
+    "hb_gemm_mfma_join": [_P, _P, _P, _I, _I, _I, _I, _F, _P, _P, _P, _P, _F, _P, _P, _P, _P],
     "hb_gemm_mfma_plan": [_I, _I, _I, _I, _I, _I, _I, ctypes.c_size_t, _I],
     "hb_gemm_mfma_plan_cost": [_I, _I, _I, _I, _I, _I, _I, ctypes.c_size_t, _I],
     "hb_gemm_mfma_split": [_I, _I, _I, _I, ctypes.c_size_t],
@@ -285,10 +287,50 @@ def gemm(a, w, out, accumulate=False, packed=False, norm=None, tile=0, leave=Non
     deferred = ctypes.c_int(1) if defer_slices else None
     lib.call("gemm_mfma", "hb_gemm_mfma", a.data_ptr(), w.data_ptr(), out.data_ptr(), M, N, K, N,
              EPI_ADD if accumulate else EPI_STORE, 1 if packed else 0, norm_ptr, eps, int(tile), ws_ptr,
-             ws_floats, *hand, ctypes.byref(deferred) if defer_slices else None, _stream())
+             ws_floats, *hand, ctypes.byref(deferred) if defer_slices else None, 0, _stream())
     if defer_slices:
         return (deferred.value, ws_ptr, M * N) if deferred.value > 1 else (1, out.data_ptr(), 0)
     return None
+
+
+_joins = {}
+
+
+def joins(M, N, K):
+    """True where `gemm_join` should do a product of these sizes and what follows it at once."""
+    key = (M, N, K)
+    found = _joins.get(key)
+    if found is None:
+        found = _joins[key] = M <= 16 and bool(lib.load("gemm_mfma").hb_gemm_mfma_joins(M, N, K, _slice_workspace_floats(M, N, K)))
+    return found
+
+
+def gemm_join(a, w, x, after, extra=None, step=None, before=None, y=None, packed=False):
+    """ops.tanh_join with part = a bf16 [M, K] @ w bf16 [N, K]^T, M <= 16, in the product's own epilogue: x f32 [M, N] in
+    place, y bf16 [M, N] or None."""
+    M, K = a.shape
+    _check(a, "a", torch.bfloat16, (M, K))
+    _check(w, "w", torch.bfloat16, (None, K))
+    N = w.shape[0]
+    if M > 16 or K % 32 or N % 16:
+        raise BackendError(f"the joining product refuses M={M}, N={N}, K={K}")
+    _check(x, "x", torch.float32, (M, N))
+    alpha_b, w_b, b_b = before if before is not None else (0.0, None, None)
+    if (y is None) != (before is None):
+        raise BackendError("the rows to write come with their norm")
+    for t, name in ((after[1], "weight after"), (after[2], "bias after"), (step, "step"), (w_b, "weight before"), (b_b, "bias before")):
+        if t is not None:
+            _check(t, name, torch.float32, (N,))
+    if extra is not None:
+        _check(extra, "extra", torch.float32, (M, N))
+    if y is not None:
+        _check(y, "y", torch.bfloat16, (M, N))
+        if y.data_ptr() == a.data_ptr():
+            raise BackendError("the joining product's rows to write must be other rows than its input")
+    ptr = lambda t: None if t is None else t.data_ptr()
+    lib.call("gemm_mfma", "hb_gemm_mfma_join", a.data_ptr(), w.data_ptr(), x.data_ptr(), M, N, K, 1 if packed else 0,
+             float(after[0]), after[1].data_ptr(), after[2].data_ptr(), ptr(extra), ptr(step), float(alpha_b), ptr(w_b), ptr(b_b),
+             ptr(y), _stream())
 
 
 QKV_FUSE_MIN_TILES = 136   # of 256 x 256; with fewer (measured: 120 lose, 144 win) the plain product's smaller tiles or K slices fill the CUs better
@@ -369,7 +411,10 @@ def interleave_gate_up(gate, up):
     return torch.stack([gate.view(I // 16, 16, K), up.view(I // 16, 16, K)], 1).reshape(2 * I, K).contiguous()
 
 
-def gemm_swiglu(a, w_interleaved, out, packed=False, norm=None, tile=0, row_scale=None, scratch=None):
+GATED_UNITS = {"silu": 0, "relu": 1}      # what the epilogue of a gate/up product applies to the gate
+
+
+def gemm_swiglu(a, w_interleaved, out, packed=False, norm=None, tile=0, row_scale=None, scratch=None, activation="silu"):
     """out bf16 [M, I] = silu(a @ gate^T) * (a @ up^T), the weights interleaved as above.
     row_scale: see _handoff_args (gate and up are scaled before the activation)."""
     M, K = a.shape
@@ -383,7 +428,7 @@ def gemm_swiglu(a, w_interleaved, out, packed=False, norm=None, tile=0, row_scal
     ws_ptr, ws_floats = _slice_workspace(scratch, a.device, M, N, K, tile)
     lib.call("gemm_mfma", "hb_gemm_mfma", a.data_ptr(), w_interleaved.data_ptr(), out.data_ptr(), M, N, K,
              N // 2, EPI_SWIGLU, 1 if packed else 0, norm_ptr, eps, int(tile), ws_ptr, ws_floats, *hand, None,
-             _stream())
+             GATED_UNITS[activation], _stream())
 
 
 lib.register_signatures("attention_mfma", {

@@ -437,11 +437,13 @@ def softcap(x, cap):
     lib.call("elementwise", "hb_softcap", x.data_ptr(), float(cap), x.numel(), _stream())
 
 
-def tanh_join(x, part=None, after=None, extra=None, step=None, x_out=None, before=None, y=None, rows=None):
+def tanh_join(x, part=None, after=None, extra=None, step=None, x_out=None, before=None, y=None, rows=None, part_slices=None):
     """s = x + n_after(part) + extra + step, row by row; x_out = s (x itself, or other rows); y = n_before(s), with
     n(v) = tanh(alpha v) w + b and after, before = (alpha, w f32 [H], b f32 [H]). x, part, extra, x_out f32 [T, H],
     step f32 [H], y [R, H] in any storage type; each of part, extra, step, x_out, y may be None. rows int32 [R]
-    (y only, no sums): the rows of x that are normed."""
+    (y only, no sums): the rows of x that are normed. part_slices = (slices, pointer, floats between two), as
+    kernels.mfma.gemm(..., defer_slices=True) returns it: part's sums still lie in that many slices (and part itself
+    is not read)."""
     _check(x, "x", torch.float32, (None, None))
     T, H = x.shape
     R = T
@@ -459,6 +461,9 @@ def tanh_join(x, part=None, after=None, extra=None, step=None, x_out=None, befor
         raise BackendError("tanh norm: a part's output and the rows to write come with their norms")
     if x_out is None and y is None:
         raise BackendError("tanh norm: nothing to do")
+    n_slices, part_ptr, stride = part_slices if part_slices is not None else (1, _ptr(part), 0)
+    if part_slices is not None and (part is None or (n_slices > 1 and stride < T * H)):
+        raise BackendError("tanh norm: slices of a part's output that do not hold it")
     alpha_a, w_a, b_a = after if after is not None else (0.0, None, None)
     alpha_b, w_b, b_b = before if before is not None else (0.0, None, None)
     for t, name in ((w_a, "weight after"), (b_a, "bias after"), (w_b, "weight before"), (b_b, "bias before")):
@@ -468,7 +473,7 @@ def tanh_join(x, part=None, after=None, extra=None, step=None, x_out=None, befor
         _check(y, "y", None, (R, H))
         if y.data_ptr() in (x.data_ptr(), None if part is None else part.data_ptr()):
             raise BackendError("tanh norm: the normed rows must be other rows than the sum's")
-    lib.call("elementwise", "hb_tanh_join", x.data_ptr(), _ptr(part), float(alpha_a), _ptr(w_a), _ptr(b_a), _ptr(extra),
+    lib.call("elementwise", "hb_tanh_join", x.data_ptr(), part_ptr, int(n_slices), int(stride), float(alpha_a), _ptr(w_a), _ptr(b_a), _ptr(extra),
              _ptr(step), _ptr(x_out), float(alpha_b), _ptr(w_b), _ptr(b_b), _ptr(y),
              dtype_code(y) if y is not None else F32, _ptr(rows), R, H, _stream())
 

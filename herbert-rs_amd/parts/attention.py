@@ -331,9 +331,7 @@ class Attention(Part):
 
     def project_out(self, ctx, attn, x):
         """x += attn @ Wo^T, the part's last product into the residual stream (or into rows that hold nothing yet)."""
-        adds = ctx.adds_to(x)
-        left = ctx.leave_norm(self.o, x) if adds else None
-        self.o.forward(attn, x, accumulate=adds, leave=None if left is None else left.leave())
+        ctx.project_out(self.o, attn, x)
 
     def forward(self, ctx, y, x, fused_norm=None, row_scale=None):
         if self.prepared:

@@ -143,6 +143,21 @@ class NormedRows:
 
 
 @dataclass
+class TanhJoin:
+    """What a block that norms after its parts does with a part's output p (see kernels.ops.tanh_join):
+    x <- x + n_after(p) + extra + step, y = n_before(x). part: the rows that the part is given for p. `done`: the
+    part's last product has done it."""
+    x: Any
+    part: Any
+    after: Any = None
+    extra: Any = None
+    step: Any = None
+    before: Any = None
+    y: Any = None
+    done: bool = False
+
+
+@dataclass
 class StepContext:
     """What one step hands down to the parts."""
     rt: Runtime
@@ -172,16 +187,31 @@ class StepContext:
     # such block's first norm to add to x (x += factors * delta, a factor a channel)
     pending_scaled: Any = None
 
-    # (x's address, rows, norm): a block that norms after its parts has left its last part's output, and the norm
-    # that it passes, for the next such block's first kernel to add to x
-    pending_join: Any = None
+    # set by a block that norms after its parts, for the part that runs: a TanhJoin that the part's last product may do
+    join: Any = None
+    # (x's address, entry, rows): such a block has left, for that entry's block of the same kind, the normed rows that its
+    # mixer reads
+    ready_rows: Any = None
     # set by the model where a pass over a stretch of the schedule starts, for a block that takes it: (rows f32
-    # [T, hidden] or None, vector f32 [hidden] or None) to be added to x before the block's first norm
+    # [T, hidden] or None, vector f32 [hidden] or None) to be added to x before the block's first norm; and the same
+    # for the next entry's block, which the block before may add
     pass_input: Any = None
+    next_pass_input: Any = None
 
     def adds_to(self, x):
         """False if x are the context's fresh rows (the part's product stores), True if it has to add."""
         return not (self.fresh_rows is not None and self.fresh_rows.data_ptr() == x.data_ptr())
+
+    def project_out(self, linear, a, x):
+        """A part's last product, a @ W^T, into x: added to it, stored where x holds nothing yet, or taken on to where a
+        block wants it (see `join`); a norm that follows a sum is prepared if that can be done."""
+        adds = self.adds_to(x)
+        if self.join is not None and not adds and x.data_ptr() == self.join.part.data_ptr():
+            linear.forward_join(a, x, self.join)
+            self.join.done = True
+            return
+        left = self.leave_norm(linear, x) if adds else None
+        linear.forward(a, x, accumulate=adds, leave=None if left is None else left.leave())
 
     def leave_norm(self, linear, x):
         """For a part, just before `linear` adds its last product into x: a NormedRows that product

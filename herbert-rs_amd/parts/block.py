@@ -21,7 +21,7 @@ import torch
 
 from ..kernels import ops
 from ..weights import TensorNeed
-from .base import Part
+from .base import Part, TanhJoin
 from .registry import build, register
 
 
@@ -272,10 +272,10 @@ class PostNormBlock(Part):
 @register("block", "sandwich")
 class SandwichBlock(Part):
     """x <- x + after_mixer(mixer(before_mixer(x))), then x <- x + after_ff(feed_forward(before_ff(x))) (the second
-    step only where the layer has a feed-forward). The parts store their outputs in float32 rows of their own; one
-    kernel between two parts norms those rows, adds them to x and writes the normed copy of x that the next part
-    reads. A layer's last sum is left for the next layer's first kernel, if that layer is such a block too,
-    and what joins x where a pass over the layers starts is added there as well."""
+    step only where the layer has a feed-forward). Between two products of such layers stand a norm of a part's
+    output, a sum and the norm that the next part reads, the next layer's first one included (with what joins x
+    where a pass over the layers starts): the part's last product does all of it in its epilogue where it can
+    (StepContext.join), else one kernel does, from float32 rows that hold the part's output."""
     graph_safe = True
     takes_pass_input = True
 
@@ -301,36 +301,41 @@ class SandwichBlock(Part):
 
     def forward(self, ctx, x):
         rt = ctx.rt
-        shape = tuple(x.shape)
-        branch = rt.buffer("sandwich_branch", shape, torch.float32)
-        y = rt.buffer("sandwich_rows", shape)
-        pending, ctx.pending_join = ctx.pending_join, None
-        extra, step = ctx.pass_input if ctx.pass_input is not None else (None, None)
-        ctx.pass_input = None
-        part_rows = after = None
-        if pending is not None and pending[0] == x.data_ptr():
-            part_rows, after = pending[1], pending[2].constants()
-        changed = part_rows is not None or extra is not None or step is not None
-        ops.tanh_join(x, part_rows, after, extra, step, x if changed else None, self.norms["before_mixer"].constants(), y)
-        self._run(ctx, self.mixer, y, branch)
-        last = self.norms["after_mixer"]
-        if self.feed_forward is not None:
-            ops.tanh_join(x, branch, last.constants(), x_out=x, before=self.norms["before_ff"].constants(), y=y)
-            self._run(ctx, self.feed_forward, y, branch)
-            last = self.norms["after_ff"]
-        if isinstance(ctx.next_block, SandwichBlock):
-            ctx.pending_join = (x.data_ptr(), branch, last)
+        branch = rt.buffer("sandwich_branch", tuple(x.shape), torch.float32)
+        y = rt.buffer("sandwich_rows", tuple(x.shape))
+        ready, ctx.ready_rows = ctx.ready_rows, None
+        joins, ctx.pass_input = ctx.pass_input, None
+        if ready is None or ready != (x.data_ptr(), ctx.entry, y.data_ptr()):
+            extra, step = joins if joins is not None else (None, None)
+            changed = extra is not None or step is not None
+            ops.tanh_join(x, extra=extra, step=step, x_out=x if changed else None, before=self.norms["before_mixer"].constants(), y=y)
+        nxt = ctx.next_block if isinstance(ctx.next_block, SandwichBlock) else None
+        last = TanhJoin(x, branch)
+        if nxt is not None:
+            last.before, last.y = nxt.norms["before_mixer"].constants(), y
+            if ctx.next_pass_input is not None:
+                last.extra, last.step = ctx.next_pass_input
+        if self.feed_forward is None:
+            last.after = self.norms["after_mixer"].constants()
+            self._run(ctx, self.mixer, y, branch, last)
         else:
-            ops.tanh_join(x, branch, last.constants(), x_out=x)
+            self._run(ctx, self.mixer, y, branch, TanhJoin(x, branch, self.norms["after_mixer"].constants(),
+                                                           before=self.norms["before_ff"].constants(), y=y))
+            last.after = self.norms["after_ff"].constants()
+            self._run(ctx, self.feed_forward, y, branch, last)
+        if nxt is not None:
+            ctx.ready_rows = (x.data_ptr(), ctx.entry + 1, y.data_ptr())
 
     @staticmethod
-    def _run(ctx, part, y, branch):
+    def _run(ctx, part, y, branch, join):
         ctx.handed = ctx.norm_ahead = ctx.left = None
-        # a part that can store its rows instead of adding them says so and finds the rows in ctx.fresh_rows;
-        # for any other the rows are cleared first
+        # a part that can store its rows instead of adding them says so and finds the rows in ctx.fresh_rows (and may do
+        # what follows it at once); for any other the rows are cleared first
         if getattr(part, "stores_fresh_rows", False):
-            ctx.fresh_rows = branch
+            ctx.fresh_rows, ctx.join = branch, join
         else:
             ops.fill_u32(branch, 0)
         part.forward(ctx, y, branch)
-        ctx.fresh_rows = None
+        ctx.fresh_rows = ctx.join = None
+        if not join.done:
+            ops.tanh_join(join.x, branch, join.after, join.extra, join.step, join.x, join.before, join.y)

@@ -176,6 +176,4 @@ class LatentAttention(Part):
             gated = rt.buffer("latent_gated", (T, H * self.vdim))
             ops.gate_heads(attn, proj, self.q_width + self.row, gated, H, self.vdim, self.vdim)
             attn = gated
-        adds = ctx.adds_to(x)
-        left = ctx.leave_norm(self.o, x) if adds else None
-        self.o.forward(attn, x, accumulate=adds, leave=None if left is None else left.leave())
+        ctx.project_out(self.o, attn, x)

@@ -56,10 +56,21 @@ class Linear:
         """Rows of the sums of squares that go with a handed-on norm of that many rows."""
         return mfma.padded_rows(rows)
 
-    def forward_swiglu(self, a, out, norm=None, row_scale=None):
-        """out bf16 [M, N / 2] = silu(gate) * up for a weight whose rows are gate/up interleaved."""
+    def forward_join(self, a, part, join):
+        """The product a @ W^T as a part's output that passes a norm and joins the residual stream (`join`, a
+        parts.base.TanhJoin): in the product's epilogue where few rows allow it, else into `part` (f32 [M, N], or the
+        slices of K that the product leaves) and from there by a kernel of its own."""
+        bf16 = self.weight.dtype == torch.bfloat16 and a.dtype == torch.bfloat16
+        if bf16 and mfma.joins(a.shape[0], self.out_features, self.in_features):
+            mfma.gemm_join(a, self.weight, join.x, join.after, join.extra, join.step, join.before, join.y, packed=self.packed)
+            return
+        slices = self.forward(a, part, defer_slices=True)
+        ops.tanh_join(join.x, part, join.after, join.extra, join.step, join.x, join.before, join.y, part_slices=slices)
+
+    def forward_swiglu(self, a, out, norm=None, row_scale=None, activation="silu"):
+        """out bf16 [M, N / 2] = f(gate) * up for a weight whose rows are gate/up interleaved, f silu or relu."""
         mfma.gemm_swiglu(a, self.weight, out, packed=self.packed, norm=norm, row_scale=row_scale,
-                         scratch=self.scratch)
+                         scratch=self.scratch, activation=activation)
 
     def fuses_norm(self, x):
         """True if RMSNorm(x) @ W^T runs as one kernel for this input (few rows, bfloat16 weights)."""

@@ -40,8 +40,8 @@ class SwiGLU(Part):
         n = self.names
         gate, up = rt.weight(tensors[n["gate"]]), rt.weight(tensors[n["up"]])
         # bfloat16 with sizes the MFMA kernel takes: gate and up rows interleaved so that the
-        # product's epilogue applies silu(gate) * up and the float32 [T, 2I] never exists
-        self.fused_epilogue = (self.activation == "silu" and rt.dtype == torch.bfloat16 and self.intermediate_size % 16 == 0
+        # product's epilogue applies f(gate) * up and the float32 [T, 2I] never exists
+        self.fused_epilogue = (self.activation in mfma.GATED_UNITS and rt.dtype == torch.bfloat16 and self.intermediate_size % 16 == 0
                                and self.hidden_size % 32 == 0 and mfma.gemm_supported(
                                    gate[:1], gate, swiglu=True))
         if self.fused_epilogue:
@@ -69,16 +69,14 @@ class SwiGLU(Part):
         T = x.shape[0]
         act = rt.buffer("act", (T, self.intermediate_size))
         if fused_norm is not None:
-            self.gate_up.forward_swiglu(x, act, norm=(fused_norm.w, fused_norm.eps))
+            self.gate_up.forward_swiglu(x, act, norm=(fused_norm.w, fused_norm.eps), activation=self.activation)
         elif self.fused_epilogue:
-            self.gate_up.forward_swiglu(y, act, row_scale=row_scale)
+            self.gate_up.forward_swiglu(y, act, row_scale=row_scale, activation=self.activation)
         else:
             gu = rt.buffer("gate_up", (T, 2 * self.intermediate_size), torch.float32)
             self.gate_up.forward(y, gu)
             ops.swiglu(gu, act, self.activation)
-        adds = ctx.adds_to(x)
-        left = ctx.leave_norm(self.down, x) if adds else None
-        self.down.forward(act, x, accumulate=adds, leave=None if left is None else left.leave())
+        ctx.project_out(self.down, act, x)
 
 
 @register("feed_forward", "squared_relu")

@@ -65,6 +65,48 @@ def test_tanh_norm_and_the_sums_beside_it(T, H, dtype):
     assert torch.allclose(y.float().cpu(), plain.dynamic_tanh(x[[T - 1, 0, T // 2]], 1.7, wb, bb), atol=tol, rtol=tol)
 
 
+@pytest.mark.parametrize("H", [64, 72, 101])
+@pytest.mark.parametrize("slices", [2, 4, 8])
+def test_tanh_norm_of_a_product_in_slices(slices, H):
+    T = 6
+    x, parts = rand(T, H, seed=1), rand(slices, T, H, seed=2)
+    wa, ba, wb, bb = 1 + 0.2 * rand(H, seed=5), 0.3 * rand(H, seed=6), 1 + 0.2 * rand(H, seed=7), 0.3 * rand(H, seed=8)
+    want = x + plain.dynamic_tanh(parts.sum(0), 0.8, wa, ba)
+    xg, y, held = g(x.clone()), torch.empty(T, H, device=DEV), g(parts)
+    ops.tanh_join(xg, torch.full((T, H), float("nan"), device=DEV), (0.8, g(wa), g(ba)), x_out=xg, before=(1.7, g(wb), g(bb)), y=y,
+                  part_slices=(slices, held.data_ptr(), T * H))
+    assert torch.allclose(xg.cpu(), want, atol=5e-6)
+    assert torch.allclose(y.cpu(), plain.dynamic_tanh(want, 1.7, wb, bb), atol=1e-5)
+
+
+@pytest.mark.parametrize("M,N,K", [(1, 64, 32), (8, 256, 128), (16, 48, 320), (5, 2048, 2048), (3, 1024, 4096), (16, 16, 64), (17, 256, 512), (64, 512, 1024),
+                                   (300, 128, 64)])
+def test_a_product_that_joins_the_stream(M, N, K):
+    """Through Linear, as the parts do it: few rows in the product's epilogue, more by way of rows or slices of K."""
+    a, w = rand(M, K, seed=1).bfloat16(), rand(N, K, seed=2, scale=K ** -0.5).bfloat16()
+    x, extra, step = rand(M, N, seed=3), rand(M, N, seed=4), rand(N, seed=5)
+    wa, ba, wb, bb = 1 + 0.2 * rand(N, seed=6), 0.3 * rand(N, seed=7), 1 + 0.2 * rand(N, seed=8), 0.3 * rand(N, seed=9)
+    p = (a.double() @ w.double().T).float()
+    linear = Linear(g(w))
+    from herbert_rs_amd.parts.base import TanhJoin
+    for use in range(4):
+        e, s = (extra if use & 1 else None), (step if use & 2 else None)
+        want = x + plain.dynamic_tanh(p, 0.9, wa, ba) + (e if e is not None else 0) + (s if s is not None else 0)
+        for with_y in (True, False):
+            calls = [lambda xg, y, rows: linear.forward_join(g(a), rows, TanhJoin(xg, rows, (0.9, g(wa), g(ba)), g(e), g(s),
+                                                                                 (1.3, g(wb), g(bb)) if with_y else None, y))]
+            if M <= 16:                                          # and by name, whatever the estimate prefers
+                calls.append(lambda xg, y, rows: mfma.gemm_join(g(a), linear.weight, xg, (0.9, g(wa), g(ba)), g(e), g(s),
+                                                                (1.3, g(wb), g(bb)) if with_y else None, y, packed=linear.packed))
+            for call in calls:
+                xg, rows = g(x.clone()), torch.empty(M, N, device=DEV)
+                y = torch.full((M, N), 9.0, dtype=torch.bfloat16, device=DEV) if with_y else None
+                call(xg, y, rows)
+                assert torch.allclose(xg.cpu(), want, atol=2e-5), f"use {use}"
+                if with_y:
+                    assert torch.allclose(y.float().cpu(), plain.dynamic_tanh(want, 1.3, wb, bb), atol=2 ** -7, rtol=2 ** -8)
+
+
 def test_tanh_norm_far_outside_its_bend():
     x = torch.tensor([[-1e30, -50.0, 0.0, 50.0, 1e30, 1e-20, -0.0, 3.0]])
     y = torch.empty(1, 8, device=DEV)
