@@ -286,7 +286,7 @@ def drawn_configuration(seed):
             kv = r.choice([1, 2, 4])
             dim, vdim = r.choice([24, 32, 48, 64, 80, 128, 160]), r.choice([16, 40, 64, 80, 128, 144])
             layers.append(attention(kv * r.choice([1, 2, 3]), kv, dim, vdim, r.choice([0.5, 1.0, 2.0]) * dim ** -0.5,
-                                    r.choice([40, 90, 240, 1000]), r.choice([None, 1, 5, 32, 50, 64, 129, 200]), r.choice([0, 1, 4, 64, 130]), mlp))
+                                    r.choice([40, 90, 260, 1000]), r.choice([None, 1, 5, 32, 50, 64, 129, 200]), r.choice([0, 1, 4, 64, 130]), mlp))
         else:
             dim, rank, q_rank = r.choice([16, 24, 32, 64]), r.choice([24, 32, 64, 96, 256]), r.choice([16, 32, 72, 128])
             args = (r.choice([16, 24, 32, 64]), rank, q_rank)

@@ -204,7 +204,7 @@ ATTENTION_CASES = [
     (4, 2, 64, 32, 200, 100, 5),
     (8, 2, 128, 16, 90, 64, 70),
     (3, 3, 32, 8, 40, 7, 2),
-    (6, 2, 96, 32, 240, None, 0),
+    (6, 2, 96, 32, 250, None, 0),
     (2, 1, 160, 12, 60, 50, 3),
     (40, 2, 32, 2, 9, 129, 1),
     (4, 4, 48, 64, 2000, 64, 64),
