@@ -8,6 +8,7 @@ from .modasun import ModasunConfig
 from .mefatar import MefatarConfig
 from .bozasun import BozasunConfig
 from .mutedra import MutedraConfig
+from .figalorn import FigalornConfig
 
-__all__ = ["Architecture", "BozasunConfig", "ChatFormat", "MefatarConfig", "ModasunConfig", "MutedraConfig", "Qwen3Config", "VipalornConfig", "load_config", "read_config_json",
+__all__ = ["Architecture", "BozasunConfig", "ChatFormat", "FigalornConfig", "MefatarConfig", "ModasunConfig", "MutedraConfig", "Qwen3Config", "VipalornConfig", "load_config", "read_config_json",
            "register_architecture", "registered_architectures", "resolve_architecture"]

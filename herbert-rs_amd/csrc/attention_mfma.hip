@@ -792,7 +792,50 @@ struct DecodeFusion {
     int q_temp_every;
 };
 
-template <int HD, bool FUSED, bool EXT, int QS = 1>
+// The second fused form of the decode kernel (FORM_HEADS): the rows of a projection whose heads are not kept as they are
+// projected (the layout of heads.hip: nq query heads of dim columns, then keys and values where k_off and v_off say;
+// biases, a norm a head or map, a rotation of rot_dims entries in either layout by the step's angles, two maps side by
+// side in a kept head, values that are the keys before their norm). One wave works them out through LDS.
+#define FORM_PLAIN 0
+#define FORM_FUSED 1
+#define FORM_HEADS 2
+struct HeadsFusion {
+    const float* proj;
+    int ld;
+    size_t slice_stride;         // of the projection's QS slices of K
+    const float* bias;           // a channel; null: none
+    const float* q_norm_w;       // [dim]; null: no norm
+    const float* k_norm_w;
+    const float2* angles;        // [sequences, rot_dims / 2]: cosine and sine
+    int rot_dims, halves;
+    int maps, dim, vdim, map_stride, k_off, v_off;
+    float eps;
+};
+
+// How the heads' outputs leave (own: at their own size vdim, a row [heads x vdim]; else at the kept size): with two maps
+// neighbouring query heads are a head's maps, o = a1 - lambda a2, over its root mean square, times factor; then times
+// sigmoid of the gate's column (null: none), which may lie in slices of K still.
+struct HeadsOut {
+    int own, maps, vdim;
+    const float* gate;
+    int gate_ld, gate_slices;
+    size_t gate_stride;
+    float lambda, factor, eps;
+};
+
+__device__ __forceinline__ float gate_of(const HeadsOut& ho, size_t row, int column) {
+    if (!ho.gate) return 1.0f;
+    const float* const p = ho.gate + row * ho.gate_ld + column;
+    float part[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) part[i] = i < ho.gate_slices ? p[(size_t)i * ho.gate_stride] : 0.f;
+    float g = part[0];
+#pragma unroll
+    for (int i = 1; i < 8; ++i) g += part[i];
+    return 1.0f / (1.0f + expf(-g));
+}
+
+template <int HD, int FUSED, bool EXT, int QS = 1>
 __global__ void __launch_bounds__(64)
 attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16* __restrict__ v_cache,
                    float* __restrict__ partial_o, float* __restrict__ partial_ml,
@@ -800,7 +843,7 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
                    const int* __restrict__ page_table, int max_pages, int nq, int nkv, float c, int window,
                    int pages_per_split, DecodeFusion fu, bf16* __restrict__ out,
                    const int* __restrict__ ranges, int n_seqs, const float* __restrict__ sinks, int chunked,
-                   float cap, AttnExtras ext) {
+                   float cap, AttnExtras ext, HeadsFusion hf, HeadsOut ho) {
     // ranges == null: the grid is (sequence, kv head, range), every sequence cut into gridDim.z
     // ranges of pages_per_split pages (those past a sequence's end hold nothing).
     // ranges != null (sequences of unequal lengths): the grid is (1, kv head, item);
@@ -841,7 +884,7 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
     // k of the MFMA steps: step s, lane group g2, element j  <->  d = g2 * HD/2 + s * 8 + j,
     // so a lane reads one contiguous half row of K
     bf16x8 qreg[HD / 16];
-    if (!FUSED) {
+    if (FUSED == FORM_PLAIN) {
         const bf16* qrow = q + ((size_t)b * nq + head) * HD + g2 * HALF;
 #pragma unroll
         for (int s = 0; s < HD / 16; ++s) qreg[s] = *(const bf16x8*)(qrow + s * 8);
@@ -853,12 +896,49 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
     constexpr int PER = 64 / HALF;                 // heads a round of the wave covers
     constexpr int PRE = 4;                         // rounds whose inputs are loaded ahead
     const int j = lane % HALF, sub = lane / HALF;
-    const bool writer = FUSED && fu.write_kv && hp >= first_page && hp < first_page + pages_per_split;
+    const bool writer = FUSED != FORM_PLAIN && (FUSED == FORM_HEADS || fu.write_kv) && hp >= first_page && hp < first_page + pages_per_split;
     float cs = 1.f, sn = 0.f, qw0 = 1.f, qw1 = 1.f, kw0 = 1.f, kw1 = 1.f;
     float xq0[PRE], xq1[PRE], k0 = 0.f, k1 = 0.f, v0 = 0.f, v1 = 0.f;
     int new_page = 0;
     const float* qin = nullptr;
-    if (FUSED) {
+    // FORM_HEADS: a lane holds the entries lane (and lane + 64) of a row of the projection
+    constexpr int E = HD > 64 ? HD / 64 : 1;
+    float hq[PRE][E], hk[E], hv[E], hqw[E], hkw[E];
+    float2 turn = {1.f, 0.f};
+    const float* hrow = nullptr;
+    auto channel = [&](int at) {
+        float part[QS];
+#pragma unroll
+        for (int i = 0; i < QS; ++i) part[i] = hrow[(size_t)i * hf.slice_stride + at];
+        float sum = part[0];
+#pragma unroll
+        for (int i = 1; i < QS; ++i) sum += part[i];
+        return hf.bias ? sum + hf.bias[at] : sum;
+    };
+    if (FUSED == FORM_HEADS) {
+        hrow = hf.proj + (size_t)b * hf.ld;
+        if (lane < hf.rot_dims / 2) turn = hf.angles[(size_t)b * (hf.rot_dims / 2) + lane];
+#pragma unroll
+        for (int e = 0; e < E; ++e) {
+            const int d = lane + 64 * e;
+            hqw[e] = hkw[e] = 1.f;
+            hk[e] = hv[e] = 0.f;
+            if (hf.q_norm_w && d < hf.dim) {
+                hqw[e] = hf.q_norm_w[d];
+                hkw[e] = hf.k_norm_w[d];
+            }
+#pragma unroll
+            for (int it = 0; it < PRE; ++it)
+                hq[it][e] = d < hf.dim ? channel((kvh * G + (it < G ? it : G - 1)) * hf.dim + d) : 0.f;
+            if (writer) {
+                if (d < hf.maps * hf.dim) hk[e] = channel(hf.k_off + kvh * hf.maps * hf.dim + d);
+                if (hf.v_off == hf.k_off) hv[e] = hk[e];
+                else if (d < hf.vdim) hv[e] = channel(hf.v_off + kvh * hf.vdim + d);
+            }
+        }
+        if (writer) new_page = pt[page_at(hp)];
+    }
+    if (FUSED == FORM_FUSED) {
         const float* row = fu.qkv + (size_t)b * (nq + 2 * nkv) * HD;
         qin = row + (size_t)kvh * G * HD;
         if (fu.cos_t) {
@@ -950,10 +1030,107 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
                 _Pragma("unroll") for (int h2 = 0; h2 < 2; ++h2)                             \
                     va[d][kb][h2] = *(const bf16x8*)(vp + (size_t)(d * 32 + c32) * PAGE + kb * 32 + h2 * 16); \
     }
-    __shared__ __attribute__((aligned(16))) bf16 qs[FUSED ? 32 * HD : 8];
+    __shared__ __attribute__((aligned(16))) bf16 qs[FUSED != FORM_PLAIN ? 32 * HD : 8];
+    // (FORM_HEADS: a row of the projection normed, and the angles)
+    __shared__ float hraw[FUSED == FORM_HEADS ? (PRE + 1) * HD : 1];
+    __shared__ float2 hturn[FUSED == FORM_HEADS ? HD / 2 : 1];
+    auto heads_prologue = [&]() {
+        if (lane < HD / 2) hturn[lane] = turn;
+        // a row's entries times their norm into LDS; of a key with two maps each has a norm of its own
+        auto lay = [&](float (&x)[E], float (&w)[E], float* raw, int maps) {
+            float inv0 = 1.f, inv1 = 1.f;
+            if (hf.q_norm_w) {
+                float s0 = 0.f, s1 = 0.f;
+#pragma unroll
+                for (int e = 0; e < E; ++e) {
+                    const int d = lane + 64 * e;
+                    if (d < hf.dim) s0 = fmaf(x[e], x[e], s0);
+                    else s1 = fmaf(x[e], x[e], s1);
+                }
+#pragma unroll
+                for (int off = 32; off > 0; off >>= 1) {
+                    s0 += __shfl_xor(s0, off, 64);
+                    s1 += __shfl_xor(s1, off, 64);
+                }
+                inv0 = 1.0f / sqrtf(s0 / (float)hf.dim + hf.eps);
+                inv1 = 1.0f / sqrtf(s1 / (float)hf.dim + hf.eps);
+            }
+#pragma unroll
+            for (int e = 0; e < E; ++e) {
+                const int d = lane + 64 * e;
+                // (the second map's weights lie dim entries on: read again, a rare case)
+                const float wd = d < hf.dim || maps == 1 || !hf.q_norm_w ? w[e] : d < maps * hf.dim ? hf.k_norm_w[d - hf.dim] : 1.f;
+                if (d < HD) raw[d] = x[e] * (d < hf.dim ? inv0 : inv1) * wd;
+            }
+        };
+        // entry d of the kept head; map < 0: a key, all maps
+        auto kept = [&](const float* raw, int d, int map) -> float {
+            const int m = hf.maps == 2 && d >= hf.map_stride ? 1 : 0;
+            const int e = d - m * hf.map_stride;
+            if (e >= hf.dim || (map >= 0 && m != map)) return 0.f;
+            const float* const r = raw + (map >= 0 ? 0 : m * hf.dim);
+            const float own = r[e];
+            if (e >= hf.rot_dims) return own;
+            const int half = hf.rot_dims / 2;
+            const bool second = hf.halves ? e >= half : (e & 1);
+            const int i = hf.halves ? (second ? e - half : e) : e >> 1;
+            const int other = hf.halves ? (second ? e - half : e + half) : e ^ 1;
+            const float2 t = hturn[i];
+            return second ? own * t.x + r[other] * t.y : own * t.x - r[other] * t.y;
+        };
+        if (writer) lay(hk, hkw, hraw + PRE * HD, hf.maps);
+#pragma unroll
+        for (int it = 0; it < PRE; ++it) lay(hq[it], hqw, hraw + it * HD, 1);
+        __syncthreads();
+        if (writer) {
+            const int in_page = hi % PAGE;
+            bf16* const kdst = k_cache + (((size_t)new_page * nkv + kvh) * PAGE + in_page) * HD;
+            bf16* const vdst = v_cache + ((size_t)new_page * nkv + kvh) * HD * PAGE + in_page;
+#pragma unroll
+            for (int e = 0; e < E; ++e) {
+                const int d = lane + 64 * e;
+                if (d < HD) {
+                    kdst[d] = hb_from_float<bf16>(kept(hraw + PRE * HD, d, -1));
+                    vdst[(size_t)d * PAGE] = hb_from_float<bf16>(d < hf.vdim ? hv[e] : 0.f);
+                }
+            }
+            __threadfence_block();      // this wave's later loads of that page see what it has just written
+        }
+        for (int it0 = 0; it0 < G; it0 += PRE) {
+            if (it0 > 0) {
+                __syncthreads();
+#pragma unroll
+                for (int it = 0; it < PRE; ++it) {
+                    const int hl = it0 + it < G ? it0 + it : G - 1;
+#pragma unroll
+                    for (int e = 0; e < E; ++e) {
+                        const int d = lane + 64 * e;
+                        hq[it][e] = d < hf.dim ? channel((kvh * G + hl) * hf.dim + d) : 0.f;
+                    }
+                }
+#pragma unroll
+                for (int it = 0; it < PRE; ++it) lay(hq[it], hqw, hraw + it * HD, 1);
+                __syncthreads();
+            }
+#pragma unroll
+            for (int it = 0; it < PRE; ++it) {
+                const int hl = it0 + it;
+                if (hl >= G) break;
+#pragma unroll
+                for (int e = 0; e < E; ++e) {
+                    const int d = lane + 64 * e;
+                    if (d < HD) qs[hl * HD + d] = hb_from_float<bf16>(kept(hraw + it * HD, d, hf.maps == 2 ? (hl & 1) : 0));
+                }
+            }
+        }
+    };
     // norm and rotation of the new key and of the query heads; the key and the value go to the pages,
     // the queries to LDS, from where each lane takes its operand
     auto prologue = [&]() {
+        if (FUSED == FORM_HEADS) {
+            heads_prologue();
+            return;
+        }
         if (writer) {
             float ss = k0 * k0 + k1 * k1;
 #pragma unroll
@@ -1011,7 +1188,7 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
     // The first page's operands go out before that work, so that it hides their way from memory,
     // unless this wave has yet to write the new key into that very page. (Two copies of the code:
     // each then knows how many loads are in flight behind the small ones it waits for.)
-    if (!FUSED) {
+    if (FUSED == FORM_PLAIN) {
         if (first_page <= last_page) {
             LOAD_K(first_page)
             LOAD_V(first_page)
@@ -1027,7 +1204,7 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
             LOAD_V(first_page)
         }
     }
-    if (FUSED) {
+    if (FUSED != FORM_PLAIN) {
         __syncthreads();
         const bf16* qrow = qs + (c32 < G ? c32 : G - 1) * HD + g2 * HALF;
 #pragma unroll
@@ -1068,6 +1245,39 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
 #undef LOAD_K
 #undef LOAD_V
     l += __shfl_xor(l, 32, 64);
+    if (FUSED == FORM_HEADS && out && ho.own) {
+        // one range a sequence, the heads leave at their own size (see HeadsOut): maps are neighbouring lanes
+        if (sinks) l += sink_share(sinks[head], m, c);
+        const float inv = l > 0.f ? 1.0f / l : 0.f;
+        float scale = 1.f;
+        if (ho.maps == 2) {
+            float ss = 0.f;
+#pragma unroll
+            for (int d = 0; d < HD / 32; ++d)
+#pragma unroll
+                for (int i = 0; i < 16; ++i) {
+                    const float a = oacc[d][i] * inv;
+                    oacc[d][i] = a - ho.lambda * __shfl_xor(a, 1, 64);
+                    ss = fmaf(oacc[d][i], oacc[d][i], ss);
+                }
+            ss += __shfl_xor(ss, 32, 64);
+            scale = ho.factor / sqrtf(ss / (float)ho.vdim + ho.eps);
+        } else {
+            scale = inv;
+        }
+        const int own_head = (kvh * G + c32) / ho.maps;
+        if (c32 < G && (ho.maps == 1 || (c32 & 1) == 0)) {
+            bf16* const dst = out + ((size_t)b * (nq / ho.maps) + own_head) * ho.vdim;
+#pragma unroll
+            for (int d = 0; d < HD / 32; ++d)
+#pragma unroll
+                for (int i = 0; i < 16; ++i) {
+                    const int at = d * 32 + 8 * (i >> 2) + 4 * g2 + (i & 3);
+                    if (at < ho.vdim) dst[at] = hb_from_float<bf16>(oacc[d][i] * scale * gate_of(ho, b, own_head * ho.vdim + at));
+                }
+        }
+        return;
+    }
     if (out) {
         // one range a sequence: nothing to merge, the output is O / l (zeros if no key was visible)
         if (c32 < G) {
@@ -1174,6 +1384,81 @@ attn_decode_merge_kernel(const float* __restrict__ partial_o, const float* __res
         for (int g = 0; g < GROUPS; ++g) total += sums[g][tid];
         out[bh * HD + tid] = hb_from_float<bf16>(total * s_inv);
     }
+}
+
+// The same where the heads leave at their own size (HeadsOut, FORM_HEADS): a workgroup a (sequence, head of the model), 256
+// threads a map of the head.
+template <int HD>
+__global__ void __launch_bounds__(512)
+attn_decode_merge_own_kernel(const float* __restrict__ partial_o, const float* __restrict__ partial_ml, bf16* __restrict__ out,
+                             int splits, float c, const int* __restrict__ ranges, int nq, const float* __restrict__ sinks,
+                             HeadsOut ho) {
+    constexpr int CHUNKS = HD / 4;
+    constexpr int GROUPS = 256 / CHUNKS;
+    __shared__ float wgt[2][1024];
+    __shared__ float sums[2][GROUPS][HD];
+    __shared__ float s_inv[2];
+    __shared__ float red[8];
+    const int map = threadIdx.x / 256, tid = threadIdx.x % 256;
+    const int heads = nq / ho.maps;
+    const int b = blockIdx.x / heads, own_head = blockIdx.x % heads;
+    const int h = own_head * ho.maps + map;
+    const int chunk = tid % CHUNKS, grp = tid / CHUNKS;
+    size_t first = ((size_t)b * nq + h) * splits;
+    if (ranges) {
+        first = (size_t)h * splits + ranges[b];
+        splits = ranges[b + 1] - ranges[b];
+    }
+    const float* const ml = partial_ml + first * 2;
+    // (asked for early: used last)
+    const float gate = map == 0 && tid < ho.vdim ? gate_of(ho, b, own_head * ho.vdim + tid) : 1.f;
+    if (tid < 64) {
+        float M = -INFINITY;
+        for (int s = tid; s < splits; s += 64) M = fmaxf(M, ml[2 * s]);
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) M = fmaxf(M, __shfl_xor(M, off, 64));
+        float denom = 0.f;
+        for (int s0 = 0; s0 < splits; s0 += 64) {
+            const int s = s0 + tid;
+            float w = 0.f, term = 0.f;
+            if (s < splits && ml[2 * s] != -INFINITY) {
+                w = fast_exp2((ml[2 * s] - M) * c);
+                term = w * ml[2 * s + 1];
+            }
+            if (s < splits) wgt[map][s] = w;
+#pragma unroll
+            for (int off = 32; off > 0; off >>= 1) term += __shfl_xor(term, off, 64);
+            denom += term;
+        }
+        if (sinks) denom += sink_share(sinks[h], M, c);
+        if (tid == 0) s_inv[map] = denom > 0.f ? 1.0f / denom : 0.f;
+    }
+    __syncthreads();
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int s = grp; s < splits; s += GROUPS) {
+        const f32x4 v = *(const f32x4*)(partial_o + (first + s) * HD + chunk * 4);
+        acc += v * wgt[map][s];
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) sums[map][grp][chunk * 4 + e] = acc[e];
+    __syncthreads();
+    float o = 0.f;
+    if (map == 0 && tid < HD) {
+        float total = 0.f;
+#pragma unroll
+        for (int g = 0; g < GROUPS; ++g) total += sums[0][g][tid];
+        o = total * s_inv[0];
+        if (ho.maps == 2) {
+            float other = 0.f;
+#pragma unroll
+            for (int g = 0; g < GROUPS; ++g) other += sums[1][g][tid];
+            o -= ho.lambda * (other * s_inv[1]);
+        }
+    }
+    float scale = 1.f;
+    if (ho.maps == 2) scale = ho.factor / sqrtf(hb_block_sum(o * o, red) / (float)ho.vdim + ho.eps);   // (entries beyond vdim are zeros)
+    if (map == 0 && tid < ho.vdim)
+        out[((size_t)b * heads + own_head) * ho.vdim + tid] = hb_from_float<bf16>(o * scale * gate);
 }
 
 // ---------------------------------------------------------------- launchers
@@ -1286,17 +1571,17 @@ extern "C" int hb_attn_decode_mfma(const void* q, void* k_cache, void* v_cache, 
     HB_REQUIRE((cos_t == nullptr) == (sin_t == nullptr), "attn_decode: cos and sin tables come together");
 #define DECODE_ARGS(QPTR) QPTR, (bf16*)k_cache, (bf16*)v_cache, partial_o, partial_ml, context_lens, slots, \
                           page_table, max_pages, nq, nkv, c, window, pages_per_split, fu, direct, ranges, B, \
-                          direct ? sinks : nullptr, chunk, softcap / scale, ext
+                          direct ? sinks : nullptr, chunk, softcap / scale, ext, HeadsFusion{}, HeadsOut{}
 #define LAUNCH_DECODE_FORM(HDV, FORM) do {                                                               \
     if (qkv)                                                                                             \
-        attn_decode_kernel<HDV, true, FORM><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr));              \
+        attn_decode_kernel<HDV, FORM_FUSED, FORM><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr));              \
     else                                                                                                 \
-        attn_decode_kernel<HDV, false, FORM><<<grid, 64, 0, stream>>>(DECODE_ARGS((const bf16*)q));      \
+        attn_decode_kernel<HDV, FORM_PLAIN, FORM><<<grid, 64, 0, stream>>>(DECODE_ARGS((const bf16*)q));      \
     } while (0)
 #define LAUNCH_DECODE(HDV) do { if (extended) LAUNCH_DECODE_FORM(HDV, true); else LAUNCH_DECODE_FORM(HDV, false); } while (0)
 #define LAUNCH_SLICES(QSV) do {                                                                          \
-    if (extended) attn_decode_kernel<128, true, true, QSV><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr)); \
-    else attn_decode_kernel<128, true, false, QSV><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr));       \
+    if (extended) attn_decode_kernel<128, FORM_FUSED, true, QSV><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr)); \
+    else attn_decode_kernel<128, FORM_FUSED, false, QSV><<<grid, 64, 0, stream>>>(DECODE_ARGS(nullptr));       \
     } while (0)
     if (qkv_slices == 2) LAUNCH_SLICES(2);
     else if (qkv_slices == 4) LAUNCH_SLICES(4);
@@ -1313,6 +1598,61 @@ extern "C" int hb_attn_decode_mfma(const void* q, void* k_cache, void* v_cache, 
     HB_CHECK_LAUNCH("attn_decode");
     if (!direct) {
 #define LAUNCH_MERGE(HDV) attn_decode_merge_kernel<HDV><<<B * nq, 256, 0, stream>>>(partial_o, partial_ml, (bf16*)out, splits, c, ranges, nq, sinks)
+        if (hd == 32) LAUNCH_MERGE(32);
+        else if (hd == 64) LAUNCH_MERGE(64);
+        else LAUNCH_MERGE(128);
+#undef LAUNCH_MERGE
+        HB_CHECK_LAUNCH("attn_decode_merge");
+    }
+    return 0;
+}
+
+// One token a sequence, from the projection's rows to the heads' outputs at their own size (HeadsFusion, HeadsOut): out bf16
+// [B, nq / maps x vdim]. gate_off < 0: no gate. slices > 1 (2, 4 or 8, heads kept at 128): the projection's K slices.
+extern "C" int hb_attn_decode_heads_mfma(const float* proj, int ld, int slices, size_t slice_stride, const float* bias,
+                                         const float* q_norm_w, const float* k_norm_w, const float* angles, int rot_dims,
+                                         int halves, int maps, int dim, int vdim, int map_stride, int k_off, int v_off,
+                                         float eps, int gate_off, float lambda, float factor, void* k_cache, void* v_cache,
+                                         void* out, float* partial_o, float* partial_ml, const int* context_lens,
+                                         const int* slots, const int* page_table, int max_pages, int page_size, int B, int nq,
+                                         int nkv, int hd, float scale, int window, int splits, int pages_per_split,
+                                         const int* ranges, const float* sinks, int chunk, float softcap, hipStream_t stream) {
+    HB_REQUIRE(!ranges || (B >= 2 && splits >= 2 && window == 0 && chunk == 0),
+               "attn_decode: a list of ranges is for two sequences or more, with a merge, without a window");
+    HB_REQUIRE(window >= 0 && chunk >= 0 && !(window > 0 && chunk > 0) && softcap >= 0.f, "attn_decode: bad window, chunk or cap");
+    HB_REQUIRE(B > 0 && nq > 0 && nkv > 0 && nq % nkv == 0 && page_size == PAGE, "attn_decode: bad sizes");
+    HB_REQUIRE(nq / nkv <= 32, "attn_decode: more than 32 query heads share a kv head");
+    HB_REQUIRE(splits > 0 && splits <= 1024 && pages_per_split > 0 && nkv <= 65535, "attn_decode: bad split");
+    HB_REQUIRE(scale > 0.f, "attn_decode: the score scale must be positive");
+    HB_REQUIRE(hd == 32 || hd == 64 || hd == 128, "attn_decode: head_dim %d is not one of 32, 64, 128", hd);
+    HB_REQUIRE(dim > 0 && vdim > 0 && dim <= hd && vdim <= hd, "attn_decode: heads of %d and %d kept at %d", dim, vdim, hd);
+    HB_REQUIRE(maps == 1 || (maps == 2 && (nq / nkv) % 2 == 0 && map_stride >= dim && map_stride + dim <= hd),
+               "attn_decode: %d maps of %d at %d in heads kept at %d", maps, dim, map_stride, hd);
+    HB_REQUIRE(k_off >= nq * dim && v_off >= k_off && ld >= k_off + nkv * maps * dim && ld >= v_off + nkv * vdim,
+               "attn_decode: rows of %d do not hold keys at %d and values at %d", ld, k_off, v_off);
+    HB_REQUIRE(v_off != k_off || (maps == 1 && vdim == dim), "attn_decode: values that are the keys have their size");
+    HB_REQUIRE(gate_off < 0 || gate_off + nq / maps * vdim <= ld, "attn_decode: the gate's columns lie outside the rows");
+    HB_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dim && (rot_dims == 0 || angles), "attn_decode: %d of %d entries turn", rot_dims, dim);
+    HB_REQUIRE((q_norm_w == nullptr) == (k_norm_w == nullptr), "attn_decode: queries and keys are normed together");
+    HB_REQUIRE(slices == 1 || (hd == 128 && (slices == 2 || slices == 4 || slices == 8) && slice_stride >= (size_t)B * ld),
+               "attn_decode: %d slices of the projection are not taken here", slices);
+    const dim3 grid(ranges ? 1 : B, nkv, splits);
+    const float c = scale * LOG2E;
+    const HeadsFusion hf = {proj, ld, slice_stride, bias, q_norm_w, k_norm_w, (const float2*)angles, rot_dims, halves,
+                            maps, dim, vdim, map_stride, k_off, v_off, eps};
+    const HeadsOut ho = {1, maps, vdim, gate_off < 0 ? nullptr : proj + gate_off, ld, slices, slice_stride, lambda, factor, eps};
+    bf16* const direct = splits == 1 ? (bf16*)out : nullptr;
+#define HEADS_GO(HDV, QSV)                                                                                                  attn_decode_kernel<HDV, FORM_HEADS, false, QSV><<<grid, 64, 0, stream>>>(                                                   nullptr, (bf16*)k_cache, (bf16*)v_cache, partial_o, partial_ml, context_lens, slots, page_table, max_pages, nq, nkv, c,         window, pages_per_split, DecodeFusion{}, direct, ranges, B, direct ? sinks : nullptr, chunk, softcap / scale,           AttnExtras{}, hf, ho)
+    if (slices == 2) HEADS_GO(128, 2);
+    else if (slices == 4) HEADS_GO(128, 4);
+    else if (slices == 8) HEADS_GO(128, 8);
+    else if (hd == 32) HEADS_GO(32, 1);
+    else if (hd == 64) HEADS_GO(64, 1);
+    else HEADS_GO(128, 1);
+#undef HEADS_GO
+    HB_CHECK_LAUNCH("attn_decode");
+    if (!direct) {
+#define LAUNCH_MERGE(HDV) attn_decode_merge_own_kernel<HDV><<<B * (nq / maps), 256 * maps, 0, stream>>>(partial_o, partial_ml, (bf16*)out, splits, c, ranges, nq, sinks, ho)
         if (hd == 32) LAUNCH_MERGE(32);
         else if (hd == 64) LAUNCH_MERGE(64);
         else LAUNCH_MERGE(128);

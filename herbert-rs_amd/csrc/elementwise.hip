@@ -764,27 +764,73 @@ extern "C" int hb_postnorm(const float* src, const float* w, float* x, void* y, 
     return 0;
 }
 
-// ---------------------------------------------------------------- squared relu
-// act[i] = max(z[i], 0)^2, float32 in, any storage type out.
-template <class TOut>
-__global__ void relu_squared_kernel(const float* __restrict__ z, TOut* __restrict__ act, size_t n) {
+// ---------------------------------------------------------------- activations between two matrices
+// act[i] = f(z[i]), float32 in, any storage type out: f = max(z, 0)^2, or the exact gelu,
+// z (1 + erf(z / sqrt 2)) / 2.
+#define HB_UNARY_RELU_SQUARED 0
+#define HB_UNARY_GELU 1
+template <class TOut, int ACT>
+__global__ void activate_kernel(const float* __restrict__ z, TOut* __restrict__ act, size_t n) {
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
-        const float r = fmaxf(z[i], 0.f);
-        act[i] = hb_from_float<TOut>(r * r);
+        const float v = z[i];
+        const float r = fmaxf(v, 0.f);
+        act[i] = hb_from_float<TOut>(ACT == HB_UNARY_GELU ? 0.5f * v * (1.0f + erff(v * 0.70710678118654752f)) : r * r);
     }
 }
 
-extern "C" int hb_relu_squared(const float* z, void* act, int act_dtype, size_t n, hipStream_t stream) {
-    HB_REQUIRE(n > 0, "relu_squared: empty input");
+extern "C" int hb_activate(const float* z, void* act, int act_dtype, size_t n, int activation, hipStream_t stream) {
+    HB_REQUIRE(n > 0, "activation: empty input");
+    HB_REQUIRE(activation == HB_UNARY_RELU_SQUARED || activation == HB_UNARY_GELU, "activation: unknown function %d", activation);
+    HB_REQUIRE(act_dtype == HB_F32 || act_dtype == HB_BF16, "activation: unknown output dtype %d", act_dtype);
     const size_t blocks = (n + 255) / 256;
     const unsigned grid = (unsigned)(blocks > 16384 ? 16384 : blocks);
-    if (act_dtype == HB_F32)
-        relu_squared_kernel<float><<<grid, 256, 0, stream>>>(z, (float*)act, n);
-    else if (act_dtype == HB_BF16)
-        relu_squared_kernel<bf16><<<grid, 256, 0, stream>>>(z, (bf16*)act, n);
-    else
-        HB_REQUIRE(false, "relu_squared: unknown output dtype %d", act_dtype);
-    HB_CHECK_LAUNCH("relu_squared");
+#define HB_ACTIVATE(TV, A) activate_kernel<TV, A><<<grid, 256, 0, stream>>>(z, (TV*)act, n)
+    if (act_dtype == HB_F32) {
+        if (activation == HB_UNARY_GELU) HB_ACTIVATE(float, HB_UNARY_GELU);
+        else HB_ACTIVATE(float, HB_UNARY_RELU_SQUARED);
+    } else {
+        if (activation == HB_UNARY_GELU) HB_ACTIVATE(bf16, HB_UNARY_GELU);
+        else HB_ACTIVATE(bf16, HB_UNARY_RELU_SQUARED);
+    }
+#undef HB_ACTIVATE
+    HB_CHECK_LAUNCH("activate");
+    return 0;
+}
+
+// ------------------------------------------- where a pass over the layers makes the stream anew
+// rows = x in the compute dtype (the rows that a product reads next), then x = base (rows that the product adds to);
+// base null: x stays as it is.
+template <class TOut, bool QUADS>
+__global__ void __launch_bounds__(256)
+rows_and_base_kernel(float* x, TOut* __restrict__ rows, const float* __restrict__ base, unsigned total) {
+    const unsigned idx = blockIdx.x * 256u + threadIdx.x;
+    if (idx >= total) return;
+    if (QUADS) {
+        const hb_f4 v = *(const hb_f4*)(x + 4 * (size_t)idx);
+        store_four(rows + 4 * (size_t)idx, v);
+        if (base) *(hb_f4*)(x + 4 * (size_t)idx) = *(const hb_f4*)(base + 4 * (size_t)idx);
+    } else {
+        rows[idx] = hb_from_float<TOut>(x[idx]);
+        if (base) x[idx] = base[idx];
+    }
+}
+
+extern "C" int hb_rows_and_base(float* x, void* rows, int dtype, const float* base, size_t n, hipStream_t stream) {
+    HB_REQUIRE(n > 0 && n < (1ull << 32), "pass rows: empty input or too many rows");
+    HB_REQUIRE(dtype == HB_F32 || dtype == HB_BF16, "pass rows: unknown dtype %d", dtype);
+    const bool quads = n % 4 == 0 && (((uintptr_t)x | (uintptr_t)rows | (uintptr_t)base) & 15) == 0;
+    const unsigned total = (unsigned)(quads ? n / 4 : n);
+    const unsigned blocks = (total + 255) / 256;
+#define HB_ROWS(TV, Q) rows_and_base_kernel<TV, Q><<<blocks, 256, 0, stream>>>(x, (TV*)rows, base, total)
+    if (dtype == HB_F32) {
+        if (quads) HB_ROWS(float, true);
+        else HB_ROWS(float, false);
+    } else {
+        if (quads) HB_ROWS(bf16, true);
+        else HB_ROWS(bf16, false);
+    }
+#undef HB_ROWS
+    HB_CHECK_LAUNCH("rows_and_base");
     return 0;
 }
 

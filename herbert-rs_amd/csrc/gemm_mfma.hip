@@ -16,7 +16,7 @@
 // (weight rows interleaved in blocks of 16: gate rows, then the up rows of the same outputs),
 // 3 (tiled, an entry point of its own) the q/k/v projection with per-head norm, rotation and
 // cache write, 4 (few rows, an entry point of its own) the sums pass a norm without mean and variance and join the
-// residual stream, which passes another one (see TanhJoin).
+// residual stream, which passes another one (see TanhJoin), 5 an activation of every sum, to bfloat16.
 // In xigh/herbert-rs: crates/backends/backend_bf16/src/kernels.rs:154-164 is the product; the inputs are rounded to
 // bfloat16 before they are multiplied, as crates/backends/backend_bf16_avx512/src/avx512_bf16_matvec.S:1-12 does
 // (float32 sums); SwiGLU in the epilogue as crates/backends/backend_metal/shaders/fused_gate_up_swiglu.metal:27-83;
@@ -39,6 +39,7 @@ typedef float f32x16 __attribute__((ext_vector_type(16)));
 #define EPI_SWIGLU 2
 #define EPI_QKV 3
 #define EPI_JOIN 4
+#define EPI_ACT 5
 
 // silu(g) u with the hardware's reciprocal (1 ulp; the result is rounded to bfloat16): a full division
 // is a dozen instructions, and the epilogue of a 256 x 256 tile does 128 of these a lane
@@ -52,6 +53,27 @@ __device__ __forceinline__ float silu_mul(float g, float u) {
 template <int GLU>
 __device__ __forceinline__ float glu_mul(float g, float u) {
     return GLU == GLU_RELU ? fmaxf(g, 0.f) * u : silu_mul(g, u);
+}
+
+// the activation of epilogue 5: max(z, 0)^2, or the exact gelu z (1 + erf(z / sqrt 2)) / 2. With q = erfc(|z| / sqrt 2) it
+// is z - z q / 2 for z >= 0 and z q / 2 below; q is Hastings' approximation (Abramowitz and Stegun, Handbook of Mathematical
+// Functions, 7.1.26: |error| <= 1.5e-7, far below the rounding to bfloat16), a polynomial in 1 / (1 + p x) times exp(-x^2).
+#define UNARY_RELU_SQUARED 0
+#define UNARY_GELU 1
+__device__ __forceinline__ float gelu_erf(float z) {
+    const float x = fabsf(z) * 0.70710678f;
+    const float t = __builtin_amdgcn_rcpf(fmaf(0.3275911f, x, 1.0f));
+    float q = fmaf(1.061405429f, t, -1.453152027f);
+    q = fmaf(q, t, 1.421413741f);
+    q = fmaf(q, t, -0.284496736f);
+    q = fmaf(q, t, 0.254829592f);
+    const float half_q = 0.5f * z * q * t * __builtin_amdgcn_exp2f(x * x * -1.44269504f);
+    return z >= 0.f ? z - half_q : half_q;
+}
+__device__ __forceinline__ float unary(float z, int act) {
+    if (act == UNARY_GELU) return gelu_erf(z);
+    const float r = fmaxf(z, 0.f);
+    return r * r;
 }
 
 // What epilogue 4 does with a product's sums p (a part's output): s = x + n_after(p) + extra + step, n(v) =
@@ -115,7 +137,7 @@ struct NormHandoff {
     int scale_parts;
     float scale_eps;             // the width of the normed rows is this product's K
     float emit_eps;
-    int glu;                     // the gated unit of epilogue 2
+    int glu;                     // the gated unit of epilogue 2, the activation of epilogue 5
 };
 
 template <int MB, int NB, int WAVES, int EPI, bool PACKED, bool NORM>
@@ -404,6 +426,20 @@ gemm_skinny_kernel(const void* __restrict__ Xv, const bf16* __restrict__ W, void
                                                  : glu_mul<GLU_SILU>(acc[a][b][i], acc[a + 1][b][i]));
                 }
             }
+    } else if (EPI == EPI_ACT) {
+        bf16* C = (bf16*)Cv;
+#pragma unroll
+        for (int a = 0; a < NB; ++a)
+#pragma unroll
+            for (int b = 0; b < MB; ++b) {
+                const int m = b * 16 + r16;
+                if (m >= M) continue;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int n = n0 + a * 16 + g4 * 4 + i;
+                    if (n < N) C[(size_t)m * ldc + n] = hb_from_float<bf16>(unary(acc[a][b][i], hand.glu));
+                }
+            }
     } else {
         float* C = (float*)Cv;
         const bool emit = EPI == EPI_ADD && MB == 1 && hand.emit_g;
@@ -557,6 +593,17 @@ __global__ void gemm_slices_swiglu_kernel(const float* __restrict__ partial, bf1
     C[(size_t)m * ldc + j] = hb_from_float<bf16>(glu_mul<GLU>(gate, up));
 }
 
+// The same for the activation of epilogue 5: C bf16 [M, N].
+__global__ void gemm_slices_act_kernel(const float* __restrict__ partial, bf16* __restrict__ C, int M, int N, int ldc, int slices,
+                                       int act) {
+    const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= (size_t)M * N) return;
+    const int m = (int)(idx / N), n = (int)(idx % N);
+    float sum = 0.f;
+    for (int s = 0; s < slices; ++s) sum += partial[(size_t)s * M * N + idx];
+    C[(size_t)m * ldc + n] = hb_from_float<bf16>(unary(sum, act));
+}
+
 template <int MB, int NB, int WAVES>
 static void launch_skinny(const void* X, const void* W, void* C, int M, int N, int K, int ldc, int epi,
                           int packed, const float* norm_w, float eps, hipStream_t stream, const NormHandoff& hand) {
@@ -581,10 +628,12 @@ static void launch_skinny(const void* X, const void* W, void* C, int M, int N, i
     } else if (packed) {
         if (epi == EPI_STORE) SKINNY_GO(EPI_STORE, true, false);
         else if (epi == EPI_ADD) SKINNY_GO(EPI_ADD, true, false);
+        else if (epi == EPI_ACT) SKINNY_GO(EPI_ACT, true, false);
         else SKINNY_GO(EPI_SWIGLU, true, false);
     } else {
         if (epi == EPI_STORE) SKINNY_GO(EPI_STORE, false, false);
         else if (epi == EPI_ADD) SKINNY_GO(EPI_ADD, false, false);
+        else if (epi == EPI_ACT) SKINNY_GO(EPI_ACT, false, false);
         else SKINNY_GO(EPI_SWIGLU, false, false);
     }
 #undef SKINNY_GO
@@ -637,7 +686,25 @@ __device__ __forceinline__ void store_wave_tile(const f32x16 (&acc)[TN32][TM32],
     for (int b = 0; b < TM32; ++b) {
         const int m = m_base + 32 * b + c32;
         if (m >= M) continue;
-        if (EPI == EPI_SWIGLU) {
+        if (EPI == EPI_ACT) {
+            bf16* C = (bf16*)Cv;
+#pragma unroll
+            for (int a = 0; a < TN32; ++a)
+#pragma unroll
+                for (int q = 0; q < 4; ++q) {
+                    const int n = n_base + 32 * a + 8 * q + 4 * g2;
+                    bf16x4 v;
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) v[j] = (__bf16)unary(acc[a][b][4 * q + j], GLU);
+                    if (n + 3 < N && (ldc & 3) == 0) {
+                        *(bf16x4*)((__bf16*)C + (size_t)m * ldc + n) = v;
+                    } else {
+#pragma unroll
+                        for (int j = 0; j < 4; ++j)
+                            if (n + j < N) ((__bf16*)C)[(size_t)m * ldc + n + j] = v[j];
+                    }
+                }
+        } else if (EPI == EPI_SWIGLU) {
             bf16* C = (bf16*)Cv;
 #pragma unroll
             for (int a = 0; a < TN32; ++a)
@@ -791,6 +858,43 @@ __device__ __forceinline__ void store_wave_tile_swiglu_lds(const f32x16 (&acc)[T
     }
 }
 
+// The outputs of epilogue 5 through LDS in the same way: rows of TN32 x 32 bfloat16.
+template <int TN32, int TM32, int ACT>
+__device__ __forceinline__ void store_wave_tile_act_lds(const f32x16 (&acc)[TN32][TM32], bf16* C, int M, int N, int ldc,
+                                                        int m_base, int n_base, int lane, bf16* stage) {
+    constexpr int CH = 4 * TN32;            // 16-byte chunks of a row (a power of two)
+    constexpr int RPI = 64 / CH;
+    constexpr int ROWS = 32 * TM32;
+    const int c32 = lane & 31, g2 = lane >> 5;
+#pragma unroll
+    for (int b = 0; b < TM32; ++b)
+#pragma unroll
+        for (int a = 0; a < TN32; ++a)
+#pragma unroll
+            for (int q = 0; q < 4; ++q) {
+                const int row = 32 * b + c32;
+                bf16x4 v;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) v[j] = (__bf16)unary(acc[a][b][4 * q + j], ACT);
+                *(bf16x4*)((__bf16*)stage + row * (CH * 8) + (((4 * a + q) ^ (row & (CH - 1))) * 8) + 4 * g2) = v;
+            }
+    const int rrow = lane / CH, rchunk = lane % CH;
+#pragma unroll
+    for (int i = 0; i < ROWS / RPI; ++i) {
+        const int row = i * RPI + rrow;
+        const int m = m_base + row, n = n_base + 8 * rchunk;
+        const bf16x8 v = *(const bf16x8*)((const __bf16*)stage + row * (CH * 8) + ((rchunk ^ (row & (CH - 1))) * 8));
+        if (m >= M) continue;
+        if (n + 7 < N) {
+            *(bf16x8*)((__bf16*)C + (size_t)m * ldc + n) = v;
+        } else {
+#pragma unroll
+            for (int j = 0; j < 8; ++j)
+                if (n + j < N) ((__bf16*)C)[(size_t)m * ldc + n + j] = v[j];
+        }
+    }
+}
+
 // The q/k/v projection of prompts with what follows it, for heads of 128 (a wave's tile is 128
 // columns wide: one head): per-head RMSNorm (if weights are given), rotation over the whole head
 // (if tables are given), queries to q_out [M, nq 128] and keys and values into the pages (values
@@ -905,7 +1009,7 @@ struct RowScale {
     const float* partial;        // [parts, MP]; null: no scaling
     int parts;
     float eps;
-    int glu;                     // the gated unit of epilogue 2
+    int glu;                     // the gated unit of epilogue 2, the activation of epilogue 5
 };
 
 // K in steps of 64. A step's weights are two k-steps of 32 (blocks as above); its activations lie
@@ -1150,6 +1254,22 @@ gemm_tile_kernel(const bf16* __restrict__ X, const bf16* __restrict__ W, void* _
             else
                 store_wave_tile_lds<EPI_ADD, TN32, TM32, PB>(acc, dst, M, N, ld, m0 + wm * TMB * 16,
                                                              n0 + wn * TNB * 16, lane, stage);
+        } else if (EPI == EPI_ACT && sliced && BM >= 128 && PB_FIT >= 1 && (N & 3) == 0 && ((size_t)dst & 15) == 0) {
+            hb_workgroup_barrier();
+            store_wave_tile_lds<EPI_STORE, TN32, TM32, PB>(acc, dst, M, N, N, m0 + wm * TMB * 16, n0 + wn * TNB * 16, lane,
+                                                           (float*)((char*)lds + wave * REGION));
+        } else if (EPI == EPI_ACT && !sliced && BM >= 128 && REGION >= 32 * TM32 * TN32 * 64 && (TN32 & (TN32 - 1)) == 0 &&
+                   (ldc & 7) == 0 && ((size_t)Cv & 15) == 0) {
+            hb_workgroup_barrier();
+            bf16* const stage = (bf16*)((char*)lds + wave * REGION);
+            if (scale.glu == UNARY_GELU)
+                store_wave_tile_act_lds<TN32, TM32, UNARY_GELU>(acc, (bf16*)Cv, M, N, ldc, m0 + wm * TMB * 16,
+                                                                n0 + wn * TNB * 16, lane, stage);
+            else
+                store_wave_tile_act_lds<TN32, TM32, UNARY_RELU_SQUARED>(acc, (bf16*)Cv, M, N, ldc, m0 + wm * TMB * 16,
+                                                                        n0 + wn * TNB * 16, lane, stage);
+        } else if (EPI == EPI_ACT && !sliced && scale.glu == UNARY_GELU) {
+            store_wave_tile<EPI, TN32, TM32, UNARY_GELU>(acc, Cv, M, N, ldc, m0 + wm * TMB * 16, n0 + wn * TNB * 16, c32, g2);
         } else if (sliced) {
             store_wave_tile<EPI_STORE, TN32, TM32>(acc, dst, M, N, N, m0 + wm * TMB * 16, n0 + wn * TNB * 16, c32, g2);
         } else if (EPI == EPI_SWIGLU && scale.glu == GLU_RELU) {
@@ -1274,7 +1394,8 @@ gemm_tile32_kernel(const bf16* __restrict__ X, const bf16* __restrict__ W, void*
         if (t + 1 < nsteps) run_step(1, t + 1);
     }
     hb_wait_vmcnt<0>();      // the loads past the end (repeats of the last step) have landed too
-    if (EPI == EPI_SWIGLU && glu == GLU_RELU)
+    static_assert((int)GLU_RELU == (int)UNARY_GELU, "the second of either kind");
+    if ((EPI == EPI_SWIGLU || EPI == EPI_ACT) && glu == GLU_RELU)
         store_wave_tile<EPI, TN32, TM32, GLU_RELU>(acc, Cv, M, N, ldc, m0 + wm * TMB * 16, n0 + wn * TNB * 16, c32, g2);
     else
         store_wave_tile<EPI, TN32, TM32>(acc, Cv, M, N, ldc, m0 + wm * TMB * 16, n0 + wn * TNB * 16, c32, g2);
@@ -1310,10 +1431,12 @@ static int launch_tiles(Kernel kern, size_t lds, int threads, long total, int sl
         if (packed) {                                                                                \
             if (epi == EPI_STORE) return launch_tiles(KERNEL<EPI_STORE, true, __VA_ARGS__>, lds, threads, total, slices, x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream EXTRA); \
             if (epi == EPI_ADD) return launch_tiles(KERNEL<EPI_ADD, true, __VA_ARGS__>, lds, threads, total, slices, x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream EXTRA); \
+            if (epi == EPI_ACT) return launch_tiles(KERNEL<EPI_ACT, true, __VA_ARGS__>, lds, threads, total, slices, x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream EXTRA); \
             return launch_tiles(KERNEL<EPI_SWIGLU, true, __VA_ARGS__>, lds, threads, total, slices, x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream EXTRA); \
         }                                                                                            \
         if (epi == EPI_STORE) return launch_tiles(KERNEL<EPI_STORE, false, __VA_ARGS__>, lds, threads, total, slices, x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream EXTRA); \
         if (epi == EPI_ADD) return launch_tiles(KERNEL<EPI_ADD, false, __VA_ARGS__>, lds, threads, total, slices, x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream EXTRA); \
+        if (epi == EPI_ACT) return launch_tiles(KERNEL<EPI_ACT, false, __VA_ARGS__>, lds, threads, total, slices, x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream EXTRA); \
         return launch_tiles(KERNEL<EPI_SWIGLU, false, __VA_ARGS__>, lds, threads, total, slices, x, w, C, M, N, K, ldc, m_tiles, n_tiles, stream EXTRA); \
     } while (0)
 
@@ -1606,7 +1729,7 @@ extern "C" double hb_gemm_mfma_plan_cost(int M, int N, int K, int epi, int norme
 
 // C (+)= X @ W^T. X [M, K] bf16, W [N, K] bf16. epi 0: C f32 [M, N] stored; 1: added to;
 // 2: W's rows are gate/up interleaved in blocks of 16 and C is bf16 [M, N / 2] = silu(gate) * up (glu 0), or
-// max(gate, 0) * up (glu 1).
+// max(gate, 0) * up (glu 1); 5: C is bf16 [M, N], every sum through the activation that glu names (unary).
 // packed != 0: W is stored as [K / 32][N / 16][64 lanes][8]: lane = 16 * (k / 8 % 4) + n % 16.
 // All blocks of one k-step lie together: workgroups that advance through K side by side read one
 // contiguous stretch of memory at a time, as a streaming copy would.
@@ -1620,7 +1743,7 @@ extern "C" int hb_gemm_mfma(const void* X, const void* W, void* C, int M, int N,
                             const float* scale_partial, int scale_parts, float scale_eps, float emit_eps,
                             int* deferred_slices, int glu, hipStream_t stream) {
     const NormHandoff hand = {emit_g, (bf16*)emit_xg, emit_partial, scale_partial, scale_parts, scale_eps, emit_eps, glu};
-    HB_REQUIRE(glu == GLU_SILU || (glu == GLU_RELU && epi == EPI_SWIGLU), "gemm_mfma: unknown gated unit %d", glu);
+    HB_REQUIRE(glu == 0 || (glu == 1 && (epi == EPI_SWIGLU || epi == EPI_ACT)), "gemm_mfma: unknown gated unit or activation %d", glu);
     const bool emit_whole = emit_g && !emit_partial;      // the second kernel of a product cut into slices norms
     HB_REQUIRE(!scale_partial || (M <= 16 && !norm_w), "gemm_mfma: a norm is handed on for at most 16 rows");
     HB_REQUIRE(!emit_g || (epi == EPI_ADD && emit_xg && !norm_w), "gemm_mfma: only the adding product leaves a norm behind");
@@ -1631,7 +1754,8 @@ extern "C" int hb_gemm_mfma(const void* X, const void* W, void* C, int M, int N,
                "gemm_mfma: the fused norm takes M <= 16, N >= 16384 and no add");
     HB_REQUIRE(!packed || N % 16 == 0, "gemm_mfma: packed weights need N %% 16 == 0");
     HB_REQUIRE(M > 0 && N > 0 && K > 0, "gemm_mfma: empty problem (M=%d, N=%d, K=%d)", M, N, K);
-    HB_REQUIRE(epi >= 0 && epi <= 2, "gemm_mfma: unknown epilogue %d", epi);
+    HB_REQUIRE((epi >= 0 && epi <= 2) || epi == EPI_ACT, "gemm_mfma: unknown epilogue %d", epi);
+    HB_REQUIRE(epi != EPI_ACT || !norm_w, "gemm_mfma: the activating product takes rows that are normed");
     HB_REQUIRE(K % 32 == 0, "gemm_mfma: K=%d is no multiple of 32", K);
     HB_REQUIRE(epi != EPI_SWIGLU || N % 32 == 0, "gemm_mfma: the SwiGLU epilogue needs N %% 32 == 0");
     HB_REQUIRE(ldc >= (epi == EPI_SWIGLU ? N / 2 : N), "gemm_mfma: output row stride %d too small", ldc);
@@ -1652,7 +1776,7 @@ extern "C" int hb_gemm_mfma(const void* X, const void* W, void* C, int M, int N,
     const int rows_main = split_rows(M, N, K, ldc, epi, norm_w || emit_g || scale_partial || deferred_slices, tile_hint,
                                      workspace_floats, plan);
     if (rows_main > 0) {
-        const size_t out_bytes = epi == EPI_SWIGLU ? sizeof(bf16) : sizeof(float);
+        const size_t out_bytes = epi == EPI_SWIGLU || epi == EPI_ACT ? sizeof(bf16) : sizeof(float);
         const int rc = hb_gemm_mfma(X, W, C, rows_main, N, K, ldc, epi, packed, nullptr, eps, 0, workspace, workspace_floats,
                                     nullptr, nullptr, nullptr, nullptr, 0, 0.f, 0.f, nullptr, glu, stream);
         if (rc != 0) return rc;
@@ -1708,6 +1832,8 @@ extern "C" int hb_gemm_mfma(const void* X, const void* W, void* C, int M, int N,
         else if (epi == EPI_SWIGLU)
             gemm_slices_swiglu_kernel<GLU_SILU><<<(unsigned)((total / 2 + 255) / 256), 256, 0, stream>>>(
                 workspace, (bf16*)C, M, N, ldc, slices);
+        else if (epi == EPI_ACT)
+            gemm_slices_act_kernel<<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(workspace, (bf16*)C, M, N, ldc, slices, glu);
         else
             gemm_slices_kernel<<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(workspace, (float*)C, M, N, ldc,
                                                                                   slices, epi == EPI_ADD);

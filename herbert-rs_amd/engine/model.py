@@ -121,13 +121,22 @@ class Model:
         if self.pass_input is not None and self.pass_input.reads_embedding:
             embedded = rt.buffer("embedding_output", tuple(x.shape), torch.float32)
             ops.tanh_join(x, x_out=embedded)         # (a copy)
-        # what joins x before an entry, where a pass starts there
-        joins = [None if e.starts_pass is None else self.pass_input.rows(e.starts_pass, embedded) for e in self.schedule]
+        # what joins x before an entry, where a pass starts there; or the pass input makes x anew there itself
+        replaces = self.pass_input is not None and getattr(self.pass_input, "replaces", False)
+        joins = [None if e.starts_pass is None or replaces else self.pass_input.rows(e.starts_pass, embedded)
+                 for e in self.schedule]
+        kept = self.pass_input.begin(ctx, x) if replaces else None
         for i, e in enumerate(self.schedule):
             ctx.pass_input = joins[i]
             ctx.next_pass_input = joins[i + 1] if i + 1 < len(joins) else None
             if ctx.pass_input is not None and not getattr(self.blocks[e.layer], "takes_pass_input", False):
                 ops.tanh_join(x, extra=joins[i][0], step=joins[i][1], x_out=x)
+            if replaces and e.starts_pass is not None:
+                # (nothing that a block left for the next one's norm may be taken on: x is another now)
+                ctx.left = ctx.join = ctx.fresh_rows = None
+                first_norm = getattr(self.blocks[e.layer], "first_norm", None)
+                ctx.norm_ahead = None if first_norm is None else (first_norm(), i)
+                self.pass_input.forward(ctx, x, kept)
             ctx.entry = i
             ctx.cache_entry = i if e.cache is None else e.cache
             ctx.owns_cache = e.cache is None
@@ -135,7 +144,7 @@ class Model:
             ctx.norm_after_block = None
             ctx.next_block = self.blocks[self.schedule[i + 1].layer] if i + 1 < len(self.schedule) else None
             if ctx.next_block is not None and self.schedule[i + 1].starts_pass is not None \
-                    and not getattr(ctx.next_block, "takes_pass_input", False):
+                    and (replaces or not getattr(ctx.next_block, "takes_pass_input", False)):
                 ctx.next_block = None       # x changes before that block: nothing of its first norm may be prepared
             if ctx.next_block is not None:
                 first_norm = getattr(self.blocks[self.schedule[i + 1].layer], "first_norm", None)

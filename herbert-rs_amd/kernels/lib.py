@@ -38,7 +38,14 @@ SIGNATURES = {
         "hb_layernorm": [_P, _P, _F, _P, _P, _I, _P, _I, _I, _F, _P],
         "hb_scale": [_P, _F, _SZ, _P],
         "hb_postnorm": [_P, _P, _P, _P, _I, _P, _I, _I, _F, _F, _P],
-        "hb_relu_squared": [_P, _P, _I, _SZ, _P],
+        "hb_activate": [_P, _P, _I, _SZ, _I, _P],
+        "hb_rows_and_base": [_P, _P, _I, _P, _SZ, _P],
+    },
+    "heads": {
+        "hb_step_angles": [_P, _P, _I, _F, _P, _I, _P],
+        "hb_heads_prepare": [_P, _I, _I, _SZ, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I,
+                             _I, _I, _I, _I, _F, _P],
+        "hb_heads_difference": [_P, _I, _P, _I, _I, _SZ, _P, _I, _I, _I, _I, _F, _F, _F, _P],
     },
     "gemm_plain": {
         "hb_gemm_plain": [_P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P],

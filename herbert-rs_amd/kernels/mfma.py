@@ -10,6 +10,7 @@ import ctypes
 import torch
 
 from ..errors import BackendError
+from . import heads
 from . import lib
 from . import ops
 from .ops import _check, _stream
@@ -28,7 +29,7 @@ lib.register_signatures("gemm_mfma", {
     "hb_gemm_qkv_mfma": [_P, _P, _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _P, _P, _P, _P, _F, _I, _I, _I, _I, _P],
 })
 
-EPI_STORE, EPI_ADD, EPI_SWIGLU = 0, 1, 2
+EPI_STORE, EPI_ADD, EPI_SWIGLU, EPI_ACT = 0, 1, 2, 5
 SLICE_WORKSPACE_FLOATS = 16 << 20     # most that the tiled product may use for its K slices (64 MB)
 
 
@@ -431,7 +432,25 @@ def gemm_swiglu(a, w_interleaved, out, packed=False, norm=None, tile=0, row_scal
              GATED_UNITS[activation], _stream())
 
 
+def gemm_activated(a, w, out, activation, packed=False, tile=0, row_scale=None, scratch=None):
+    """out bf16 [M, N] = f(a bf16 [M, K] @ w bf16 [N, K]^T), f one of ops.UNARY_ACTIVATIONS, in the product's epilogue.
+    row_scale: see _handoff_args (the sums are scaled before f)."""
+    M, K = a.shape
+    _check(a, "a", torch.bfloat16, (M, K))
+    _check(w, "w", torch.bfloat16, (None, K))
+    N = w.shape[0]
+    _check(out, "out", torch.bfloat16, (M, N))
+    if K % 32:
+        raise BackendError(f"gemm_mfma (activated) refuses M={M}, N={N}, K={K}")
+    hand = _handoff_args(M, N, K, None, row_scale, False, None)
+    ws_ptr, ws_floats = _slice_workspace(scratch, a.device, M, N, K, tile)
+    lib.call("gemm_mfma", "hb_gemm_mfma", a.data_ptr(), w.data_ptr(), out.data_ptr(), M, N, K, N, EPI_ACT, 1 if packed else 0,
+             None, 0.0, int(tile), ws_ptr, ws_floats, *hand, None, ops.UNARY_ACTIVATIONS[activation], _stream())
+
+
 lib.register_signatures("attention_mfma", {
+    "hb_attn_decode_heads_mfma": [_P, _I, _I, ctypes.c_size_t, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _F, _F, _P,
+                                  _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _P, _I, _F, _P],
     "hb_attn_prefill_mfma": [_P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I, _P, _I, _F, _P, _I, _I, _I, _P],
     "hb_attn_decode_mfma": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I,
                             _P, _P, _P, _P, _P, _F, _I, _I, ctypes.c_size_t, _P, _F, _I, _P, _I, _F, _P, _I, _I, _I, _P],
@@ -643,6 +662,54 @@ def attention_decode_fused(qkv, q_norm_w, k_norm_w, cos, sin, meta, kv, out, nq,
              None if sin is None else sin.data_ptr(), float(eps), 1, n_slices, stride,
              None if ranges is None else ranges.data_ptr(), coef, every, None if sinks is None else sinks.data_ptr(), 0, 0.0,
              *extras, _stream())
+
+
+def decode_heads_fusable(meta, kv, layout, dtype):
+    """True if the decode kernel can take the projection's rows themselves (see attention_decode_heads)."""
+    return decode_fusable(meta, kv, layout.nq, layout.nkv, layout.hd, 0, dtype)
+
+
+def attention_decode_heads(proj, layout, bias, q_norm_w, k_norm_w, angles, rot_dims, halves, eps, meta, kv, out, scale, window=None,
+                           chunk=None, softcap=None, sinks=None, gate_off=None, lam=0.0, factor=1.0, slices=None, scratch=None):
+    """One token a sequence: what heads.prepare does, the attention over the pages, and what heads.difference (layout.maps 2)
+    or a gate (gate_off: the gate's first column in proj) does with its outputs, in one kernel (+ merge).
+    proj f32 [B, ld] (or its K slices, as gemm(..., defer_slices=True) gives them, with heads kept at 128); out bf16
+    [B, nq / maps x vdim]."""
+    L, B = layout, meta.num_seqs
+    heads.check_operands(L, proj, angles, rot_dims, bias, q_norm_w, k_norm_w)
+    _check(proj, "proj", torch.float32, (B, None))
+    _check(out, "out", torch.bfloat16, (B, L.nq // L.maps * L.vdim))
+    pages = kv.k.shape[0]
+    _check(kv.k, "key pages", torch.bfloat16, (pages, L.nkv, 64, L.hd))
+    _check(kv.v, "value pages", torch.bfloat16, (pages, L.nkv, L.hd, 64))
+    _check(kv.page_table, "page_table", torch.int32, (None, None))
+    _check(meta.slots, "slots", torch.int32, (B,))
+    _check(meta.context_lens, "context_lens", torch.int32, (B,))
+    if not decode_heads_fusable(meta, kv, L, torch.bfloat16):
+        raise BackendError(f"fused decode attention refuses heads kept at {L.hd} with {L.nq}/{L.nkv} of them in this step")
+    if sinks is not None:
+        _check(sinks, "sinks", torch.float32, (L.nq,))
+    ld = proj.shape[1]
+    if gate_off is not None and not 0 <= gate_off <= ld - L.nq // L.maps * L.vdim:
+        raise BackendError("fused decode attention: the gate's columns lie outside the rows")
+    window, chunk = int(window or 0), int(chunk or 0)
+    listed = _decode_ranges(meta, L.nkv, window, chunk)
+    if listed:
+        (splits, ranges), per = listed, 1
+        po, pml = _partial_buffers(scratch, proj.device, L.nq, splits, L.hd)
+    else:
+        (splits, per), ranges = _decode_split(meta, L.nkv, window, chunk), None
+        po, pml = _partial_buffers(scratch, proj.device, B * L.nq, splits, L.hd)
+    n, src, stride = heads.slice_args(slices, proj)
+    if n > 1 and (n not in DEFERRED_SLICES or L.hd != 128 or stride < proj.numel()):
+        raise BackendError(f"fused decode attention does not add up {n} slices of the projection")
+    ptr = lambda t: None if t is None else t.data_ptr()
+    lib.call("attention_mfma", "hb_attn_decode_heads_mfma", src, ld, n, stride, ptr(bias), ptr(q_norm_w), ptr(k_norm_w),
+             ptr(angles), int(rot_dims), 1 if halves else 0, L.maps, L.dim, L.vdim, L.map_stride, L.k_off, L.v_off, float(eps),
+             -1 if gate_off is None else int(gate_off), float(lam), float(factor), kv.k.data_ptr(), kv.v.data_ptr(),
+             out.data_ptr(), po.data_ptr(), pml.data_ptr(), meta.context_lens.data_ptr(), meta.slots.data_ptr(),
+             kv.page_table.data_ptr(), kv.page_table.shape[1], kv.page_size, B, L.nq, L.nkv, L.hd, float(scale), window, splits, per,
+             ptr(ranges), ptr(sinks), chunk, float(softcap or 0.0), _stream())
 
 
 DEFERRED_SLICES = (2, 4, 8)     # numbers of slices of the projection that the decode kernel adds up itself

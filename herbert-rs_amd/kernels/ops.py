@@ -522,11 +522,32 @@ def postnorm(src, weight, x, y, eps, alpha_next, acc=None):
              _stream())
 
 
-def relu_squared(z, out):
-    """out = max(z, 0)^2; z f32, out of the same shape in any storage type."""
-    _check(z, "z", torch.float32)
+UNARY_ACTIVATIONS = {"relu_squared": 0, "gelu": 1}
+
+
+def activate(z, out, activation):
+    """out = max(z, 0)^2 ("relu_squared") or z (1 + erf(z / sqrt 2)) / 2 ("gelu"); z f32, out any storage type, alike in
+    shape."""
+    if activation not in UNARY_ACTIVATIONS:
+        raise BackendError(f"unknown activation {activation!r}")
+    _check(z, "z", torch.float32, tuple(z.shape))
     _check(out, "out", None, tuple(z.shape))
-    lib.call("elementwise", "hb_relu_squared", z.data_ptr(), out.data_ptr(), dtype_code(out), z.numel(), _stream())
+    lib.call("elementwise", "hb_activate", z.data_ptr(), out.data_ptr(), dtype_code(out), z.numel(), UNARY_ACTIVATIONS[activation],
+             _stream())
+
+
+def relu_squared(z, out):
+    """out = max(z, 0)^2 (see activate)."""
+    activate(z, out, "relu_squared")
+
+
+def rows_and_base(x, rows, base=None):
+    """rows = x in their own storage type, then x = base (None: x stays): x, base f32, all of one shape."""
+    _check(x, "x", torch.float32, tuple(x.shape))
+    _check(rows, "rows", None, tuple(x.shape))
+    if base is not None:
+        _check(base, "base", torch.float32, tuple(x.shape))
+    lib.call("elementwise", "hb_rows_and_base", x.data_ptr(), rows.data_ptr(), dtype_code(rows), _ptr(base), x.numel(), _stream())
 
 
 def gemm_plain_columns(a, col0, K, w, c, accumulate=False, decay=None):

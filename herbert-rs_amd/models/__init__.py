@@ -1,4 +1,4 @@
 """Architectures: each module turns its typed configuration into a ModelSpec and registers itself."""
-from . import bozasun, mefatar, modasun, mutedra, qwen3, vipalorn
+from . import bozasun, figalorn, mefatar, modasun, mutedra, qwen3, vipalorn
 
-__all__ = ["bozasun", "mefatar", "modasun", "mutedra", "qwen3", "vipalorn"]
+__all__ = ["bozasun", "figalorn", "mefatar", "modasun", "mutedra", "qwen3", "vipalorn"]

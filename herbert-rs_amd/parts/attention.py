@@ -23,9 +23,17 @@ a position of the kind "rope_pairs" (neighbouring pairs turn), `sink` (the softm
 holds exp(s_h), a stored number a head without key or value), `gate` (the joined heads times sigmoid(W_g y)
 before the output projection), `bias` (q, k, v and the output projection have biases), `chunk` (a query sees
 the keys of its own chunk of that many positions only, the chunks counted from the sequence's start),
-`softcap` (a scaled score s becomes softcap tanh(s / softcap) before the softmax). Such a part filters, norms
+`softcap` (a scaled score s becomes softcap tanh(s / softcap) before the softmax), `difference` (a head is the
+difference of two softmax attentions, its maps, over the same values: q and k have two maps a head, map by map;
+o = a1 - lambda a2 with lambda = exp(sum lq1 lk1) - exp(sum lq2 lk2) + difference, then o over its root mean square
+times 1 - difference, before the gate), `keys_are_values` (the values are the keys as projected, before norm and
+rotation), a position of the kind "rope_halves" (halves turn). Such a part filters, norms
 (over the whole projection, or head by head with weights that all heads share), rotates and writes the cache in
-one kernel of its own; rotation and values of another size than the keys go together there.
+one kernel of its own; rotation and values of another size than the keys go together there. Without a filter and a
+norm over the whole projection that kernel is heads.prepare, and for one token a sequence in bfloat16 it is the decode
+attention itself (mfma.attention_decode_heads), the heads' difference, gate and own size included. The two maps of a
+head are two query heads of one kept key, which holds both maps' keys side by side, with zeros in a query where
+the other map lies: the values are kept and read once.
 
 Three further options go with either form (not in the reference): `keep_first` (with a window: the sequence's first
 so many keys are seen as well; the cache keeps their pages), `distance_bias=(bias_max,)` (a learned bias by the
@@ -45,7 +53,7 @@ import math
 import torch
 
 from ..cache import KVNeed, StateNeed
-from ..kernels import mfma, ops, recurrent
+from ..kernels import heads, mfma, ops, recurrent
 from ..weights import TensorNeed
 from .base import Part
 from .linear import Linear
@@ -68,6 +76,11 @@ def _sink_init(shape, gen, device, std, norm_std):
     return torch.randn(shape, generator=gen, device=device, dtype=torch.float32)
 
 
+def _lambda_init(shape, gen, device, std, norm_std):
+    """Vectors of a random model whose exponentiated dot products differ from one, not by an order of magnitude."""
+    return torch.randn(shape, generator=gen, device=device, dtype=torch.float32) * (0.4 / shape[0] ** 0.25)
+
+
 RANDOM_BIAS_ROWS = 32
 
 
@@ -84,9 +97,11 @@ class Attention(Part):
     def __init__(self, hidden_size, num_heads, num_kv_heads, head_dim, eps, position, names,
                  qk_norm=True, window=None, scale=None, shared=None, reads_cache_only=False,
                  value_dim=None, q_temp=None, conv=None, sink=False, gate=False, bias=False, chunk=None,
-                 softcap=None, keep_first=0, distance_bias=None):
+                 softcap=None, keep_first=0, distance_bias=None, difference=None, keys_are_values=False):
         """names: dict with q, k, v, o (and q_norm, k_norm when qk_norm is True or "whole"; q_conv, k_conv, v_conv
-        with conv; sink with sink=True; rel with distance_bias; g with gate; q_bias, k_bias, v_bias, o_bias with bias) -> tensor names.
+        with conv; sink with sink=True; rel with distance_bias; g with gate; q_bias, k_bias, v_bias, o_bias with bias;
+        lq1, lk1, lq2, lk2 with difference) -> tensor names.
+        bias: True, or "qkv" for queries, keys and values alone. difference: the constant of the two maps (None: one map).
         qk_norm: True (a weight [head_dim] each for queries and keys), "plain" (no weights), "whole" (over all
         heads of a token at once, weights of that size) or False.
         conv: taps of a filter along time on queries, keys and values (None: none).
@@ -117,7 +132,15 @@ class Attention(Part):
         if sink not in (True, False, "unit"):
             raise ValueError(f"sink is True, False or 'unit', not {sink!r}")
         self.unit_sink = sink == "unit"
-        self.sink, self.gate, self.bias = sink is True, bool(gate), bool(bias)
+        if bias not in (True, False, "qkv"):
+            raise ValueError(f"bias is True, False or 'qkv', not {bias!r}")
+        self.sink, self.gate, self.bias, self.o_bias = sink is True, bool(gate), bool(bias), bias is True
+        self.difference = None if difference is None else float(difference)
+        self.maps = 1 if difference is None else 2
+        self.keys_are_values = bool(keys_are_values)
+        self.hd = max(self.hd, self.maps * self.dim)
+        if self.keys_are_values and (self.maps != 1 or self.vdim != self.dim):
+            raise ValueError("values that are the keys have their size and go with one map a head")
         self.keep_first = int(keep_first)
         if self.keep_first < 0 or (self.keep_first and self.window is None):
             raise ValueError("keep_first is a number of positions and goes with a window")
@@ -135,7 +158,14 @@ class Attention(Part):
         self.sink_w = self.taps_w = self.bias_w = self.o_bias_w = None
         # the form with a kernel of its own before the attention (see the module's text)
         self.prepared = bool(self.taps or self.sink or self.gate or qk_norm == "whole" or self.bias or self.chunk
-                             or self.softcap or hasattr(self.position, "pair_rates"))
+                             or self.softcap or self.maps == 2 or self.keys_are_values or hasattr(self.position, "step_angles"))
+        self.filtered = bool(self.taps or qk_norm == "whole")       # prepared by the kernel with a filter
+        if self.filtered and (self.maps == 2 or self.keys_are_values or (
+                hasattr(self.position, "step_angles") and not hasattr(self.position, "pair_rates"))):
+            raise ValueError("a filter or a norm over the whole projection goes with one map a head, values of their own and "
+                             "neighbouring pairs that turn")
+        if self.maps == 2 and (sink or self.keep_first or self.bias_max is not None):
+            raise ValueError("two maps a head go without sinks, kept first keys and biases by distance")
         if self.prepared:
             if self.reads_cache_only or self.q_temp is not None or qk_norm == "plain" or \
                     self.position.rotation() is not None:
@@ -146,8 +176,13 @@ class Attention(Part):
                 raise ValueError(f"the filter takes up to {recurrent.MAX_TAPS} taps, not {self.taps}")
 
     @property
+    def kept_heads(self):
+        """Query heads as the attention kernels count them: a map each."""
+        return self.nq * self.maps
+
+    @property
     def q_dim(self):
-        return self.nq * self.hd
+        return self.kept_heads * self.hd
 
     @property
     def kv_dim(self):
@@ -169,7 +204,7 @@ class Attention(Part):
 
     def tensor_needs(self):
         n, W = self.names, self.hidden_size
-        needs = {n["q"]: TensorNeed((self.nq * self.dim, W)),
+        needs = {n["q"]: TensorNeed((self.nq * self.maps * self.dim, W)),
                  n["o"]: TensorNeed((W, self.nq * self.vdim))}
         if self.qk_norm == "whole":
             needs[n["q_norm"]] = TensorNeed((self.nq * self.dim,), "scale")
@@ -184,13 +219,18 @@ class Attention(Part):
         if self.gate:
             needs[n["g"]] = TensorNeed((self.nq * self.vdim, W))
         if self.bias:
-            needs[n["q_bias"]] = TensorNeed((self.nq * self.dim,), "bias", _bias_init)
-            needs[n["k_bias"]] = TensorNeed((self.nkv * self.dim,), "bias", _bias_init)
-            needs[n["v_bias"]] = TensorNeed((self.nkv * self.vdim,), "bias", _bias_init)
-            needs[n["o_bias"]] = TensorNeed((W,), "bias", _bias_init)
+            needs[n["q_bias"]] = TensorNeed((self.nq * self.maps * self.dim,), "bias", _bias_init)
+            needs[n["k_bias"]] = TensorNeed((self.nkv * self.maps * self.dim,), "bias", _bias_init)
+            if not self.keys_are_values:
+                needs[n["v_bias"]] = TensorNeed((self.nkv * self.vdim,), "bias", _bias_init)
+            if self.o_bias:
+                needs[n["o_bias"]] = TensorNeed((W,), "bias", _bias_init)
+        if self.maps == 2:
+            needs.update({n[k]: TensorNeed((self.dim,), "bias", _lambda_init) for k in ("lq1", "lk1", "lq2", "lk2")})
         if not self.reads_cache_only:
-            needs[n["k"]] = TensorNeed((self.nkv * self.dim, W))
-            needs[n["v"]] = TensorNeed((self.nkv * self.vdim, W))
+            needs[n["k"]] = TensorNeed((self.nkv * self.maps * self.dim, W))
+            if not self.keys_are_values:
+                needs[n["v"]] = TensorNeed((self.nkv * self.vdim, W))
         if self.qk_norm is True:
             needs[n["q_norm"]] = TensorNeed((self.dim,), "scale")
             if not self.reads_cache_only:
@@ -200,7 +240,7 @@ class Attention(Part):
     def _kept_size(self, rt):
         """The head size the kernels run at: the larger of keys and values, and in bfloat16 the next size
         that the matrix cores take, unless the rotation or a cache that another entry fills forbids it."""
-        size = max(self.dim, self.vdim)
+        size = max(self.maps * self.dim, self.vdim)
         if self.prepared:
             if rt.dtype == torch.bfloat16:
                 for takes in mfma.ATTENTION_HEAD_DIMS:
@@ -243,24 +283,67 @@ class Attention(Part):
         self.hd = self._kept_size(rt)
         # one fused projection [q | k | v | gate], the heads at their own sizes: the kernel that follows reads
         # its float32 sums where they lie and keeps the heads at the size the attention runs at
-        rows = [tensors[n[k]].to(rt.device) for k in ("q", "k", "v") + (("g",) if self.gate else ())]
+        stored = ("q", "k") if self.keys_are_values else ("q", "k", "v")
+        rows = [tensors[n[k]].to(rt.device) for k in stored + (("g",) if self.gate else ())]
         self.qkv = Linear(rt.weight(torch.cat(rows, 0)), scratch=rt.scratch)
-        self.proj_width = self.channels + (self.nq * self.vdim if self.gate else 0)
+        self.layout = heads.HeadsLayout(self.kept_heads, self.nkv, self.maps, self.dim, self.vdim, self.hd, self.keys_are_values)
+        self.proj_width = self.layout.channels + (self.nq * self.vdim if self.gate else 0)
+        if self.maps == 2:
+            dot = lambda a, b: float((tensors[n[a]].double() * tensors[n[b]].double()).sum())
+            self.lam = math.exp(dot("lq1", "lk1")) - math.exp(dot("lq2", "lk2")) + self.difference
         self.o = Linear(rt.weight(tensors[n["o"]]), scratch=rt.scratch)
         if self.qk_norm in ("whole", True):
             self.q_norm_w = rt.weight(tensors[n["q_norm"]], matrix=False)
             self.k_norm_w = rt.weight(tensors[n["k_norm"]], matrix=False)
         if self.bias:
-            self.bias_w = torch.cat([rt.weight(tensors[n[k]], matrix=False) for k in ("q_bias", "k_bias", "v_bias")],
-                                    0).contiguous()
-            self.o_bias_w = rt.weight(tensors[n["o_bias"]], matrix=False)
+            self.bias_w = torch.cat([rt.weight(tensors[n[k + "_bias"]], matrix=False) for k in stored], 0).contiguous()
+            if self.o_bias:
+                self.o_bias_w = rt.weight(tensors[n["o_bias"]], matrix=False)
         if self.taps:
             self.taps_w = torch.cat([rt.weight(tensors[n[k]], matrix=False) for k in ("q_conv", "k_conv", "v_conv")],
                                     0).contiguous()
         if self.sink:
             self.sink_w = rt.weight(tensors[n["sink"]], matrix=False)
 
-    def _forward_prepared(self, ctx, y, x):
+    def _forward_heads(self, ctx, y, x, row_scale=None):
+        rt, meta, L = ctx.rt, ctx.meta, self.layout
+        T = x.shape[0]
+        kv = ctx.cache.kv_view(ctx.cache_entry)
+        proj = rt.buffer("attn_proj", (T, self.proj_width), torch.float32)
+        angles, rot_dims, halves = self.position.step_angles(ctx) if hasattr(self.position, "step_angles") else (None, 0, False)
+        gate_off = L.channels if self.gate else None
+        plain_masks = not self.keep_first and self.distance_raw is None
+        fused = plain_masks and mfma.decode_heads_fusable(meta, kv, L, rt.dtype)
+        # (slices of K are added up by the kernels that read the projection, but for the one that only gates heads)
+        defer = rt.dtype == torch.bfloat16 and (self.hd == 128 if fused else self.maps == 2 or not self.gate)
+        slices = self.qkv.forward(y, proj, row_scale=row_scale, defer_slices=defer)
+        own = rt.buffer("attn_own", (T, self.nq * self.vdim))
+        mixing = {"lam": self.lam, "factor": 1.0 - self.difference} if self.maps == 2 else {}
+        if fused:
+            mfma.attention_decode_heads(proj, L, self.bias_w, self.q_norm_w, self.k_norm_w, angles, rot_dims, halves, self.eps, meta,
+                                        kv, own, self.scale, self.window, self.chunk, self.softcap, self.sink_w, gate_off,
+                                        slices=slices, scratch=rt.scratch, **mixing)
+        else:
+            q = rt.buffer("q", (T, self.q_dim))
+            heads.prepare(proj, L, self.bias_w, self.q_norm_w, self.k_norm_w, angles, rot_dims, halves, self.eps, meta, kv, q, slices)
+            attn = rt.buffer("attn", (T, self.q_dim))
+            self.attend(ctx, q, kv, attn)
+            if self.maps == 2:
+                heads.difference(attn, proj, gate_off, own, self.nq, self.hd, self.vdim, eps=self.eps, slices=slices, **mixing)
+            elif self.gate or self.hd != self.vdim:
+                ops.gate_heads(attn, proj if self.gate else None, L.channels, own, self.nq, self.hd, self.vdim)
+            else:
+                own = attn
+        if self.o_bias_w is None:
+            self.project_out(ctx, own, x)
+        else:
+            self.o.forward(own, x, accumulate=ctx.adds_to(x))
+            ops.add_bias(x, self.o_bias_w)
+
+    def _forward_prepared(self, ctx, y, x, row_scale=None):
+        if not self.filtered:
+            self._forward_heads(ctx, y, x, row_scale)
+            return
         rt = ctx.rt
         T = x.shape[0]
         kv = ctx.cache.kv_view(ctx.cache_entry)
@@ -318,13 +401,13 @@ class Attention(Part):
     def forward_from_residual(self, ctx, x, norm):
         """With few rows and bfloat16 weights no norm kernel runs: the projection takes what the
         product before left of the norm, or else does the norm itself on the way."""
-        if self.prepared:
+        if self.filtered:
             return False
         handed = ctx.take_handed(self.qkv, x)
         if handed is not None:
             self.forward(ctx, handed.xg, x, row_scale=handed.row_scale())
             return True
-        if not (hasattr(norm, "w") and hasattr(norm, "eps") and self.qkv.fuses_norm(x)):
+        if self.prepared or not (hasattr(norm, "w") and hasattr(norm, "eps") and self.qkv.fuses_norm(x)):
             return False
         self.forward(ctx, None, x, fused_norm=norm)
         return True
@@ -335,7 +418,7 @@ class Attention(Part):
 
     def forward(self, ctx, y, x, fused_norm=None, row_scale=None):
         if self.prepared:
-            self._forward_prepared(ctx, y, x)
+            self._forward_prepared(ctx, y, x, row_scale)
             return
         rt = ctx.rt
         T = x.shape[0]
@@ -387,10 +470,10 @@ class Attention(Part):
     def attend(self, ctx, q, kv, out):
         scale = self.scale if self.prepared else self.kernel_scale
         if q.dtype == torch.bfloat16:
-            if mfma.attention_supported(q, kv, self.nq, self.nkv, self.hd):
-                mfma.attention(q, ctx.meta, kv, out, self.nq, self.nkv, self.hd, scale, self.window,
+            if mfma.attention_supported(q, kv, self.kept_heads, self.nkv, self.hd):
+                mfma.attention(q, ctx.meta, kv, out, self.kept_heads, self.nkv, self.hd, scale, self.window,
                                scratch=ctx.rt.scratch, sinks=self.sink_w, chunk=self.chunk, softcap=self.softcap,
                                bias=self.distance_raw, keep_first=self.keep_first)
                 return
-        ops.attention_plain(q, ctx.meta, kv, out, self.nq, self.nkv, self.hd, scale, self.window, sinks=self.sink_w,
+        ops.attention_plain(q, ctx.meta, kv, out, self.kept_heads, self.nkv, self.hd, scale, self.window, sinks=self.sink_w,
                             chunk=self.chunk, softcap=self.softcap, bias=self.distance_plain, keep_first=self.keep_first)

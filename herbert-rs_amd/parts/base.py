@@ -20,7 +20,7 @@ and a mixer has
   cache_need() -> None, KVNeed, StateNeed or a tuple of them.
 A part whose forward() only enqueues GPU work sets `graph_safe = True`.
 """
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 from typing import Any
 
 import torch
@@ -197,6 +197,8 @@ class StepContext:
     # for the next entry's block, which the block before may add
     pass_input: Any = None
     next_pass_input: Any = None
+    # what position encodings have worked out for this step's positions (see position.TurnsByAngles)
+    angles: dict = field(default_factory=dict)
 
     def adds_to(self, x):
         """False if x are the context's fresh rows (the part's product stores), True if it has to add."""

@@ -72,6 +72,14 @@ class Linear:
         mfma.gemm_swiglu(a, self.weight, out, packed=self.packed, norm=norm, row_scale=row_scale,
                          scratch=self.scratch, activation=activation)
 
+    def activates(self, a):
+        """True if this product applies an activation to its sums in its epilogue (forward_activated)."""
+        return self.weight.dtype == torch.bfloat16 and (self.packed or mfma.gemm_supported(a, self.weight))
+
+    def forward_activated(self, a, out, activation, row_scale=None):
+        """out bf16 [M, N] = f(a @ W^T), f one of ops.UNARY_ACTIVATIONS."""
+        mfma.gemm_activated(a, self.weight, out, activation, packed=self.packed, row_scale=row_scale, scratch=self.scratch)
+
     def fuses_norm(self, x):
         """True if RMSNorm(x) @ W^T runs as one kernel for this input (few rows, bfloat16 weights)."""
         if self.weight.dtype != torch.bfloat16:

@@ -1,5 +1,5 @@
 """Dense feed-forwards without biases. "swiglu": down(f(gate(y)) * up(y)) with f = silu, or with `activation="gelu_tanh"`
-the tanh form of gelu or with `activation="relu"` max(z, 0). "squared_relu": down(max(up(y), 0)^2).
+the tanh form of gelu or with `activation="relu"` max(z, 0). "up_down": down(f(up(y))), f = max(z, 0)^2 ("squared_relu") or the exact gelu.
 
 crates/backends/backend_common/src/generic_mlp.rs:83-96 and kernels.rs:676-687
 of the reference; gate and up are one fused matrix here so that the activations
@@ -79,13 +79,18 @@ class SwiGLU(Part):
         ctx.project_out(self.down, act, x)
 
 
-@register("feed_forward", "squared_relu")
-class SquaredRelu(Part):
-    """down(max(up(y), 0)^2): two matrices, the activation on the first product's float32 sums."""
+@register("feed_forward", "up_down")
+class UpDown(Part):
+    """down(f(up(y))): two matrices with an activation between them, max(z, 0)^2 ("relu_squared") or the exact gelu
+    z (1 + erf(z / sqrt 2)) / 2 ("gelu"); in bfloat16 in the first product's epilogue."""
     graph_safe = True
+    stores_fresh_rows = True
 
-    def __init__(self, hidden_size, intermediate_size, names, shared=None):
+    def __init__(self, hidden_size, intermediate_size, names, shared=None, activation="gelu"):
         """names: dict with up, down -> tensor names."""
+        if activation not in ops.UNARY_ACTIVATIONS:
+            raise ValueError(f"the activation is one of {sorted(ops.UNARY_ACTIVATIONS)}, not {activation!r}")
+        self.activation = activation
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
         self.names = dict(names)
@@ -101,12 +106,30 @@ class SquaredRelu(Part):
         self.up = Linear(rt.weight(tensors[n["up"]]), scratch=rt.scratch)
         self.down = Linear(rt.weight(tensors[n["down"]]), scratch=rt.scratch)
 
-    def forward(self, ctx, y, x):
+    def forward_from_residual(self, ctx, x, norm):
+        """With few rows the product takes what the one before left of the norm."""
+        handed = ctx.take_handed(self.up, x)
+        if handed is None or not self.up.activates(handed.xg):
+            return False
+        self.forward(ctx, handed.xg, x, row_scale=handed.row_scale())
+        return True
+
+    def forward(self, ctx, y, x, row_scale=None):
         rt = ctx.rt
         T = x.shape[0]
-        z = rt.buffer("ff_up", (T, self.intermediate_size), torch.float32)
-        self.up.forward(y, z)
         act = rt.buffer("act", (T, self.intermediate_size))
-        ops.relu_squared(z, act)
-        left = ctx.leave_norm(self.down, x)
-        self.down.forward(act, x, accumulate=True, leave=None if left is None else left.leave())
+        if self.up.activates(y):
+            self.up.forward_activated(y, act, self.activation, row_scale=row_scale)
+        else:
+            z = rt.buffer("ff_up", (T, self.intermediate_size), torch.float32)
+            self.up.forward(y, z)
+            ops.activate(z, act, self.activation)
+        ctx.project_out(self.down, act, x)
+
+
+@register("feed_forward", "squared_relu")
+class SquaredRelu(UpDown):
+    """"up_down" with max(z, 0)^2."""
+
+    def __init__(self, hidden_size, intermediate_size, names, shared=None):
+        super().__init__(hidden_size, intermediate_size, names, shared, activation="relu_squared")

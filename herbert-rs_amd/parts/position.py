@@ -13,6 +13,7 @@ import math
 
 import torch
 
+from ..kernels import heads
 from .base import Part
 from .registry import register
 
@@ -109,8 +110,71 @@ class RotaryHalfSplit(Part):
         return self.rates, self.rotary_dims
 
 
+class TurnsByAngles(Part):
+    """Rotations without tables for all positions: rates [rotary_dims / 2] in float64, from which a step's angles are worked
+    out once for all layers that turn alike, so no table bounds the positions. A subclass has theta, rotary_dims, halves
+    (True: entry i turns with entry i + rotary_dims / 2; False: 2i with 2i + 1), amplitude (cosine and sine are
+    multiplied by it) and pair_rates_host()."""
+    graph_safe = True
+    halves = False
+    amplitude = 1.0
+
+    def pair_rates_host(self):
+        raise NotImplementedError
+
+    def load(self, tensors, rt):
+        self.rates = torch.tensor(self.pair_rates_host(), dtype=torch.float64).to(rt.device)
+
+    def rotation(self):
+        return None
+
+    def rotation_rates(self):
+        return None
+
+    def step_angles(self, ctx):
+        """(angles f32 [T, rotary_dims / 2, 2]: cosine and sine for the step's tokens, rotary_dims, halves)."""
+        table = ctx.angles.get(id(self))
+        if table is None:
+            table = ctx.rt.buffer(f"step angles {id(self)}", (ctx.meta.num_tokens, self.rotary_dims // 2, 2), torch.float32)
+            heads.step_angles(ctx.meta.positions, self.rates, self.amplitude, table)
+            ctx.angles[id(self)] = table
+        return table, self.rotary_dims, self.halves
+
+
+@register("position", "rope_halves")
+class RotaryHalves(TurnsByAngles):
+    """Rotation of halves: entries i and i + rotary_dims / 2 of a head turn by position x theta^(-2i / rotary_dims).
+    scaling = (factor, original, fast, slow): pair i keeps its rate up to i = lo, has it divided by factor from i = hi on, and
+    goes over in a straight line between; lo and hi are the (rounded outwards) pairs that turn `fast` and `slow` times in
+    `original` positions. Cosine and sine are then multiplied by 0.1 ln(factor) + 1."""
+    halves = True
+
+    def __init__(self, theta, rotary_dims, scaling=None):
+        if rotary_dims % 2 or rotary_dims <= 0:
+            raise ValueError("rotary_dims must be even and positive")
+        self.theta, self.rotary_dims = float(theta), int(rotary_dims)
+        self.scaling = None if scaling is None else tuple(float(v) for v in scaling)
+        if self.scaling is not None:
+            self.amplitude = 0.1 * math.log(self.scaling[0]) + 1.0
+        self.rates = None
+
+    def pair_rates_host(self):
+        dims = self.rotary_dims
+        rates = [self.theta ** (-2.0 * i / dims) for i in range(dims // 2)]
+        if self.scaling is None:
+            return rates
+        factor, original, fast, slow = self.scaling
+        turning = lambda times: dims * math.log(original / (2.0 * math.pi * times)) / (2.0 * math.log(self.theta))
+        lo, hi = max(math.floor(turning(fast)), 0), min(math.ceil(turning(slow)), dims - 1)
+        out = []
+        for i, rate in enumerate(rates):
+            ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+            out.append(rate / factor * ramp + rate * (1.0 - ramp))
+        return out
+
+
 @register("position", "rope_pairs")
-class RotaryPairs(Part):
+class RotaryPairs(TurnsByAngles):
     """Rotation of neighbouring pairs: entries 2i and 2i + 1 of a head's first `rotary_dims` turn by
     position x theta^(-2i / rotary_dims). No tables: a mixer's kernel takes the rates (float64) and computes
     a position's angle, its sine and its cosine itself, so no table bounds the positions.
@@ -118,8 +182,6 @@ class RotaryPairs(Part):
     divided by factor, one under original / high stays, and between the two, with
     s = (original / wavelength - low) / (high - low), the rate is (1 - s) rate / factor + s rate.
     scaling = ("linear", factor): every rate is divided by factor."""
-    graph_safe = True
-
     def __init__(self, theta, rotary_dims, scaling=None):
         if rotary_dims % 2 or rotary_dims <= 0:
             raise ValueError("rotary_dims must be even and positive")
@@ -148,15 +210,6 @@ class RotaryPairs(Part):
                     rate = (1.0 - s) * rate / factor + s * rate
             rates.append(rate)
         return rates
-
-    def load(self, tensors, rt):
-        self.rates = torch.tensor(self.pair_rates_host(), dtype=torch.float64).to(rt.device)
-
-    def rotation(self):
-        return None
-
-    def rotation_rates(self):
-        return None
 
     def pair_rates(self):
         """(rates float64 [rotary_dims / 2] on the GPU, rotary_dims)."""
