@@ -21,7 +21,7 @@ step is what the generation loop does for a token: the step function (a HIP-grap
 greedy choice on the GPU, and the chosen tokens read by the host, which as in that loop reads
 the tokens of a step while the next step, fed from the GPU, already runs.
 
-`--workload vipalorn|modasun|mefatar|bozasun|mutedra --size small|medium|wide` measures one of the other designs instead (random weights at
+`--workload vipalorn|modasun|mefatar|bozasun|mutedra|figalorn --size small|medium|wide` measures one of the other designs instead (random weights at
 sizes that resemble a real model's layers) beside the closest other model at equal size, through the generation
 loop; the default workload and its JSON line stay as they are.
 """
@@ -250,10 +250,29 @@ def mutedra_configs(size):
     return (mut,) + family_configs(size)[::-1]
 
 
+def figalorn_configs(size):
+    """(Figalorn config dict, Qwen3 config dict) of one size, as many layer runs as the dense decoder has layers: the first
+    two layers run twice. Layers take turns: a window of 1,024 keys whose values are the keys (a norm a head, the whole
+    head rotated by halves at rates scaled by a ramp, scores capped at 50), and the difference of two maps of half the
+    head's size (biases, a quarter of a map rotated by neighbouring pairs, chunks of 2,048 positions, a gate an entry); every
+    layer has two matrices with the exact gelu between them, together as large as the dense decoder's three."""
+    W, L, H, D, V, rank, rot, E, top, ff, vocab = FAMILY_SIZES[size]
+    mlp = {"kind": "dense", "ff": 3 * top * ff // 2}
+    window = {"heads": H, "kv_heads": H // 2, "dim": D, "vdim": D, "scale": D ** -0.5, "softcap": 50.0, "mask": {"size": 1024},
+              "rot": {"base": 10000.0, "dims": D, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    maps = {"heads": H, "kv_heads": H // 2, "dim": D // 2, "vdim": V, "scale": (D // 2) ** -0.5, "diff": 0.5, "mask": {"size": 2048},
+            "rot": {"base": 10000.0, "dims": D // 8, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    kinds = [("attention_2", window), ("attention", maps)]
+    layers = [{"type": kinds[i % 2][0], "mixer": kinds[i % 2][1], "mlp": mlp} for i in range(L - 2)]
+    fig = {"architecture": "Figalorn", "vocab": vocab, "width": W, "layers": layers, "norm": {"eps": 1e-5},
+           "loop": {"start": 0, "stop": 2, "times": 2}}
+    return fig, family_configs(size)[1]
+
+
 def run_family(args, names=("vipalorn", "qwen3"), configs=family_configs):
     """Prompt and decode throughput of a design at one size (random weights) beside the closest other model at
     equal size (Vipalorn beside the dense Qwen3 decoder, Modasun beside Vipalorn, Mefatar beside Modasun, Bozasun beside
-    Vipalorn, Mutedra beside the dense decoder and Vipalorn), all through the generation loop: prompts of 512 and 2,048 tokens alone, and batches of 1, 8 and 32 sequences of 1,024 prompt tokens
+    Vipalorn, Mutedra beside the dense decoder and Vipalorn, Figalorn beside the dense decoder), all through the generation loop: prompts of 512 and 2,048 tokens alone, and batches of 1, 8 and 32 sequences of 1,024 prompt tokens
     decoding `--steps` tokens each."""
     import torch
     import herbert_rs_amd as hb
@@ -323,9 +342,9 @@ def main():
     ap.add_argument("--no-sweep", action="store_true", help="time the full context only, not 512 and the mean")
     ap.add_argument("--no-long", action="store_true",
                     help="skip the further sizes and lengths (contexts of 16 K and 32 K, batch 128 and 256, long prompts)")
-    ap.add_argument("--size", default="medium", choices=sorted(FAMILY_SIZES), help="layer sizes of --workload vipalorn, modasun, mefatar, bozasun and mutedra")
+    ap.add_argument("--size", default="medium", choices=sorted(FAMILY_SIZES), help="layer sizes of --workload vipalorn, modasun, mefatar, bozasun, mutedra and figalorn")
     ap.add_argument("--workload", default="headline", choices=["headline", "qwen3-1.7b", "qwen3-32b", "vipalorn", "modasun", "mefatar", "bozasun",
-                                                                "mutedra"],
+                                                                "mutedra", "figalorn"],
                     help="headline: BASELINE.json configs[2]; qwen3-*: configs[3] and configs[4]; vipalorn, modasun, mefatar: "
                          "that design at --size beside the closest other model at equal size")
     ap.add_argument("--prefill-tokens", type=int, default=2048, help="length of the prompt of the prefill figure")
@@ -357,6 +376,9 @@ def main():
     if args.workload == "mutedra":
         print(json.dumps(run_family(args, names=("mutedra", "qwen3", "vipalorn"), configs=mutedra_configs)))
         return
+    if args.workload == "figalorn":
+        print(json.dumps(run_family(args, names=("figalorn", "qwen3"), configs=figalorn_configs)))
+        return 0
     if args.workload == "bozasun":
         print(json.dumps(run_family(args, names=("bozasun", "vipalorn"), configs=bozasun_configs)))
         return 0

@@ -901,42 +901,45 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
     float xq0[PRE], xq1[PRE], k0 = 0.f, k1 = 0.f, v0 = 0.f, v1 = 0.f;
     int new_page = 0;
     const float* qin = nullptr;
-    // FORM_HEADS: a lane holds the entries lane (and lane + 64) of a row of the projection
+    // FORM_HEADS: a lane holds the entries lane (and lane + 64) of a row of the projection. All of it is asked for without a
+    // condition in between (an address past a head's own entries is moved back to its first, and what it brings not used),
+    // so that nothing waits before everything is on its way.
     constexpr int E = HD > 64 ? HD / 64 : 1;
-    float hq[PRE][E], hk[E], hv[E], hqw[E], hkw[E];
+    float hq[PRE][E][QS], hk[E][QS], hv[E][QS], hqb[PRE][E], hkb[E], hvb[E], hqw[E], hkw[E];
     float2 turn = {1.f, 0.f};
     const float* hrow = nullptr;
-    auto channel = [&](int at) {
-        float part[QS];
+    const float* hbias = nullptr;
+    auto ask = [&](int first, int d, int size, float (&part)[QS], float& with) {
+        const int at = first + (d < size ? d : 0);
 #pragma unroll
         for (int i = 0; i < QS; ++i) part[i] = hrow[(size_t)i * hf.slice_stride + at];
+        with = hbias[at];
+    };
+    auto channel = [&](int d, int size, const float (&part)[QS], float with) {
         float sum = part[0];
 #pragma unroll
         for (int i = 1; i < QS; ++i) sum += part[i];
-        return hf.bias ? sum + hf.bias[at] : sum;
+        return d < size ? (hf.bias ? sum + with : sum) : 0.f;
     };
+    const int key_size = hf.maps * hf.dim, q_first = kvh * G * hf.dim;
     if (FUSED == FORM_HEADS) {
         hrow = hf.proj + (size_t)b * hf.ld;
-        if (lane < hf.rot_dims / 2) turn = hf.angles[(size_t)b * (hf.rot_dims / 2) + lane];
+        hbias = hf.bias ? hf.bias : hrow;
+        const float* const qw = hf.q_norm_w ? hf.q_norm_w : hrow;
+        const float* const kw = hf.q_norm_w ? hf.k_norm_w : hrow;
+        const int half = hf.rot_dims / 2;
+        if (half > 0) turn = hf.angles[(size_t)b * half + (lane < half ? lane : 0)];
+        if (writer) new_page = pt[page_at(hp)];
 #pragma unroll
         for (int e = 0; e < E; ++e) {
-            const int d = lane + 64 * e;
-            hqw[e] = hkw[e] = 1.f;
-            hk[e] = hv[e] = 0.f;
-            if (hf.q_norm_w && d < hf.dim) {
-                hqw[e] = hf.q_norm_w[d];
-                hkw[e] = hf.k_norm_w[d];
-            }
+            const int d = lane + 64 * e, dn = d < hf.dim ? d : 0;
+            hqw[e] = qw[dn];
+            hkw[e] = kw[dn];
 #pragma unroll
-            for (int it = 0; it < PRE; ++it)
-                hq[it][e] = d < hf.dim ? channel((kvh * G + (it < G ? it : G - 1)) * hf.dim + d) : 0.f;
-            if (writer) {
-                if (d < hf.maps * hf.dim) hk[e] = channel(hf.k_off + kvh * hf.maps * hf.dim + d);
-                if (hf.v_off == hf.k_off) hv[e] = hk[e];
-                else if (d < hf.vdim) hv[e] = channel(hf.v_off + kvh * hf.vdim + d);
-            }
+            for (int it = 0; it < PRE; ++it) ask(q_first + (it < G ? it : G - 1) * hf.dim, d, hf.dim, hq[it][e], hqb[it][e]);
+            ask(hf.k_off + kvh * key_size, d, key_size, hk[e], hkb[e]);
+            ask(hf.v_off + kvh * hf.vdim, d, hf.vdim, hv[e], hvb[e]);
         }
-        if (writer) new_page = pt[page_at(hp)];
     }
     if (FUSED == FORM_FUSED) {
         const float* row = fu.qkv + (size_t)b * (nq + 2 * nkv) * HD;
@@ -1034,53 +1037,76 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
     // (FORM_HEADS: a row of the projection normed, and the angles)
     __shared__ float hraw[FUSED == FORM_HEADS ? (PRE + 1) * HD : 1];
     __shared__ float2 hturn[FUSED == FORM_HEADS ? HD / 2 : 1];
-    auto heads_prologue = [&]() {
+    auto heads_prologue = [&]() __attribute__((always_inline)) {
         if (lane < HD / 2) hturn[lane] = turn;
-        // a row's entries times their norm into LDS; of a key with two maps each has a norm of its own
-        auto lay = [&](float (&x)[E], float (&w)[E], float* raw, int maps) {
-            float inv0 = 1.f, inv1 = 1.f;
-            if (hf.q_norm_w) {
-                float s0 = 0.f, s1 = 0.f;
+        const bool normed = hf.q_norm_w != nullptr;
+        // a row's entries, times their norm, into LDS (a query: one map)
+        auto lay = [&](const float (&x)[E], float* raw) __attribute__((always_inline)) {
+            float inv = 1.f;
+            if (normed) {
+                float ss = 0.f;
 #pragma unroll
-                for (int e = 0; e < E; ++e) {
-                    const int d = lane + 64 * e;
-                    if (d < hf.dim) s0 = fmaf(x[e], x[e], s0);
-                    else s1 = fmaf(x[e], x[e], s1);
-                }
+                for (int e = 0; e < E; ++e) ss = fmaf(x[e], x[e], ss);
+#pragma unroll
+                for (int off = 32; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+                inv = 1.0f / sqrtf(ss / (float)hf.dim + hf.eps);
+            }
+#pragma unroll
+            for (int e = 0; e < E; ++e)
+                if (lane + 64 * e < HD) raw[lane + 64 * e] = normed ? x[e] * inv * hqw[e] : x[e];
+        };
+        // a key: of two maps each has a norm of its own
+        auto lay_key = [&](const float (&x)[E], float* raw) __attribute__((always_inline)) {
+            float s0 = 0.f, s1 = 0.f;
+#pragma unroll
+            for (int e = 0; e < E; ++e) {
+                if (lane + 64 * e < hf.dim) s0 = fmaf(x[e], x[e], s0);
+                else s1 = fmaf(x[e], x[e], s1);
+            }
+            if (normed) {
 #pragma unroll
                 for (int off = 32; off > 0; off >>= 1) {
                     s0 += __shfl_xor(s0, off, 64);
                     s1 += __shfl_xor(s1, off, 64);
                 }
-                inv0 = 1.0f / sqrtf(s0 / (float)hf.dim + hf.eps);
-                inv1 = 1.0f / sqrtf(s1 / (float)hf.dim + hf.eps);
             }
+            const float inv0 = 1.0f / sqrtf(s0 / (float)hf.dim + hf.eps), inv1 = 1.0f / sqrtf(s1 / (float)hf.dim + hf.eps);
 #pragma unroll
             for (int e = 0; e < E; ++e) {
                 const int d = lane + 64 * e;
-                // (the second map's weights lie dim entries on: read again, a rare case)
-                const float wd = d < hf.dim || maps == 1 || !hf.q_norm_w ? w[e] : d < maps * hf.dim ? hf.k_norm_w[d - hf.dim] : 1.f;
-                if (d < HD) raw[d] = x[e] * (d < hf.dim ? inv0 : inv1) * wd;
+                if (d >= HD) continue;
+                float w = hkw[e];
+                if (normed && d >= hf.dim && d < key_size) w = hf.k_norm_w[d - hf.dim];      // (two normed maps: a rare case)
+                raw[d] = normed ? x[e] * (d < hf.dim ? inv0 : inv1) * w : x[e];
             }
         };
-        // entry d of the kept head; map < 0: a key, all maps
-        auto kept = [&](const float* raw, int d, int map) -> float {
+        const int half = hf.rot_dims / 2;
+        // entry d of the kept head; map < 0: a key, all maps. Two reads of LDS and one of the angles, whatever d is.
+        auto kept = [&](const float* raw, int d, int map) __attribute__((always_inline)) -> float {
             const int m = hf.maps == 2 && d >= hf.map_stride ? 1 : 0;
             const int e = d - m * hf.map_stride;
-            if (e >= hf.dim || (map >= 0 && m != map)) return 0.f;
-            const float* const r = raw + (map >= 0 ? 0 : m * hf.dim);
-            const float own = r[e];
-            if (e >= hf.rot_dims) return own;
-            const int half = hf.rot_dims / 2;
+            const bool there = e < hf.dim && (map < 0 || m == map), turns = e < hf.rot_dims;
             const bool second = hf.halves ? e >= half : (e & 1);
             const int i = hf.halves ? (second ? e - half : e) : e >> 1;
             const int other = hf.halves ? (second ? e - half : e + half) : e ^ 1;
-            const float2 t = hturn[i];
-            return second ? own * t.x + r[other] * t.y : own * t.x - r[other] * t.y;
+            const float* const r = raw + (map >= 0 ? 0 : m * hf.dim);
+            const float own = r[there ? e : 0], o = r[there && turns ? other : 0];
+            const float2 t = hturn[turns ? i : 0];
+            const float turned = own * t.x + (second ? o * t.y : -o * t.y);
+            return there ? (turns ? turned : own) : 0.f;
         };
-        if (writer) lay(hk, hkw, hraw + PRE * HD, hf.maps);
+        float x[PRE + 2][E];
 #pragma unroll
-        for (int it = 0; it < PRE; ++it) lay(hq[it], hqw, hraw + it * HD, 1);
+        for (int e = 0; e < E; ++e) {
+            const int d = lane + 64 * e;
+#pragma unroll
+            for (int it = 0; it < PRE; ++it) x[it][e] = channel(d, hf.dim, hq[it][e], hqb[it][e]);
+            x[PRE][e] = channel(d, key_size, hk[e], hkb[e]);
+            x[PRE + 1][e] = channel(d, hf.vdim, hv[e], hvb[e]);
+        }
+        if (writer) lay_key(x[PRE], hraw + PRE * HD);
+#pragma unroll
+        for (int it = 0; it < PRE; ++it) lay(x[it], hraw + it * HD);
         __syncthreads();
         if (writer) {
             const int in_page = hi % PAGE;
@@ -1091,7 +1117,7 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
                 const int d = lane + 64 * e;
                 if (d < HD) {
                     kdst[d] = hb_from_float<bf16>(kept(hraw + PRE * HD, d, -1));
-                    vdst[(size_t)d * PAGE] = hb_from_float<bf16>(d < hf.vdim ? hv[e] : 0.f);
+                    vdst[(size_t)d * PAGE] = hb_from_float<bf16>(x[PRE + 1][e]);
                 }
             }
             __threadfence_block();      // this wave's later loads of that page see what it has just written
@@ -1100,33 +1126,33 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
             if (it0 > 0) {
                 __syncthreads();
 #pragma unroll
+                for (int e = 0; e < E; ++e)
+#pragma unroll
+                    for (int it = 0; it < PRE; ++it)
+                        ask(q_first + (it0 + it < G ? it0 + it : G - 1) * hf.dim, lane + 64 * e, hf.dim, hq[it][e], hqb[it][e]);
+#pragma unroll
                 for (int it = 0; it < PRE; ++it) {
-                    const int hl = it0 + it < G ? it0 + it : G - 1;
 #pragma unroll
-                    for (int e = 0; e < E; ++e) {
-                        const int d = lane + 64 * e;
-                        hq[it][e] = d < hf.dim ? channel((kvh * G + hl) * hf.dim + d) : 0.f;
-                    }
+                    for (int e = 0; e < E; ++e) x[it][e] = channel(lane + 64 * e, hf.dim, hq[it][e], hqb[it][e]);
+                    lay(x[it], hraw + it * HD);
                 }
-#pragma unroll
-                for (int it = 0; it < PRE; ++it) lay(hq[it], hqw, hraw + it * HD, 1);
                 __syncthreads();
             }
 #pragma unroll
             for (int it = 0; it < PRE; ++it) {
                 const int hl = it0 + it;
-                if (hl >= G) break;
 #pragma unroll
                 for (int e = 0; e < E; ++e) {
                     const int d = lane + 64 * e;
-                    if (d < HD) qs[hl * HD + d] = hb_from_float<bf16>(kept(hraw + it * HD, d, hf.maps == 2 ? (hl & 1) : 0));
+                    const float v = kept(hraw + it * HD, d < HD ? d : 0, hf.maps == 2 ? (hl & 1) : 0);
+                    if (d < HD && hl < G) qs[hl * HD + d] = hb_from_float<bf16>(v);
                 }
             }
         }
     };
     // norm and rotation of the new key and of the query heads; the key and the value go to the pages,
     // the queries to LDS, from where each lane takes its operand
-    auto prologue = [&]() {
+    auto prologue = [&]() __attribute__((always_inline)) {
         if (FUSED == FORM_HEADS) {
             heads_prologue();
             return;
@@ -1268,13 +1294,24 @@ attn_decode_kernel(const bf16* __restrict__ q, bf16* __restrict__ k_cache, bf16*
         const int own_head = (kvh * G + c32) / ho.maps;
         if (c32 < G && (ho.maps == 1 || (c32 & 1) == 0)) {
             bf16* const dst = out + ((size_t)b * (nq / ho.maps) + own_head) * ho.vdim;
+            const float* const gp = ho.gate ? ho.gate + (size_t)b * ho.gate_ld + own_head * ho.vdim : nullptr;
 #pragma unroll
-            for (int d = 0; d < HD / 32; ++d)
+            for (int d = 0; d < HD / 32; ++d) {
+                float g[16];
+                auto entry = [&](int i) { return d * 32 + 8 * (i >> 2) + 4 * g2 + (i & 3); };
+                if (gp) {
 #pragma unroll
-                for (int i = 0; i < 16; ++i) {
-                    const int at = d * 32 + 8 * (i >> 2) + 4 * g2 + (i & 3);
-                    if (at < ho.vdim) dst[at] = hb_from_float<bf16>(oacc[d][i] * scale * gate_of(ho, b, own_head * ho.vdim + at));
+                    for (int i = 0; i < 16; ++i) g[i] = gp[entry(i) < ho.vdim ? entry(i) : 0];
+                    for (int s = 1; s < ho.gate_slices; ++s)
+#pragma unroll
+                        for (int i = 0; i < 16; ++i) g[i] += gp[(size_t)s * ho.gate_stride + (entry(i) < ho.vdim ? entry(i) : 0)];
+#pragma unroll
+                    for (int i = 0; i < 16; ++i) oacc[d][i] *= 1.0f / (1.0f + __expf(-g[i]));
                 }
+#pragma unroll
+                for (int i = 0; i < 16; ++i)
+                    if (entry(i) < ho.vdim) dst[entry(i)] = hb_from_float<bf16>(oacc[d][i] * scale);
+            }
         }
         return;
     }

@@ -48,6 +48,7 @@ struct HeadsLayout {
     int k_off, v_off;            // first key and value column; v_off == k_off: the values are the keys as projected
     int rot_dims, halves;        // pairs (i, i + rot_dims / 2) with halves, else (2i, 2i + 1); 0: no rotation
     float eps;
+    int octets;                  // maps and the turned part begin and end at multiples of eight entries (of sixteen with halves)
 };
 
 // QS: the projection was cut into QS slices of K whose sums lie slice_stride floats apart; they are added up in their order.
@@ -182,7 +183,65 @@ heads_prepare_kernel(const float* __restrict__ proj, int ld, size_t slice_stride
             const int page = page_table[(size_t)slots[seq_of[t]] * max_pages + pos / page_size];
             return k_cache + (((size_t)page * L.nkv + g) * page_size + pos % page_size) * L.hd;
         };
-        if (L.hd % 8 == 0) {
+        if (L.octets) {
+            // eight entries of a kept head belong to one map and turn together or not at all, each with a neighbour among
+            // them or, with halves, with one of eight others in a row
+            const int per = L.hd / 8;
+#pragma unroll 2
+            for (int i = tid; i < rows * per; i += 256) {
+                const int r = i / per, d = (i - r * per) * 8;
+                const int m = L.maps == 2 && d >= L.map_stride ? 1 : 0;
+                const int e0 = d - m * L.map_stride;
+                const bool there = e0 < L.dim && (!is_q || m == q_map);
+                const int e = there ? e0 : 0;
+                const float* const row = raw + r * LW + (is_q ? 0 : m * L.dim) + e;
+                const float scale = norm_w ? inv[r * maps + (is_q ? 0 : m)] : 1.0f;
+                float v[8], o[8];
+#pragma unroll
+                for (int k = 0; k < 8; ++k) v[k] = row[k];
+                if (norm_w) {
+                    const f32x4 w0 = *(const f32x4*)(norm_w + e), w1 = *(const f32x4*)(norm_w + e + 4);
+#pragma unroll
+                    for (int k = 0; k < 8; ++k) v[k] *= scale * (k < 4 ? w0[k & 3] : w1[k & 3]);
+                }
+                if (e < L.rot_dims) {
+                    const float2* const at = angles + (size_t)(t0 + r) * half;
+                    if (L.halves) {
+                        const bool second = e >= half;
+                        const int other = second ? -half : half;
+#pragma unroll
+                        for (int k = 0; k < 8; ++k) o[k] = row[other + k];
+                        if (norm_w) {
+                            const f32x4 w0 = *(const f32x4*)(norm_w + e + other), w1 = *(const f32x4*)(norm_w + e + other + 4);
+#pragma unroll
+                            for (int k = 0; k < 8; ++k) o[k] *= scale * (k < 4 ? w0[k & 3] : w1[k & 3]);
+                        }
+                        const f32x4* const cs4 = (const f32x4*)(at + (second ? e - half : e));
+#pragma unroll
+                        for (int k = 0; k < 8; k += 2) {
+                            const f32x4 cs = cs4[k / 2];
+                            v[k] = v[k] * cs[0] + (second ? o[k] : -o[k]) * cs[1];
+                            v[k + 1] = v[k + 1] * cs[2] + (second ? o[k + 1] : -o[k + 1]) * cs[3];
+                        }
+                    } else {
+                        const f32x4* const cs4 = (const f32x4*)(at + e / 2);
+                        const f32x4 cs0 = cs4[0], cs1 = cs4[1];
+#pragma unroll
+                        for (int k = 0; k < 8; k += 2) {
+                            const f32x4 cs = k < 4 ? cs0 : cs1;
+                            const float c = cs[(k & 2)], sn = cs[(k & 2) + 1], u = v[k], w = v[k + 1];
+                            v[k] = u * c - w * sn;
+                            v[k + 1] = w * c + u * sn;
+                        }
+                    }
+                }
+                if (!there) {
+#pragma unroll
+                    for (int k = 0; k < 8; ++k) v[k] = 0.f;
+                }
+                store_eight<T>(destination(r) + d, v);
+            }
+        } else if (L.hd % 8 == 0) {
             const int per = L.hd / 8;
             for (int i = tid; i < rows * per; i += 256) {
                 const int r = i / per, d = (i - r * per) * 8;
@@ -233,7 +292,9 @@ extern "C" int hb_heads_prepare(const float* proj, int ld, int slices, size_t sl
     HB_REQUIRE(slices == 1 || slice_stride >= (size_t)T * ld, "heads: slices overlap");
     const dim3 grid((T + tile - 1) / tile, nq + nkv + (v_off == k_off ? 0 : nkv));
     HB_REQUIRE(grid.y <= 65535, "heads: too many heads for the grid");
-    const HeadsLayout L = {nq, nkv, maps, dim, vdim, hd, map_stride, k_off, v_off, rot_dims, halves, eps};
+    const HeadsLayout L = {nq, nkv, maps, dim, vdim, hd, map_stride, k_off, v_off, rot_dims, halves, eps,
+                           dim % 8 == 0 && hd % 8 == 0 && map_stride % 8 == 0 && rot_dims % (halves ? 16 : 8) == 0 &&
+                               (((uintptr_t)angles | (uintptr_t)q_norm_w | (uintptr_t)k_norm_w) & 15) == 0};
     const bool quads = dim % 4 == 0 && vdim % 4 == 0 && ld % 4 == 0 && k_off % 4 == 0 && v_off % 4 == 0 && slice_stride % 4 == 0 &&
                        (((uintptr_t)proj | (uintptr_t)bias) & 15) == 0;
 #define HB_HEADS(TV, QSV, QD)                                                                                            \
@@ -245,10 +306,11 @@ extern "C" int hb_heads_prepare(const float* proj, int ld, int slices, size_t sl
         HB_REQUIRE(slices == 1, "heads: a float32 projection is not cut into slices");
         HB_HEADS_Q(float, 1);
     } else if (dtype == HB_BF16) {
+        HB_REQUIRE(slices == 1 || quads, "heads: slices of the projection are taken where its columns come in fours");
         if (slices == 1) HB_HEADS_Q(bf16, 1);
-        else if (slices == 2) HB_HEADS_Q(bf16, 2);
-        else if (slices == 4) HB_HEADS_Q(bf16, 4);
-        else if (slices == 8) HB_HEADS_Q(bf16, 8);
+        else if (slices == 2) HB_HEADS(bf16, 2, true);
+        else if (slices == 4) HB_HEADS(bf16, 4, true);
+        else if (slices == 8) HB_HEADS(bf16, 8, true);
         else HB_REQUIRE(false, "heads: %d slices of the projection are not taken", slices);
     } else {
         HB_REQUIRE(false, "heads: unknown dtype %d", dtype);
@@ -314,6 +376,59 @@ heads_difference_kernel(const T* __restrict__ attn, const float* __restrict__ ga
     }
 }
 
+// The same for heads of up to 128 in steps of four: half a wave a (token, head), four entries a lane.
+template <class T>
+__global__ void __launch_bounds__(256)
+heads_difference_quads_kernel(const T* __restrict__ attn, const float* __restrict__ gate, int ld, int slices, size_t slice_stride,
+                              T* __restrict__ out, int heads, int hd, int vdim, float lambda, float factor, float eps, unsigned total) {
+    const unsigned th = blockIdx.x * 8u + (threadIdx.x >> 5);
+    const int d = (threadIdx.x & 31) * 4;
+    const bool mine = th < total && d < vdim;
+    const unsigned at = mine ? th : 0, t = at / heads, h = at - t * heads;
+    const int dd = mine ? d : 0;
+    auto four = [](const T* p) {
+        f32x4 v;
+        if constexpr (sizeof(T) == 4) {
+            v = *(const f32x4*)p;
+        } else {
+            const bf16x4 raw = *(const bf16x4*)p;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = (float)raw[e];
+        }
+        return v;
+    };
+    const T* const a1 = attn + (size_t)at * 2 * hd + dd;
+    const f32x4 x1 = four(a1), x2 = four(a1 + hd);
+    f32x4 g = {0.f, 0.f, 0.f, 0.f};
+    if (gate) {
+        const float* const grow = gate + (size_t)t * ld + (size_t)h * vdim + dd;
+        g = *(const f32x4*)grow;
+        for (int s = 1; s < slices; ++s) g += *(const f32x4*)(grow + (size_t)s * slice_stride);
+    }
+    f32x4 o;
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        o[e] = x1[e] - lambda * x2[e];
+        if (mine) ss = fmaf(o[e], o[e], ss);
+    }
+#pragma unroll
+    for (int off = 16; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+    const float scale = factor / sqrtf(ss / (float)vdim + eps);
+    if (!mine) return;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] *= gate ? scale / (1.0f + __expf(-g[e])) : scale;
+    T* const dst = out + (size_t)th * vdim + d;
+    if constexpr (sizeof(T) == 4) {
+        *(f32x4*)dst = o;
+    } else {
+        bf16x4 b;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) b[e] = (__bf16)o[e];
+        *(bf16x4*)dst = b;
+    }
+}
+
 extern "C" int hb_heads_difference(const void* attn, int dtype, const float* gate, int ld, int slices, size_t slice_stride,
                                    void* out, int T, int heads, int hd, int vdim, float lambda, float factor, float eps,
                                    hipStream_t stream) {
@@ -323,14 +438,25 @@ extern "C" int hb_heads_difference(const void* attn, int dtype, const float* gat
     const size_t total = (size_t)T * heads;
     HB_REQUIRE(total < (1ull << 32), "difference: too many heads");
     const unsigned blocks = (unsigned)((total + 3) / 4);
+    HB_REQUIRE(dtype == HB_F32 || dtype == HB_BF16, "difference: unknown dtype %d", dtype);
+    if (vdim <= 128 && vdim % 4 == 0 && hd % 4 == 0 && (!gate || (ld % 4 == 0 && slice_stride % 4 == 0)) &&
+        (((uintptr_t)attn | (uintptr_t)gate | (uintptr_t)out) & 15) == 0 && total < (1ull << 31)) {
+        const unsigned eighths = (unsigned)((total + 7) / 8);
+        if (dtype == HB_F32)
+            heads_difference_quads_kernel<float><<<eighths, 256, 0, stream>>>((const float*)attn, gate, ld, slices, slice_stride,
+                                                                              (float*)out, heads, hd, vdim, lambda, factor, eps, (unsigned)total);
+        else
+            heads_difference_quads_kernel<bf16><<<eighths, 256, 0, stream>>>((const bf16*)attn, gate, ld, slices, slice_stride,
+                                                                             (bf16*)out, heads, hd, vdim, lambda, factor, eps, (unsigned)total);
+        HB_CHECK_LAUNCH("heads_difference");
+        return 0;
+    }
     if (dtype == HB_F32)
         heads_difference_kernel<float><<<blocks, 256, 0, stream>>>((const float*)attn, gate, ld, slices, slice_stride, (float*)out,
                                                                    heads, hd, vdim, lambda, factor, eps, total);
-    else if (dtype == HB_BF16)
+    else
         heads_difference_kernel<bf16><<<blocks, 256, 0, stream>>>((const bf16*)attn, gate, ld, slices, slice_stride, (bf16*)out,
                                                                   heads, hd, vdim, lambda, factor, eps, total);
-    else
-        HB_REQUIRE(false, "difference: unknown dtype %d", dtype);
     HB_CHECK_LAUNCH("heads_difference");
     return 0;
 }

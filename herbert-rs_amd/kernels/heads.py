@@ -32,6 +32,11 @@ class HeadsLayout:
         return self.hd // 2 if self.maps == 2 and self.hd % 2 == 0 else self.dim
 
     @property
+    def adds_slices(self):
+        """True if `prepare` adds up the K slices of such a projection (of a row width that four divides) itself."""
+        return self.dim % 4 == 0 and self.vdim % 4 == 0
+
+    @property
     def k_off(self):
         return self.nq * self.dim
 

@@ -315,7 +315,8 @@ class Attention(Part):
         plain_masks = not self.keep_first and self.distance_raw is None
         fused = plain_masks and mfma.decode_heads_fusable(meta, kv, L, rt.dtype)
         # (slices of K are added up by the kernels that read the projection, but for the one that only gates heads)
-        defer = rt.dtype == torch.bfloat16 and (self.hd == 128 if fused else self.maps == 2 or not self.gate)
+        defer = rt.dtype == torch.bfloat16 and (self.hd == 128 if fused else
+                                                    L.adds_slices and self.proj_width % 4 == 0 and (self.maps == 2 or not self.gate))
         slices = self.qkv.forward(y, proj, row_scale=row_scale, defer_slices=defer)
         own = rt.buffer("attn_own", (T, self.nq * self.vdim))
         mixing = {"lam": self.lam, "factor": 1.0 - self.difference} if self.maps == 2 else {}
