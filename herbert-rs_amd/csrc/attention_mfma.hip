@@ -346,6 +346,97 @@ struct PageBias {
 };
 #define PAGE_BIAS_FLOATS 128
 
+// How the heads' outputs leave (own: at their own size vdim, a row [heads x vdim]; else at the kept size): with two maps
+// neighbouring query heads are a head's maps, o = a1 - lambda a2, over its root mean square, times factor; then times
+// sigmoid of the gate's column (null: none), which may lie in slices of K still.
+struct HeadsOut {
+    int own, maps, vdim;
+    const float* gate;
+    int gate_ld, gate_slices;
+    size_t gate_stride;
+    float lambda, factor, eps;
+};
+
+__device__ __forceinline__ float gate_of(const HeadsOut& ho, size_t row, int column) {
+    if (!ho.gate) return 1.0f;
+    const float* const p = ho.gate + row * ho.gate_ld + column;
+    float part[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) part[i] = i < ho.gate_slices ? p[(size_t)i * ho.gate_stride] : 0.f;
+    float g = part[0];
+#pragma unroll
+    for (int i = 1; i < 8; ++i) g += part[i];
+    return 1.0f / (1.0f + expf(-g));
+}
+
+// The end of a prompt kernel's wave where the heads leave at their own size (OWN): a lane has row c32's sums o of one query head
+// (times 1 / its denominator); with two maps the wave of the second (`second`) hands its sums over through `hand` ([value]
+// [lane], the pair's own stretch of LDS) to the first's, which leaves their difference. Every wave of the workgroup
+// comes here (there is a barrier). row: the step's row of this lane; stores: false for a lane or wave without one.
+template <int HD>
+__device__ __forceinline__ void leave_own(f32x16 (&oacc)[HD / 32], float inv, float* hand, bool second, bool stores,
+                                          size_t row, int own_head, int heads, int g2, const HeadsOut& ho, bf16* out) {
+#pragma unroll
+    for (int d = 0; d < HD / 32; ++d)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) oacc[d][i] *= inv;
+    float scale = 1.f;
+    if (ho.maps == 2) {
+        if (second)
+#pragma unroll
+            for (int d = 0; d < HD / 32; ++d)
+#pragma unroll
+                for (int i = 0; i < 16; ++i) hand[(d * 16 + i) * 64] = oacc[d][i];
+        __syncthreads();
+        if (second) return;
+        float ss = 0.f;
+#pragma unroll
+        for (int d = 0; d < HD / 32; ++d)
+#pragma unroll
+            for (int i = 0; i < 16; ++i) {
+                oacc[d][i] -= ho.lambda * hand[(d * 16 + i) * 64];
+                ss = fmaf(oacc[d][i], oacc[d][i], ss);
+            }
+        ss += __shfl_xor(ss, 32, 64);
+        scale = ho.factor / sqrtf(ss / (float)ho.vdim + ho.eps);          // (entries beyond vdim are zeros)
+    }
+    if (!stores) return;
+    bf16* const dst = out + (row * heads + own_head) * ho.vdim;
+    const float* const gate = ho.gate ? ho.gate + row * ho.gate_ld + (size_t)own_head * ho.vdim : nullptr;
+    const bool fours = (ho.vdim & 3) == 0 && (ho.gate_ld & 3) == 0 && (ho.gate_stride & 3) == 0 && (((uintptr_t)ho.gate) & 15) == 0;
+#pragma unroll
+    for (int d = 0; d < HD / 32; ++d)
+#pragma unroll
+        for (int qd = 0; qd < 4; ++qd) {
+            const int at = d * 32 + 8 * qd + 4 * g2;
+            f32x4 v;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] = oacc[d][4 * qd + r] * scale;
+            if (fours) {
+                if (at >= ho.vdim) continue;
+                if (gate) {
+                    f32x4 g = *(const f32x4*)(gate + at);
+                    for (int s = 1; s < ho.gate_slices; ++s) g += *(const f32x4*)(gate + (size_t)s * ho.gate_stride + at);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) v[r] *= __builtin_amdgcn_rcpf(1.0f + __expf(-g[r]));
+                }
+                bf16x4 b;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) b[r] = (__bf16)v[r];
+                *(bf16x4*)((__bf16*)dst + at) = b;
+            } else {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    if (at + r >= ho.vdim) continue;
+                    float g = 0.f;
+                    if (gate)
+                        for (int s = 0; s < ho.gate_slices; ++s) g += gate[(size_t)s * ho.gate_stride + at + r];
+                    dst[at + r] = hb_from_float<bf16>(gate ? v[r] / (1.0f + __expf(-g)) : v[r]);
+                }
+            }
+        }
+}
+
 // A workgroup: 32 queries x up to 4 query heads of one kv head, by eight waves in two groups of
 // four (a wave a head in each group). The groups take the tile's pages in turn, the first the
 // even ones and the second the odd ones, each with a reference, a sum and an output of its
@@ -358,7 +449,8 @@ struct PageBias {
 // reads of 16 rows at one chunk fall into 16 different bank groups.
 // Workgroups are numbered by falling work (the host sorts the tiles): a CU that is done takes
 // the heaviest tile left.
-template <int HD, bool EXT>
+// OWN: the heads leave at their own size, their maps' difference taken and gated (HeadsOut).
+template <int HD, bool EXT, bool OWN>
 __global__ void __launch_bounds__(512, 1)
 attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache,
                     const bf16* __restrict__ v_cache, bf16* __restrict__ out,
@@ -366,7 +458,7 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache
                     const int* __restrict__ tile_rows, const int* __restrict__ positions,
                     const int* __restrict__ slots, const int* __restrict__ page_table, int max_pages, int nq,
                     int nkv, float c, int window, int per_tile, const float* __restrict__ sinks, int chunked,
-                    float cap, AttnExtras ext) {
+                    float cap, AttnExtras ext, HeadsOut ho) {
     constexpr int KCH = HD / 8;                   // 16-byte chunks of a key row
     constexpr int KRPB = 128 / HD > 0 ? 128 / HD : 1;   // key rows in 256 bytes
     constexpr int KROWS = 512 / HD;               // key rows a load instruction brings (1 KB)
@@ -541,8 +633,8 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache
             for (int i = 0; i < 16; ++i) hand[(2 + d * 16 + i) * 64] = oacc[d][i];
     }
     __syncthreads();
-    if (grp == 1 || !active || c32 >= rows) return;
-    {
+    if (!OWN && (grp == 1 || !active || c32 >= rows)) return;
+    if (grp == 0) {
         const float m1 = hand[0], l1 = hand[64];
         const float mm = fmaxf(m, m1);
         // (a group without a visible key has the reference -inf, the sum 0 and the output 0)
@@ -558,6 +650,13 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache
     l += __shfl_xor(l, 32, 64);
     if (sinks) l += sink_share(sinks[h], m, c);
     const float inv = l > 0.f ? 1.0f / l : 0.f;
+    if constexpr (OWN) {
+        // (a wave's stretch of the hand-over above is its own by now: read by its first group, in order, before it writes)
+        float* const pair = (float*)attn_lds + (size_t)(wave | (ho.maps == 2 ? 1 : 0)) * (HD / 2 + 2) * 64 + lane;
+        leave_own<HD>(oacc, inv, pair, grp == 0 && ho.maps == 2 && (wave & 1), grp == 0 && active && c32 < rows, row0 + c32,
+                      h / ho.maps, nq / ho.maps, g2, ho, out);
+        return;
+    }
     bf16* orow = out + ((size_t)(row0 + c32) * nq + h) * HD;
 #pragma unroll
     for (int d = 0; d < HD / 32; ++d)
@@ -579,7 +678,7 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache
 // Every wave issues the same number of loads in every step (past the last page: that page again,
 // into a stage nobody reads any more), so that the wait before the barrier can count: all but
 // the loads of the step before have landed.
-template <int HD, bool EXT>
+template <int HD, bool EXT, bool OWN>
 __global__ void __launch_bounds__(512, 1)
 attn_prefill_long_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_cache,
                          const bf16* __restrict__ v_cache, bf16* __restrict__ out,
@@ -587,7 +686,7 @@ attn_prefill_long_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
                          const int* __restrict__ tile_rows, const int* __restrict__ positions,
                          const int* __restrict__ slots, const int* __restrict__ page_table, int max_pages,
                          int nq, int nkv, float c, int window, int per_tile,
-                         const float* __restrict__ sinks, int chunked, float cap, AttnExtras ext) {
+                         const float* __restrict__ sinks, int chunked, float cap, AttnExtras ext, HeadsOut ho) {
     constexpr int KCH = HD / 8;
     constexpr int KRPB = 128 / HD > 0 ? 128 / HD : 1;
     constexpr int KROWS = 512 / HD;
@@ -753,10 +852,17 @@ attn_prefill_long_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
         if (i + 1 < steps) step(i + 1, sb, sa);
     }
     hb_wait_vmcnt<0>();          // nothing of this workgroup's is in flight when it ends
-    if (!active || c32 >= rows) return;
+    if (!OWN && (!active || c32 >= rows)) return;
     l += __shfl_xor(l, 32, 64);
     if (sinks) l += sink_share(sinks[h], m, c);
     const float inv = l > 0.f ? 1.0f / l : 0.f;
+    if constexpr (OWN) {
+        __syncthreads();         // nobody reads the rings any more
+        float* const pair = (float*)attn_lds + (size_t)(wave8 >> 1) * (HD / 2) * 64 + lane;
+        leave_own<HD>(oacc, inv, pair, ho.maps == 2 && (wave & 1), active && c32 < rows, row0 + c32, h / ho.maps, nq / ho.maps, g2,
+                      ho, out);
+        return;
+    }
     bf16* orow = out + ((size_t)(row0 + c32) * nq + h) * HD;
 #pragma unroll
     for (int d = 0; d < HD / 32; ++d)
@@ -811,29 +917,6 @@ struct HeadsFusion {
     int maps, dim, vdim, map_stride, k_off, v_off;
     float eps;
 };
-
-// How the heads' outputs leave (own: at their own size vdim, a row [heads x vdim]; else at the kept size): with two maps
-// neighbouring query heads are a head's maps, o = a1 - lambda a2, over its root mean square, times factor; then times
-// sigmoid of the gate's column (null: none), which may lie in slices of K still.
-struct HeadsOut {
-    int own, maps, vdim;
-    const float* gate;
-    int gate_ld, gate_slices;
-    size_t gate_stride;
-    float lambda, factor, eps;
-};
-
-__device__ __forceinline__ float gate_of(const HeadsOut& ho, size_t row, int column) {
-    if (!ho.gate) return 1.0f;
-    const float* const p = ho.gate + row * ho.gate_ld + column;
-    float part[8];
-#pragma unroll
-    for (int i = 0; i < 8; ++i) part[i] = i < ho.gate_slices ? p[(size_t)i * ho.gate_stride] : 0.f;
-    float g = part[0];
-#pragma unroll
-    for (int i = 1; i < 8; ++i) g += part[i];
-    return 1.0f / (1.0f + expf(-g));
-}
 
 template <int HD, int FUSED, bool EXT, int QS = 1>
 __global__ void __launch_bounds__(64)
@@ -1509,14 +1592,15 @@ static int check_extras(const float* rel, int rel_len, int rel_ld, int keep_firs
     return 0;
 }
 
-extern "C" int hb_attn_prefill_mfma(const void* q, const void* k_cache, const void* v_cache, void* out,
+static int launch_attn_prefill(const void* q, const void* k_cache, const void* v_cache, void* out,
                                     const int* tile_seq, const int* tile_row0, const int* tile_rows,
                                     int num_tiles, const int* positions, const int* slots,
                                     const int* page_table, int max_pages, int page_size, int nq, int nkv,
                                     int hd, float scale, int window, int tile_height, const float* sinks,
                                     int chunk, float softcap, const float* rel, int rel_len, int rel_ld,
-                                    int keep_first, hipStream_t stream) {
+                                    int keep_first, const HeadsOut& ho, hipStream_t stream) {
     const bool extended = rel || keep_first > 0;
+    HB_REQUIRE(!ho.own || !extended, "attn_prefill: heads of their own size go without biases by distance and kept keys");
     if (check_extras(rel, rel_len, rel_ld, keep_first, window, chunk, softcap)) return 1;
     const AttnExtras ext = {rel, rel_len, rel_ld, REL_FRONT, keep_first};
     HB_REQUIRE(num_tiles > 0 && nq > 0 && nkv > 0 && nq % nkv == 0, "attn_prefill: bad sizes");
@@ -1535,24 +1619,25 @@ extern "C" int hb_attn_prefill_mfma(const void* q, const void* k_cache, const vo
     // tiles of 64: one ring of three stages of keys and three of values
     const size_t lds = (size_t)(tile_height == 64 ? 6 : 8) * PAGE * hd * sizeof(bf16) +
                        (extended ? 8 * PAGE_BIAS_FLOATS * sizeof(float) : 0);
-#define LAUNCH_PREFILL_FORM(KERNEL, HDV, FORM)                                                           \
+#define LAUNCH_PREFILL_FORM(KERNEL, HDV, ...)                                                           \
     do {                                                                                                 \
         static bool allowed = false;            /* once a process (the attribute is the function's) */   \
         if (lds > 64 * 1024 && !allowed) {                                                               \
-            hipError_t e_ = hipFuncSetAttribute((const void*)KERNEL<HDV, FORM>,                          \
+            hipError_t e_ = hipFuncSetAttribute((const void*)KERNEL<HDV, __VA_ARGS__>,                          \
                                                 hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);   \
             HB_REQUIRE(e_ == hipSuccess, "attn_prefill: cannot have %zu bytes of LDS: %s", lds, hipGetErrorString(e_)); \
             allowed = true;                                                                              \
         }                                                                                                \
-        KERNEL<HDV, FORM><<<total, 512, lds, stream>>>((const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, \
+        KERNEL<HDV, __VA_ARGS__><<<total, 512, lds, stream>>>((const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, \
                                                  (bf16*)out, tile_seq, tile_row0, tile_rows, positions, slots, \
                                                  page_table, max_pages, nq, nkv, c, window, per_tile, sinks, \
-                                                 chunk, cap, ext); \
+                                                 chunk, cap, ext, ho); \
     } while (0)
 #define LAUNCH_PREFILL(KERNEL, HDV)                                                                      \
     do {                                                                                                 \
-        if (extended) LAUNCH_PREFILL_FORM(KERNEL, HDV, true);                                            \
-        else LAUNCH_PREFILL_FORM(KERNEL, HDV, false);                                                    \
+        if (ho.own) LAUNCH_PREFILL_FORM(KERNEL, HDV, false, true);                                       \
+        else if (extended) LAUNCH_PREFILL_FORM(KERNEL, HDV, true, false);                                \
+        else LAUNCH_PREFILL_FORM(KERNEL, HDV, false, false);                                             \
     } while (0)
     if (tile_height == 64) {
         if (hd == 32) LAUNCH_PREFILL(attn_prefill_long_kernel, 32);
@@ -1569,6 +1654,36 @@ extern "C" int hb_attn_prefill_mfma(const void* q, const void* k_cache, const vo
 #undef LAUNCH_PREFILL_FORM
     HB_CHECK_LAUNCH("attn_prefill");
     return 0;
+}
+
+extern "C" int hb_attn_prefill_mfma(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                    const int* tile_seq, const int* tile_row0, const int* tile_rows,
+                                    int num_tiles, const int* positions, const int* slots,
+                                    const int* page_table, int max_pages, int page_size, int nq, int nkv,
+                                    int hd, float scale, int window, int tile_height, const float* sinks,
+                                    int chunk, float softcap, const float* rel, int rel_len, int rel_ld,
+                                    int keep_first, hipStream_t stream) {
+    return launch_attn_prefill(q, k_cache, v_cache, out, tile_seq, tile_row0, tile_rows, num_tiles, positions, slots, page_table,
+                               max_pages, page_size, nq, nkv, hd, scale, window, tile_height, sinks, chunk, softcap, rel, rel_len,
+                               rel_ld, keep_first, HeadsOut{}, stream);
+}
+
+// The same where the heads leave at their own size (HeadsOut): out bf16 [T, nq / maps x vdim]; gate null: none, else the first of
+// gate_slices slices of its columns, rows of gate_ld floats.
+extern "C" int hb_attn_prefill_heads_mfma(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                          const int* tile_seq, const int* tile_row0, const int* tile_rows, int num_tiles,
+                                          const int* positions, const int* slots, const int* page_table, int max_pages,
+                                          int page_size, int nq, int nkv, int hd, float scale, int window, int tile_height,
+                                          const float* sinks, int chunk, float softcap, int maps, int vdim, const float* gate,
+                                          int gate_ld, int gate_slices, size_t gate_stride, float lambda, float factor, float eps,
+                                          hipStream_t stream) {
+    HB_REQUIRE(vdim > 0 && vdim <= hd, "attn_prefill: heads of %d kept at %d", vdim, hd);
+    HB_REQUIRE(maps == 1 || (maps == 2 && nkv > 0 && nq % (2 * nkv) == 0), "attn_prefill: %d maps of %d query heads", maps, nq);
+    HB_REQUIRE(!gate || (gate_ld >= nq / maps * vdim && gate_slices >= 1 && gate_slices <= 8), "attn_prefill: bad gates");
+    const HeadsOut ho = {1, maps, vdim, gate, gate_ld, gate_slices, gate_stride, lambda, factor, eps};
+    return launch_attn_prefill(q, k_cache, v_cache, out, tile_seq, tile_row0, tile_rows, num_tiles, positions, slots, page_table,
+                               max_pages, page_size, nq, nkv, hd, scale, window, tile_height, sinks, chunk, softcap, nullptr, 0, 0, 0,
+                               ho, stream);
 }
 
 // qkv != null: the fused form (see DecodeFusion); q is then not read. qkv_slices > 1 (2, 4 or 8, heads

@@ -116,13 +116,13 @@ attention_plain_kernel(const TQ* __restrict__ q, const TC* __restrict__ k_cache,
 }
 
 // q, out: [T, nq * hd]; keys [pages, nkv, page_size, hd], values [pages, nkv, hd, page_size];
-// dtype covers q, cache and out.
+// dtype covers q and cache, and out unless out_dtype says float32.
 extern "C" int hb_attention_plain(const void* q, const void* k_cache, const void* v_cache, void* out,
                                   int dtype, const int* positions, const int* seq_of, const int* slots,
                                   const int* page_table, int max_pages, int page_size, int T, int nq,
                                   int nkv, int hd, float scale, int window, const float* sinks,
                                   int chunk, float softcap, const float* bias, int bias_ld, int bias_at,
-                                  int bias_len, int keep_first, hipStream_t stream) {
+                                  int bias_len, int keep_first, int out_dtype, hipStream_t stream) {
     HB_REQUIRE(T > 0 && nq > 0 && nkv > 0, "attention: empty input");
     HB_REQUIRE(nq % nkv == 0, "attention: %d query heads not divisible by %d kv heads", nq, nkv);
     HB_REQUIRE(hd > 0 && hd <= HB_MAX_HEAD_DIM, "attention: head_dim %d not in 1..%d", hd,
@@ -132,8 +132,14 @@ extern "C" int hb_attention_plain(const void* q, const void* k_cache, const void
     HB_REQUIRE(keep_first >= 0 && (keep_first == 0 || window > 0), "attention: kept first keys go with a window");
     HB_REQUIRE(!bias || (bias_len > 0 && bias_at >= 0 && bias_at + bias_len <= bias_ld), "attention: bad table of biases");
     HB_REQUIRE(nq <= 65535, "attention: too many heads for the grid");
+    HB_REQUIRE(out_dtype == dtype || out_dtype == HB_F32, "attention: the output is stored as the cache is, or in float32");
     dim3 grid(T, nq);
-    if (dtype == HB_F32)
+    if (dtype == HB_BF16 && out_dtype == HB_F32)
+        attention_plain_kernel<bf16, bf16, float><<<grid, HB_WAVE, 0, stream>>>(
+            (const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, (float*)out, positions, seq_of,
+            slots, page_table, max_pages, page_size, nq, nkv, hd, scale, window, sinks, chunk, softcap, bias,
+            bias_ld, bias_at, bias_len, keep_first);
+    else if (dtype == HB_F32)
         attention_plain_kernel<float, float, float><<<grid, HB_WAVE, 0, stream>>>(
             (const float*)q, (const float*)k_cache, (const float*)v_cache, (float*)out, positions, seq_of,
             slots, page_table, max_pages, page_size, nq, nkv, hd, scale, window, sinks, chunk, softcap, bias,

@@ -325,17 +325,17 @@ extern "C" int hb_heads_prepare(const float* proj, int ld, int slices, size_t sl
 // With a1 and a2 the weighted sums of a head's two maps (neighbouring query heads, kept at hd entries):
 //   o = a1 - lambda a2;   o <- o / sqrt(mean(o^2) + eps) x factor;   out[t, h vdim + d] = o x sigmoid(gate[t, h vdim + d])
 // (gate null: none; its columns may still lie in slices of K, added up here). One wave a (token, head).
-template <class T>
+template <class TIn, class T>
 __global__ void __launch_bounds__(256)
-heads_difference_kernel(const T* __restrict__ attn, const float* __restrict__ gate, int ld, int slices, size_t slice_stride,
+heads_difference_kernel(const TIn* __restrict__ attn, const float* __restrict__ gate, int ld, int slices, size_t slice_stride,
                         T* __restrict__ out, int heads, int hd, int vdim, float lambda, float factor, float eps, size_t total) {
     const size_t th = (size_t)blockIdx.x * 4 + (threadIdx.x >> 6);
     const int lane = threadIdx.x & 63;
     if (th >= total) return;
     const size_t t = th / heads;
     const int h = (int)(th - t * heads);
-    const T* const a1 = attn + th * 2 * hd;
-    const T* const a2 = a1 + hd;
+    const TIn* const a1 = attn + th * 2 * hd;
+    const TIn* const a2 = a1 + hd;
     const float* const grow = gate ? gate + t * ld + (size_t)h * vdim : nullptr;
     T* const dst = out + th * vdim;
     constexpr int HELD = 4;
@@ -377,18 +377,18 @@ heads_difference_kernel(const T* __restrict__ attn, const float* __restrict__ ga
 }
 
 // The same for heads of up to 128 in steps of four: half a wave a (token, head), four entries a lane.
-template <class T>
+template <class TIn, class T>
 __global__ void __launch_bounds__(256)
-heads_difference_quads_kernel(const T* __restrict__ attn, const float* __restrict__ gate, int ld, int slices, size_t slice_stride,
+heads_difference_quads_kernel(const TIn* __restrict__ attn, const float* __restrict__ gate, int ld, int slices, size_t slice_stride,
                               T* __restrict__ out, int heads, int hd, int vdim, float lambda, float factor, float eps, unsigned total) {
     const unsigned th = blockIdx.x * 8u + (threadIdx.x >> 5);
     const int d = (threadIdx.x & 31) * 4;
     const bool mine = th < total && d < vdim;
     const unsigned at = mine ? th : 0, t = at / heads, h = at - t * heads;
     const int dd = mine ? d : 0;
-    auto four = [](const T* p) {
+    auto four = [](const TIn* p) {
         f32x4 v;
-        if constexpr (sizeof(T) == 4) {
+        if constexpr (sizeof(TIn) == 4) {
             v = *(const f32x4*)p;
         } else {
             const bf16x4 raw = *(const bf16x4*)p;
@@ -397,7 +397,7 @@ heads_difference_quads_kernel(const T* __restrict__ attn, const float* __restric
         }
         return v;
     };
-    const T* const a1 = attn + (size_t)at * 2 * hd + dd;
+    const TIn* const a1 = attn + (size_t)at * 2 * hd + dd;
     const f32x4 x1 = four(a1), x2 = four(a1 + hd);
     f32x4 g = {0.f, 0.f, 0.f, 0.f};
     if (gate) {
@@ -429,34 +429,30 @@ heads_difference_quads_kernel(const T* __restrict__ attn, const float* __restric
     }
 }
 
-extern "C" int hb_heads_difference(const void* attn, int dtype, const float* gate, int ld, int slices, size_t slice_stride,
-                                   void* out, int T, int heads, int hd, int vdim, float lambda, float factor, float eps,
-                                   hipStream_t stream) {
+extern "C" int hb_heads_difference(const void* attn, int attn_dtype, int dtype, const float* gate, int ld, int slices,
+                                   size_t slice_stride, void* out, int T, int heads, int hd, int vdim, float lambda, float factor,
+                                   float eps, hipStream_t stream) {
     HB_REQUIRE(T > 0 && heads > 0 && vdim > 0 && hd >= vdim, "difference: empty input or heads of %d kept at %d", vdim, hd);
     HB_REQUIRE(!gate || ld >= heads * vdim, "difference: rows of %d do not hold the gates", ld);
     HB_REQUIRE(slices >= 1 && (slices == 1 || slice_stride > 0), "difference: bad slices");
     const size_t total = (size_t)T * heads;
-    HB_REQUIRE(total < (1ull << 32), "difference: too many heads");
-    const unsigned blocks = (unsigned)((total + 3) / 4);
-    HB_REQUIRE(dtype == HB_F32 || dtype == HB_BF16, "difference: unknown dtype %d", dtype);
-    if (vdim <= 128 && vdim % 4 == 0 && hd % 4 == 0 && (!gate || (ld % 4 == 0 && slice_stride % 4 == 0)) &&
-        (((uintptr_t)attn | (uintptr_t)gate | (uintptr_t)out) & 15) == 0 && total < (1ull << 31)) {
-        const unsigned eighths = (unsigned)((total + 7) / 8);
-        if (dtype == HB_F32)
-            heads_difference_quads_kernel<float><<<eighths, 256, 0, stream>>>((const float*)attn, gate, ld, slices, slice_stride,
-                                                                              (float*)out, heads, hd, vdim, lambda, factor, eps, (unsigned)total);
-        else
-            heads_difference_quads_kernel<bf16><<<eighths, 256, 0, stream>>>((const bf16*)attn, gate, ld, slices, slice_stride,
-                                                                             (bf16*)out, heads, hd, vdim, lambda, factor, eps, (unsigned)total);
-        HB_CHECK_LAUNCH("heads_difference");
-        return 0;
-    }
-    if (dtype == HB_F32)
-        heads_difference_kernel<float><<<blocks, 256, 0, stream>>>((const float*)attn, gate, ld, slices, slice_stride, (float*)out,
-                                                                   heads, hd, vdim, lambda, factor, eps, total);
-    else
-        heads_difference_kernel<bf16><<<blocks, 256, 0, stream>>>((const bf16*)attn, gate, ld, slices, slice_stride, (bf16*)out,
-                                                                  heads, hd, vdim, lambda, factor, eps, total);
+    HB_REQUIRE(total < (1ull << 31), "difference: too many heads");
+    HB_REQUIRE((dtype == HB_F32 || dtype == HB_BF16) && (attn_dtype == dtype || attn_dtype == HB_F32), "difference: dtypes %d and %d", attn_dtype, dtype);
+    const bool quads = vdim <= 128 && vdim % 4 == 0 && hd % 4 == 0 && (!gate || (ld % 4 == 0 && slice_stride % 4 == 0)) &&
+                       (((uintptr_t)attn | (uintptr_t)gate | (uintptr_t)out) & 15) == 0;
+#define HB_DIFFERENCE(TIn, TOut)                                                                                             \
+    do {                                                                                                                     \
+        if (quads)                                                                                                           \
+            heads_difference_quads_kernel<TIn, TOut><<<(unsigned)((total + 7) / 8), 256, 0, stream>>>((const TIn*)attn, gate, ld, slices, \
+                slice_stride, (TOut*)out, heads, hd, vdim, lambda, factor, eps, (unsigned)total);                            \
+        else                                                                                                                 \
+            heads_difference_kernel<TIn, TOut><<<(unsigned)((total + 3) / 4), 256, 0, stream>>>((const TIn*)attn, gate, ld, slices, \
+                slice_stride, (TOut*)out, heads, hd, vdim, lambda, factor, eps, total);                                      \
+    } while (0)
+    if (dtype == HB_F32) HB_DIFFERENCE(float, float);
+    else if (attn_dtype == HB_F32) HB_DIFFERENCE(float, bf16);
+    else HB_DIFFERENCE(bf16, bf16);
+#undef HB_DIFFERENCE
     HB_CHECK_LAUNCH("heads_difference");
     return 0;
 }

@@ -103,10 +103,11 @@ def prepare(proj, layout, bias, q_norm_w, k_norm_w, angles, rot_dims, halves, ep
 
 def difference(attn, proj, gate_off, out, heads, hd, vdim, lam, factor, eps, slices=None):
     """out[t, h vdim + d] = o factor / sqrt(mean(o^2) + eps) x sigmoid(gate), o = a1 - lam a2 with a1, a2 the kept heads 2h and
-    2h + 1 of attn [T, 2 heads x hd] and the gate in proj's columns from gate_off on (None: no gate)."""
+    2h + 1 of attn [T, 2 heads x hd] and the gate in proj's columns from gate_off on (None: no gate). attn may be
+    float32 beside outputs of another type: the maps' sums are then not rounded before they are taken from each other."""
     T = attn.shape[0]
-    _check(attn, "attn", None, (T, 2 * heads * hd))
-    _check(out, "out", attn.dtype, (T, heads * vdim))
+    _check(attn, "attn", torch.float32 if attn.dtype == torch.float32 else out.dtype, (T, 2 * heads * hd))
+    _check(out, "out", None, (T, heads * vdim))
     gate, ld, n, stride = None, 0, 1, 0
     if gate_off is not None:
         _check(proj, "gate", torch.float32, (T, None))
@@ -115,5 +116,5 @@ def difference(attn, proj, gate_off, out, heads, hd, vdim, lam, factor, eps, sli
             raise BackendError("difference: the gate's columns lie outside the rows")
         n, src, stride = slice_args(slices, proj)
         gate = src + 4 * gate_off
-    lib.call("heads", "hb_heads_difference", attn.data_ptr(), dtype_code(attn), gate, ld, n, stride, out.data_ptr(), T, heads, hd,
+    lib.call("heads", "hb_heads_difference", attn.data_ptr(), dtype_code(attn), dtype_code(out), gate, ld, n, stride, out.data_ptr(), T, heads, hd,
              vdim, float(lam), float(factor), float(eps), _stream())

@@ -45,7 +45,7 @@ SIGNATURES = {
         "hb_step_angles": [_P, _P, _I, _F, _P, _I, _P],
         "hb_heads_prepare": [_P, _I, _I, _SZ, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I,
                              _I, _I, _I, _I, _F, _P],
-        "hb_heads_difference": [_P, _I, _P, _I, _I, _SZ, _P, _I, _I, _I, _I, _F, _F, _F, _P],
+        "hb_heads_difference": [_P, _I, _I, _P, _I, _I, _SZ, _P, _I, _I, _I, _I, _F, _F, _F, _P],
     },
     "gemm_plain": {
         "hb_gemm_plain": [_P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P],
@@ -78,7 +78,7 @@ SIGNATURES = {
     },
     "attention_plain": {
         "hb_attention_plain": [_P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _P, _I, _F, _P, _I, _I, _I, _I,
-                               _P],
+                               _I, _P],
     },
     "sampling": {
         "hb_argmax": [_P, _I, _I, _I, _P, _P, _P, _I, _P],

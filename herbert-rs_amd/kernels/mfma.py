@@ -449,6 +449,8 @@ def gemm_activated(a, w, out, activation, packed=False, tile=0, row_scale=None, 
 
 
 lib.register_signatures("attention_mfma", {
+    "hb_attn_prefill_heads_mfma": [_P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I, _P, _I, _F, _I, _I, _P, _I,
+                                   _I, ctypes.c_size_t, _F, _F, _F, _P],
     "hb_attn_decode_heads_mfma": [_P, _I, _I, ctypes.c_size_t, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _F, _F, _P,
                                   _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _P, _I, _F, _P],
     "hb_attn_prefill_mfma": [_P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I, _P, _I, _F, _P, _I, _I, _I, _P],
@@ -664,6 +666,12 @@ def attention_decode_fused(qkv, q_norm_w, k_norm_w, cos, sin, meta, kv, out, nq,
              *extras, _stream())
 
 
+def heads_supported(kv, layout, dtype):
+    """True if the matrix cores take such heads (see attention_heads)."""
+    return (dtype == torch.bfloat16 and kv.k.dtype == torch.bfloat16 and kv.page_size == 64 and layout.hd in ATTENTION_HEAD_DIMS
+            and layout.nq % layout.nkv == 0 and layout.nq // layout.nkv <= 32)
+
+
 def decode_heads_fusable(meta, kv, layout, dtype):
     """True if the decode kernel can take the projection's rows themselves (see attention_decode_heads)."""
     return decode_fusable(meta, kv, layout.nq, layout.nkv, layout.hd, 0, dtype)
@@ -710,6 +718,43 @@ def attention_decode_heads(proj, layout, bias, q_norm_w, k_norm_w, angles, rot_d
              out.data_ptr(), po.data_ptr(), pml.data_ptr(), meta.context_lens.data_ptr(), meta.slots.data_ptr(),
              kv.page_table.data_ptr(), kv.page_table.shape[1], kv.page_size, B, L.nq, L.nkv, L.hd, float(scale), window, splits, per,
              ptr(ranges), ptr(sinks), chunk, float(softcap or 0.0), _stream())
+
+
+def attention_heads(q, layout, meta, kv, out, scale, window=None, chunk=None, softcap=None, sinks=None, proj=None, gate_off=None, lam=0.0,
+                    factor=1.0, eps=0.0, slices=None, tile_height=None):
+    """`attention` of a step of prompts' tokens whose heads leave at their own size: q [T, nq x hd] as heads.prepare writes it, out
+    bf16 [T, nq / maps x vdim]; two maps leave as their difference and a gate (gate_off: its first column in proj, whole or in
+    K slices) is applied, as heads.difference does, all in the attention's kernel."""
+    L, T = layout, q.shape[0]
+    _check(q, "q", torch.bfloat16, (T, L.nq * L.hd))
+    _check(out, "out", torch.bfloat16, (T, L.nq // L.maps * L.vdim))
+    pages = kv.k.shape[0]
+    _check(kv.k, "key pages", torch.bfloat16, (pages, L.nkv, 64, L.hd))
+    _check(kv.v, "value pages", torch.bfloat16, (pages, L.nkv, L.hd, 64))
+    _check(kv.page_table, "page_table", torch.int32, (None, None))
+    _check(meta.slots, "slots", torch.int32, (meta.num_seqs,))
+    _check(meta.positions, "positions", torch.int32, (T,))
+    if not attention_supported(q, kv, L.nq, L.nkv, L.hd):
+        raise BackendError(f"attention_mfma refuses heads kept at {L.hd} with {L.nq}/{L.nkv} of them")
+    if sinks is not None:
+        _check(sinks, "sinks", torch.float32, (L.nq,))
+    gate, ld, n, stride = None, 0, 1, 0
+    if gate_off is not None:
+        _check(proj, "gate", torch.float32, (T, None))
+        ld = proj.shape[1]
+        if not 0 <= gate_off <= ld - L.nq // L.maps * L.vdim:
+            raise BackendError("attention: the gate's columns lie outside the rows")
+        n, src, stride = heads.slice_args(slices, proj)
+        gate = src + 4 * gate_off
+    height = tile_height or _prefill_tile_height(meta, L.nkv, L.nq // L.nkv)
+    if height not in (32, 64):
+        raise BackendError("prompt attention has tiles of 32 or of 64 tokens")
+    tile_seq, tile_row0, tile_rows, n_tiles = _prefill_tiles(meta, height)
+    lib.call("attention_mfma", "hb_attn_prefill_heads_mfma", q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), out.data_ptr(),
+             tile_seq.data_ptr(), tile_row0.data_ptr(), tile_rows.data_ptr(), n_tiles, meta.positions.data_ptr(), meta.slots.data_ptr(),
+             kv.page_table.data_ptr(), kv.page_table.shape[1], kv.page_size, L.nq, L.nkv, L.hd, float(scale), int(window or 0), height,
+             None if sinks is None else sinks.data_ptr(), int(chunk or 0), float(softcap or 0.0), L.maps, L.vdim, gate, ld, n, stride,
+             float(lam), float(factor), float(eps), _stream())
 
 
 DEFERRED_SLICES = (2, 4, 8)     # numbers of slices of the projection that the decode kernel adds up itself

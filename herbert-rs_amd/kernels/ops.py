@@ -211,14 +211,14 @@ def attention_plain(q, meta, cache, out, nq, nkv, hd, scale, window, sinks=None,
     denominator of head h also holds exp(sinks[h]). chunk: a query sees the keys of its own chunk of that many
     positions only (counted from the sequence's start; not together with a window). softcap: a scaled score s
     becomes softcap tanh(s / softcap). bias: a DistanceBias, added to the scaled scores. keep_first (with a window):
-    the sequence's first so many keys are seen as well."""
+    the sequence's first so many keys are seen as well. out has the cache's storage type or is float32."""
     if bias is not None:
         bias.check(nq)
     T = q.shape[0]
     if sinks is not None:
         _check(sinks, "sinks", torch.float32, (nq,))
     _check(q, "q", cache.k.dtype, (T, nq * hd))
-    _check(out, "out", cache.k.dtype, (T, nq * hd))
+    _check(out, "out", torch.float32 if out.dtype == torch.float32 else cache.k.dtype, (T, nq * hd))
     _check_paged(meta, cache, T)
     if tuple(cache.k.shape[1:]) != (nkv, cache.page_size, hd):
         raise BackendError(f"cache pages {list(cache.k.shape)} do not fit {nkv} kv heads of {hd}")
@@ -228,7 +228,7 @@ def attention_plain(q, meta, cache, out, nq, nkv, hd, scale, window, sinks=None,
              cache.page_table.shape[1], cache.page_size, T, nq, nkv, hd, float(scale),
              int(window or 0), _ptr(sinks), int(chunk or 0), float(softcap or 0.0),
              None if bias is None else bias.rows.data_ptr(), 0 if bias is None else bias.rows.shape[1],
-             0 if bias is None else bias.at, 0 if bias is None else bias.length, int(keep_first or 0), _stream())
+             0 if bias is None else bias.at, 0 if bias is None else bias.length, int(keep_first or 0), dtype_code(out), _stream())
 
 
 GLU_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "relu": 2}

@@ -314,9 +314,10 @@ class Attention(Part):
         gate_off = L.channels if self.gate else None
         plain_masks = not self.keep_first and self.distance_raw is None
         fused = plain_masks and mfma.decode_heads_fusable(meta, kv, L, rt.dtype)
+        cores = plain_masks and mfma.heads_supported(kv, L, rt.dtype)
         # (slices of K are added up by the kernels that read the projection, but for the one that only gates heads)
-        defer = rt.dtype == torch.bfloat16 and (self.hd == 128 if fused else
-                                                    L.adds_slices and self.proj_width % 4 == 0 and (self.maps == 2 or not self.gate))
+        defer = rt.dtype == torch.bfloat16 and (self.hd == 128 if fused else L.adds_slices and self.proj_width % 4 == 0 and (
+            cores or self.maps == 2 or not self.gate))
         slices = self.qkv.forward(y, proj, row_scale=row_scale, defer_slices=defer)
         own = rt.buffer("attn_own", (T, self.nq * self.vdim))
         mixing = {"lam": self.lam, "factor": 1.0 - self.difference} if self.maps == 2 else {}
@@ -327,14 +328,19 @@ class Attention(Part):
         else:
             q = rt.buffer("q", (T, self.q_dim))
             heads.prepare(proj, L, self.bias_w, self.q_norm_w, self.k_norm_w, angles, rot_dims, halves, self.eps, meta, kv, q, slices)
-            attn = rt.buffer("attn", (T, self.q_dim))
-            self.attend(ctx, q, kv, attn)
-            if self.maps == 2:
-                heads.difference(attn, proj, gate_off, own, self.nq, self.hd, self.vdim, eps=self.eps, slices=slices, **mixing)
-            elif self.gate or self.hd != self.vdim:
-                ops.gate_heads(attn, proj if self.gate else None, L.channels, own, self.nq, self.hd, self.vdim)
+            if cores:
+                mfma.attention_heads(q, L, meta, kv, own, self.scale, self.window, self.chunk, self.softcap, self.sink_w, proj, gate_off,
+                                     eps=self.eps, slices=slices, **mixing)
             else:
-                own = attn
+                # (the sums of two maps stay float32 until they are taken from each other)
+                attn = rt.buffer("attn", (T, self.q_dim), torch.float32 if self.maps == 2 else None)
+                self.attend(ctx, q, kv, attn)
+                if self.maps == 2:
+                    heads.difference(attn, proj, gate_off, own, self.nq, self.hd, self.vdim, eps=self.eps, slices=slices, **mixing)
+                elif self.gate or self.hd != self.vdim:
+                    ops.gate_heads(attn, proj if self.gate else None, L.channels, own, self.nq, self.hd, self.vdim)
+                else:
+                    own = attn
         if self.o_bias_w is None:
             self.project_out(ctx, own, x)
         else:
@@ -471,7 +477,7 @@ class Attention(Part):
     def attend(self, ctx, q, kv, out):
         scale = self.scale if self.prepared else self.kernel_scale
         if q.dtype == torch.bfloat16:
-            if mfma.attention_supported(q, kv, self.kept_heads, self.nkv, self.hd):
+            if out.dtype == q.dtype and mfma.attention_supported(q, kv, self.kept_heads, self.nkv, self.hd):
                 mfma.attention(q, ctx.meta, kv, out, self.kept_heads, self.nkv, self.hd, scale, self.window,
                                scratch=ctx.rt.scratch, sinks=self.sink_w, chunk=self.chunk, softcap=self.softcap,
                                bias=self.distance_raw, keep_first=self.keep_first)

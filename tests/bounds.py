@@ -35,9 +35,13 @@ F32_ABS = 1e-4
 #  to 0.11 on single rows of the narrowest (widths of 64 and 72 through seven to nine layer runs, vocabularies of
 #  96 to 320), which is why its model-level tests let one row in fifty pass the bound by half; "boz": the Bozasun
 #  configurations, whose stream, scores, routing and state stay float32; "mut": the
-#  Mutedra configurations, worst seen 0.0065 and 0.024 (drawn ones, and sharpened scores).)
-BF16_REL_L2 = {"mut": 0.015, "boz": 0.03, "mef": 0.03, "mod": 0.03, "vip": 0.03, "A": 0.012, "B": 0.018, "C": 0.018, "D": 0.02, "F": 0.02, "wide": 0.02, "odd": 0.02, "random": 0.02, "long": 0.025, "deep": 0.02}
-BF16_REL_RMS = {"mut": 0.045, "boz": 0.1, "mef": 0.1, "mod": 0.1, "vip": 0.1, "A": 0.04, "B": 0.05, "C": 0.05, "D": 0.05, "F": 0.05, "wide": 0.08, "odd": 0.04, "random": 0.06, "long": 0.08, "deep": 0.08}
+#  Mutedra configurations, worst seen 0.0065 and 0.024 (drawn ones, and sharpened scores); "fig": the Figalorn configurations, whose difference of
+#  two attentions is divided by its own root mean square: where the two are nearly alike (a chunk's first tokens) the
+#  rounding of values and weights grows with the quotient. The plain formulas with their inputs rounded to bfloat16 at the
+#  engine's places give the same rows the same errors: up to 0.021 and 0.067; "figfar": scores sharpened for far keys, 0.024
+#  and 0.075.)
+BF16_REL_L2 = {"fig": 0.03, "figfar": 0.05, "mut": 0.015, "boz": 0.03, "mef": 0.03, "mod": 0.03, "vip": 0.03, "A": 0.012, "B": 0.018, "C": 0.018, "D": 0.02, "F": 0.02, "wide": 0.02, "odd": 0.02, "random": 0.02, "long": 0.025, "deep": 0.02}
+BF16_REL_RMS = {"fig": 0.1, "figfar": 0.15, "mut": 0.045, "boz": 0.1, "mef": 0.1, "mod": 0.1, "vip": 0.1, "A": 0.04, "B": 0.05, "C": 0.05, "D": 0.05, "F": 0.05, "wide": 0.08, "odd": 0.04, "random": 0.06, "long": 0.08, "deep": 0.08}
 
 
 def rel_rms_error(got, ref):
