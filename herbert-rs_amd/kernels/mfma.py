@@ -726,6 +726,9 @@ def attention_heads(q, layout, meta, kv, out, scale, window=None, chunk=None, so
     bf16 [T, nq / maps x vdim]; two maps leave as their difference and a gate (gate_off: its first column in proj, whole or in
     K slices) is applied, as heads.difference does, all in the attention's kernel."""
     L, T = layout, q.shape[0]
+    if L.maps == 1 and gate_off is None and L.hd == L.vdim:          # they leave as they are kept
+        attention(q, meta, kv, out, L.nq, L.nkv, L.hd, scale, window, tile_height=tile_height, sinks=sinks, chunk=chunk, softcap=softcap)
+        return
     _check(q, "q", torch.bfloat16, (T, L.nq * L.hd))
     _check(out, "out", torch.bfloat16, (T, L.nq // L.maps * L.vdim))
     pages = kv.k.shape[0]
