@@ -8,6 +8,9 @@ Scaled frequencies, all in float32 as there: "linear" divides every inv_freq by 
 (:205-228); "yarn" keeps those whose wavelength 2 pi / inv_freq is below original_max / beta_fast,
 divides by the factor those above original_max / beta_slow, and blends in between with
 smooth = (original_max / wavelength - beta_slow) / (beta_fast - beta_slow) (:239-287).
+
+"rope_pairs" and "rope_halves" (not in the reference): rates in float64, a table of the step's own angles instead of one
+for all positions (TurnsByAngles).
 """
 import math
 
